@@ -312,15 +312,17 @@ int yalm_set_prefill_forms(yalm_decoder d, const char *spec);
  * A second decoder kind beside yalm_decoder, for designs whose layers differ from one
  * another: every layer names a token mixer (latent attention over a cached low-rank
  * key/value latent, a real-gated linear recurrence, a gated delta rule, softmax attention
- * over cached keys and values with a window or chunk mask, a selective state-space layer; or
- * two of them side by side on the same input) and a feed-forward (none, dense
+ * over cached keys and values with a window or chunk mask, a selective state-space layer, a
+ * matrix memory with exponential gates; or two of them side by side on the same input) and a feed-forward (none, dense
  * GLU, routed experts with an optional shared expert, a plain two-matrix one), each with
  * its own sizes and constants. Serial blocks (block_kind = YALM_BLOCK_SERIAL): around every
  * sublayer x += norm_b(f(norm(x))) (pre_norm = 1) or x += norm_b(f(x)) (pre_norm = 0).
  * Parallel blocks (YALM_BLOCK_PARALLEL): h = norm1(x), x += ls1 * mixer(h) + ls2 * ff(h), one
  * norm read by both sublayers, each result scaled elementwise by its own vector (NULL: 1); a
- * layer of such a block that has norm2 feeds its feed-forward norm2(x) of the same x. The norms
- * are rms norms or mean-subtracting layer norms (norm_kind), both with a weight and no bias.
+ * layer of such a block that has norm2 feeds its feed-forward norm2(x) of the same x. Every
+ * sublayer's result is also scaled by residual_scale. The norms are rms norms or mean-subtracting
+ * layer norms (both with a weight and no bias), or YALM_NORM_TANH: tanh(alpha x) w + b elementwise, no
+ * statistics, its vector [2 width + 1] holding w, b and alpha one after the other (norm_kind).
  * The layer array is the order the layers RUN in: a block of layers that is walked several
  * times with the same weights is passed unrolled, its entries naming the same tensors, and
  * every entry has its own caches and states; pre_add is a vector added to the stream before
@@ -333,22 +335,27 @@ int yalm_set_prefill_forms(yalm_decoder d, const char *spec);
  * matrices: YALM_BF16 (bf16 MFMA products with f32 accumulation for portions, bf16
  * weight-streaming GEMVs for single tokens) or YALM_F32 (true f32 products).
  * Matrices are row-major [out][in]. */
-enum { YALM_MIX_LATENT = 0, YALM_MIX_RGLRU = 1, YALM_MIX_DELTA = 2, YALM_MIX_ATTN = 3, YALM_MIX_SSM = 4 };
+enum { YALM_MIX_LATENT = 0, YALM_MIX_RGLRU = 1, YALM_MIX_DELTA = 2, YALM_MIX_ATTN = 3, YALM_MIX_SSM = 4,
+	   YALM_MIX_MEMORY = 5 };
 enum { YALM_FF_NONE = 0, YALM_FF_DENSE = 1, YALM_FF_MOE = 2, YALM_FF_PLAIN = 3 };
-enum { YALM_NORM_RMS = 0, YALM_NORM_LAYER = 1 };
+enum { YALM_NORM_RMS = 0, YALM_NORM_LAYER = 1, YALM_NORM_TANH = 2 };
 enum { YALM_BLOCK_SERIAL = 0, YALM_BLOCK_PARALLEL = 1 };
 /* gated feed-forwards: y = w_down (act(w_gate x) (.) w_up x) */
 enum { YALM_ACT_DEFAULT = 0, /* dense: gelu; experts and shared expert: clamp */
 	   YALM_ACT_GELU = 1,  /* gelu_tanh(g) u */
 	   YALM_ACT_CLAMP = 2, /* g' sigmoid(1.702 g') (u' + 1), g' = min(g, limit), u' = clamp(u, -limit, limit) */
 	   YALM_ACT_SILU = 3,  /* g sigmoid(g) u */
-	   YALM_ACT_RELU2 = 4  /* plain feed-forward only: w_down max(w_up x, 0)^2 */ };
+	   YALM_ACT_RELU2 = 4, /* ungated only (plain, experts without w_gate): w_down max(w_up x, 0)^2 */
+	   YALM_ACT_GELU_ERF = 5 /* ungated only: w_down gelu(w_up x), gelu(z) = z (1 + erf(z / sqrt 2)) / 2 */ };
 /* routed experts: how the `top` experts and their weights come from the router logits */
 enum { YALM_ROUTER_SOFTMAX_TOP = 0, /* softmax over all experts, best groups, top scores, weight = score * router_scale */
 	   YALM_ROUTER_TOP_SOFTMAX = 1, /* the top logits (+ router_bias) win, weights = softmax over the chosen logits only */
-	   YALM_ROUTER_SIGMOID_GROUPS = 2 /* scores sigmoid(logit); the choice ranks score + router_bias: a group by the sum of
+	   YALM_ROUTER_SIGMOID_GROUPS = 2, /* scores sigmoid(logit); the choice ranks score + router_bias: a group by the sum of
 	                                    its two largest, the `top` largest within the groups_keep best groups win (ties: the
-	                                    lower index); weight = score * router_scale (without the bias, not renormalised) */ };
+	                                    lower index); weight = score * router_scale (without the bias, not renormalised) */
+	   YALM_ROUTER_SOFTMAX_NORMED = 3 /* scores softmax over experts and identity outputs; the `top` largest score + router_bias
+	                                    win (ties: the lower index, no groups); weight = score (without the bias) divided by the
+	                                    chosen scores' sum + 1e-20, times router_scale */ };
 /* attn: which earlier positions j <= i a position i sees */
 enum { YALM_MASK_CAUSAL = 0, /* all of them */
 	   YALM_MASK_WINDOW = 1, /* i - j < mask_size */
@@ -358,6 +365,13 @@ enum { YALM_QK_NONE = 0,
 	   YALM_QK_HEAD_UNIT = 1, /* after the rotation, every head divided by its rms over dim, no weight */
 	   YALM_QK_WHOLE = 2, /* before the rotation, rms norm over the whole projection with weights q_norm / kv_norm */
 	   YALM_QK_HEAD_W = 3 /* every head rms-normed over dim, times q_norm / kv_norm [dim] shared by all heads (no rotation) */ };
+/* attn, latent: which entries of a head's first rot_dims turn together */
+enum { YALM_ROT_INTERLEAVED = 0, /* (2i, 2i + 1) */
+	   YALM_ROT_HALVES = 1 /* (i, i + rot_dims / 2) (attn) */ };
+/* attn: how rot_factor > 0 rescales the frequencies */
+enum { YALM_RAMP_INDEX = 0, /* a linear ramp over the pair index; cos and sin scaled, see rot_factor */
+	   YALM_RAMP_TURNS = 1 /* by t, the times a pair turns within rot_orig positions: f kept for t > rot_fast, f / rot_factor
+	                          for t < rot_slow, between (1 - s) f / rot_factor + s f with s = (t - slow) / (fast - slow) */ };
 /* delta: activation of the output gate */
 enum { YALM_GATE_SILU = 0, YALM_GATE_SIGMOID = 1 };
 
@@ -418,22 +432,34 @@ typedef struct yalm_seq_layer {
 	int rel_rows;
 	float rel_max;
 	float join_scale;              /* side != NULL: mixer result = join_scale (rms(a) join_w + rms(b) side_join_w) */
+	float side_join_scale;         /* side != NULL with join_w NULL: mixer result = join_scale a + side_join_scale b */
+	int rot_pairs, rot_ramp;       /* attn: YALM_ROT_*, YALM_RAMP_* */
+	float softcap;                 /* attn: > 0: the scaled score s becomes softcap tanh(s / softcap), before mask and softmax */
+	/* memory (YALM_MIX_MEMORY, the matrix memory of xLSTM): heads heads of dim keys and vdim values; w_in rows [q: heads
+	   dim | k: heads dim | v: heads vdim | output gate: heads vdim | i: heads | f: heads] (+ in_bias); per head the log
+	   gates i = gate_cap tanh(i / gate_cap) and f = log sigmoid(gate_cap tanh(f / gate_cap)), a running maximum m
+	   from 0, m' = max(f + m, i), S <- exp(f + m - m') S + exp(i - m') k v^T, n <- the same with k alone, q scaled
+	   by dim^-1/2, o = S^T q / (max(|n . q|, exp(-m')) + 1e-6); o rms-normed per head, times out_norm [heads vdim],
+	   times sigmoid(output gate); then w_o */
+	float gate_cap;
+	int identity;                  /* moe: identity outputs after the experts (router and router_bias have experts +
+	                                  identity rows): a chosen one adds the feed-forward's input times its weight */
 	/* f32 vectors */
 	const float *norm1, *norm1b, *norm2, *norm2b; /* [width] each; norm2* unused without a feed-forward; parallel blocks: norm1 only */
 	const float *ls1, *ls2;         /* parallel blocks: [width] scales of the mixer's and the feed-forward's result */
 	const float *pre_add;           /* [width] added to the stream before this entry's opening norm, or NULL */
 	const float *sink_w;            /* [heads], see sink */
 	const float *o_bias;            /* attn: [width] bias of the output projection, or NULL */
-	const float *router_bias;       /* moe: [experts] added to the router logits, or NULL */
+	const float *router_bias;       /* moe: [experts + identity] added as router_kind says, or NULL */
 	const float *q_norm, *kv_norm;  /* latent: [q_rank], [kv_rank]; attn with YALM_QK_WHOLE: [heads dim], [kv_heads dim] */
-	const float *in_bias;           /* rglru: [2 rec_width] (gate branch, recurrent branch); attn: [rows of w_in] or NULL */
+	const float *in_bias;           /* rglru: [2 rec_width] (gate branch, recurrent branch); attn, memory: [rows of w_in] or NULL */
 	const float *head_temp;         /* attn: [heads], score of head h times head_temp[h], or NULL */
 	const float *talk;              /* attn: [heads][heads], score_h <- sum_g talk[h][g] score_g before mask and softmax, or NULL */
 	const float *conv_w, *conv_b;   /* [channels][conv] (last column = current token); rglru bias [rec_width] */
 	const float *gate_a, *gate_a_b, *gate_i, *gate_i_b; /* rglru: [blocks][bs][bs], [rec_width] (bs = rec_width / blocks) */
 	const float *lam;               /* rglru: [rec_width] */
-	const float *a_log, *dt_bias, *out_norm; /* delta: [heads], [heads] ([heads dim] with decay_rank), [vdim]; ssm: [heads], [heads], [heads vdim] */
-	const float *router, *shared_sg; /* moe: [experts][width]; [width]: the shared expert times sigmoid(shared_sg . x), NULL: times 1 */
+	const float *a_log, *dt_bias, *out_norm; /* delta: [heads], [heads] ([heads dim] with decay_rank), [vdim]; ssm: [heads], [heads], [heads vdim]; memory: -, -, [heads vdim] */
+	const float *router, *shared_sg; /* moe: [experts + identity][width]; [width]: the shared expert times sigmoid(shared_sg . x), NULL: times 1 */
 	/* matrices of weight_dtype */
 	const void *w_in;  /* latent: [q_rank (+ kv_rank if own latent)][width] (query down, latent down), with q_rank = 0
 	                      [heads (dim + rot_dim) + kv_rank + rot_dim][width] (queries, latent down, rotated key part);
@@ -450,16 +476,20 @@ typedef struct yalm_seq_layer {
 	                      and values instead of attending over the latents */
 	const void *w_o;   /* [width][heads vdim | rec_width] */
 	const void *w_gate, *w_up, *w_down; /* dense: [ff][width] x2, [width][ff]; moe: the same per expert, stacked;
-	                                       plain: w_down gelu(w_up x), no w_gate */
-	const void *ws_gate, *ws_up, *ws_down; /* moe shared expert */
+	                                       plain: w_down gelu(w_up x), no w_gate; moe without w_gate: the
+	                                       experts and the shared expert are plain (ff_act) */
+	const void *ws_gate, *ws_up, *ws_down; /* moe shared expert (ws_gate unused without w_gate) */
 	const float *rel;              /* attn: [rel_rows][heads], see rel_rows */
 	const float *d_skip;           /* ssm: [heads] */
-	const float *join_w, *side_join_w; /* side != NULL: [width] each */
+	const float *join_w, *side_join_w; /* side != NULL: [width] each, or both NULL (see side_join_scale) */
 	const void *w_a2, *w_g2;       /* delta: see decay_rank / gate_rank */
 	const struct yalm_seq_layer *side; /* HOST pointer or NULL: a second mixer that reads the same input beside this
 	                                  one (its mixer fields and tensors only; no norms, no feed-forward, no side of its
 	                                  own), with caches and states of its own; the two results are each rms-normed over
-	                                  the width (no mean taken off) and summed, see join_scale */
+	                                  the width (no mean taken off) and summed, see join_scale, or summed as they are,
+	                                  see side_join_scale. Its w_in may be NULL: its rows then follow this mixer's own in
+	                                  this layer's w_in (and in_bias), one projection for both (attn without a per-head
+	                                  output gate beside memory) */
 } yalm_seq_layer;
 
 typedef struct yalm_seq_config {
@@ -471,11 +501,13 @@ typedef struct yalm_seq_config {
 	int pos_embed;    /* 1: the interleaved sin / cos position vector (frequencies 10000^(-2i / width)) is added to the embedding */
 	float logit_scale; /* logits = head . norm(x) * logit_scale */
 	int block_kind;   /* YALM_BLOCK_*; parallel blocks need pre_norm = 1 */
+	float residual_scale; /* every sublayer's result times this as it joins the stream */
+	float logit_softcap;  /* > 0: logits <- logit_softcap tanh(logits / logit_softcap) */
 } yalm_seq_config;
 
 typedef struct yalm_seq_weights {
 	const void *embed;       /* [vocab][width] */
-	const float *final_norm; /* [width] */
+	const float *final_norm; /* [width] (YALM_NORM_TANH: [2 width + 1], as every norm) */
 	const void *head;        /* [vocab][width] */
 	const yalm_seq_layer *layers; /* HOST array of n_layers entries, copied by yalm_seq_create */
 	const float *embed_norm;  /* [width] or NULL: the embedding row (scaled, with its position vector) is normed

@@ -1,7 +1,7 @@
 // seq.hip — the layer-list engine of the C ABI (include/yalm_hip.h, "layer-list models"):
 // a decoder whose layers each name their token mixer (latent attention, real-gated linear
 // recurrence, gated delta rule, softmax attention with a window or chunk mask, selective
-// state-space layer, or two of them side by side) and
+// state-space layer, matrix memory with exponential gates, or two of them side by side) and
 // feed-forward (dense GLU, routed experts, plain), holding one sequence's latent and
 // key / value caches and recurrent / convolution states in HBM. One step function
 // serves whole prompts, portions of prompts and single decoded tokens; the device greedy
@@ -54,7 +54,11 @@ struct yalm_seq_s {
 	const float *In = nullptr;   // what a sublayer reads: Hn (pre_norm) or X itself
 	float *Xalt = nullptr, *Xbase = nullptr; // single tokens without opening norms: the stream alternates between two rows
 	const float *pend_wb = nullptr; // a closing norm not yet applied: X += norm(Y) pend_wb, owed to the next product
-	bool ln = false;             // the model's norms are layer norms
+	int nk = NK_RMS;             // the kind of the model's norms
+	// a pair whose two mixers share one input projection: where the mixer being enqueued finds its
+	// columns of the result, and that result's row length (nullptr: the mixer projects for itself)
+	float *Zin = nullptr;
+	int ldz = 0;
 	float *inv_freq = nullptr;
 	uint16_t *a16 = nullptr;     // [cap][bw] bf16 copy of a product's activations (large-tile GEMM operand)
 	int *tok = nullptr, *want = nullptr;
@@ -122,6 +126,7 @@ static int in_rows(const yalm_seq_layer &l) {
 		return l.heads * l.dim + l.kv_heads * (l.dim + l.vdim) +
 		       (l.out_gate == 2 ? l.heads * l.vdim : (l.out_gate ? l.heads : 0));
 	case YALM_MIX_SSM: return 2 * l.heads * l.vdim + 2 * l.ssm_groups * l.ssm_state + l.heads;
+	case YALM_MIX_MEMORY: return 2 * l.heads * (l.dim + l.vdim + 1);
 	default:
 		return 2 * l.kv_heads * l.dim + l.heads * l.vdim + (l.gate_rank > 0 ? l.gate_rank : l.heads * l.vdim) + l.heads +
 		       (l.decay_rank > 0 ? l.decay_rank : l.heads);
@@ -134,28 +139,53 @@ static bool latent_direct(const yalm_seq_layer &l) {
 	return l.mixer == YALM_MIX_LATENT && l.q_rank == 0;
 }
 
+// The recurrence kernel's lanes per column of the state (16: twice the workgroups, half the rows per
+// lane; 8 for the smallest keys), and the workgroups per head over `cols` columns.
+static int delta_lpc(int K) {
+	return K <= 32 ? 8 : 16;
+}
+static int delta_blocks(int K, int cols) {
+	return cdiv(cols, SEQ_THREADS / delta_lpc(K));
+}
+// Floats of a matrix memory's state: [heads][dim][vdim + 1] (the last column is the normaliser), then a
+// running maximum per head and workgroup of the recurrence kernel.
+static size_t memory_state(const yalm_seq_layer &l) {
+	return (size_t)l.heads * l.dim * (l.vdim + 1) + (size_t)l.heads * delta_blocks(l.dim, l.vdim + 1);
+}
+
 static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> &L) {
 	ARGCHK(c.width > 0 && c.vocab > 0 && c.n_layers > 0 && c.max_tokens > 0, "yalm_seq_create: bad model sizes");
 	ARGCHK(c.weight_dtype == YALM_BF16 || c.weight_dtype == YALM_F32, "yalm_seq_create: weight_dtype must be bf16 or f32");
-	ARGCHK(c.norm_kind == YALM_NORM_RMS || c.norm_kind == YALM_NORM_LAYER, "yalm_seq_create: unknown norm kind");
+	ARGCHK(c.norm_kind == YALM_NORM_RMS || c.norm_kind == YALM_NORM_LAYER || c.norm_kind == YALM_NORM_TANH,
+	       "yalm_seq_create: unknown norm kind");
+	ARGCHK(c.logit_softcap >= 0.0f, "yalm_seq_create: bad logit cap");
 	ARGCHK(c.block_kind == YALM_BLOCK_SERIAL || (c.block_kind == YALM_BLOCK_PARALLEL && c.pre_norm),
 	       "yalm_seq_create: blocks are serial, or parallel with pre_norm");
 	const bool par = c.block_kind == YALM_BLOCK_PARALLEL;
+	std::vector<int> owner; // of each second mixer: the layer it stands beside
+	for (int i = 0; i < c.n_layers; ++i)
+		if (L[i].side)
+			owner.push_back(i);
 	for (int i = 0; i < (int)L.size(); ++i) { // the n_layers entries, then their second mixers
 		const yalm_seq_layer &l = L[i];
 		const bool is_side = i >= c.n_layers;
 		const std::string at = "yalm_seq_create: " + std::string(is_side ? "second mixer " : "layer ") +
 		                       std::to_string(is_side ? i - c.n_layers : i) + ": ";
-		ARGCHK(l.w_in && l.w_o, at + "missing tensors");
+		ARGCHK((l.w_in || is_side) && l.w_o, at + "missing tensors");
 		if (is_side) {
+			const yalm_seq_layer &a = L[owner[i - c.n_layers]];
+			ARGCHK(l.w_in || (l.mixer == YALM_MIX_MEMORY && a.mixer == YALM_MIX_ATTN && a.out_gate != 1 && !l.in_bias),
+			       at + "only a matrix memory beside an attention without a per-head output gate shares its projection");
 			ARGCHK(l.ff_kind == YALM_FF_NONE && !l.side && !l.pre_add, at + "a second mixer has no feed-forward, no vector and no side of its own");
 		} else {
 			ARGCHK((l.norm1 || !c.pre_norm) && (l.norm1b || par), at + "missing tensors");
-			ARGCHK(!l.side || (l.join_w && l.side_join_w), at + "two mixers side by side need the norm weights of their results");
+			ARGCHK(!l.side || !l.join_w == !l.side_join_w, at + "two mixers side by side need both norm weights of their results, or neither");
 		}
-		ARGCHK(l.ff_act >= YALM_ACT_DEFAULT && l.ff_act <= YALM_ACT_RELU2 &&
-		           (l.ff_act != YALM_ACT_RELU2 || l.ff_kind == YALM_FF_PLAIN || l.ff_kind == YALM_FF_NONE),
-		       at + "unknown feed-forward activation (relu^2 belongs to the plain feed-forward)");
+		const bool ungated = l.ff_kind == YALM_FF_PLAIN || (l.ff_kind == YALM_FF_MOE && !l.w_gate);
+		ARGCHK(l.ff_kind == YALM_FF_NONE || (l.ff_act >= YALM_ACT_DEFAULT && l.ff_act <= YALM_ACT_GELU_ERF &&
+		                                     (ungated ? l.ff_act != YALM_ACT_CLAMP && l.ff_act != YALM_ACT_SILU
+		                                              : l.ff_act < YALM_ACT_RELU2)),
+		       at + "unknown feed-forward activation (clamp and silu belong to gated pairs, relu^2 and the exact gelu to ungated ones)");
 		ARGCHK(!l.pre_add || i == 0 || par, at + "a vector added before an entry after the first needs parallel blocks");
 		if (latent_direct(l)) {
 			ARGCHK(l.heads > 0 && l.dim > 0 && l.vdim > 0 && l.kv_rank > 0 && l.rot_dim >= 0 && l.kv_from < 0,
@@ -214,9 +244,19 @@ static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> 
 			}
 			ARGCHK(l.conv >= 1 && l.conv <= SEQ_MAX_TAPS, at + "convolution taps out of range");
 			ARGCHK(l.conv_w && l.a_log && l.dt_bias && l.d_skip && l.out_norm, at + "missing state-space tensors");
+		} else if (l.mixer == YALM_MIX_MEMORY) {
+			ARGCHK(l.heads > 0 && l.dim > 0 && l.vdim > 0 && l.gate_cap > 0.0f, at + "bad matrix memory sizes");
+			if (l.dim > 256) {
+				set_err(at + "dim above 256 is not implemented by the recurrence kernel");
+				return YALM_ERR_UNSUPPORTED;
+			}
+			ARGCHK(l.out_norm, at + "missing matrix memory tensors");
 		} else if (l.mixer == YALM_MIX_ATTN) {
 			ARGCHK(l.heads > 0 && l.kv_heads > 0 && l.heads % l.kv_heads == 0 && l.dim > 0 && l.vdim > 0,
 			       at + "bad attention sizes");
+			ARGCHK((l.rot_pairs == YALM_ROT_INTERLEAVED || l.rot_pairs == YALM_ROT_HALVES) &&
+			           (l.rot_ramp == YALM_RAMP_INDEX || l.rot_ramp == YALM_RAMP_TURNS) && l.softcap >= 0.0f,
+			       at + "unknown rotary layout or bad score cap");
 			if (l.dim > 256 || l.vdim > 256 || (size_t)l.heads * ((l.vdim + 3) / 4) > (size_t)SA_MAX_NA4 * SEQ_THREADS) {
 				set_err(at + "heads of more than 256 entries (or heads x vdim above 16384) are not implemented by the attention kernels");
 				return YALM_ERR_UNSUPPORTED;
@@ -232,7 +272,8 @@ static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> 
 			ARGCHK(l.out_gate >= 0 && l.out_gate <= 2, at + "unknown output gate");
 			ARGCHK(l.rot_dims >= 0 && l.rot_dims <= l.dim && l.rot_dims % 2 == 0 && (l.rot_dims == 0 || l.rot_base > 0.0f),
 			       at + "rotary sizes must be even and at most dim");
-			ARGCHK(!(l.rot_factor > 0.0f) || (l.rot_orig > 0 && l.rot_fast > 0.0f && l.rot_slow > 0.0f && l.rot_base != 1.0f),
+			ARGCHK(!(l.rot_factor > 0.0f) || (l.rot_orig > 0 && l.rot_fast > 0.0f && l.rot_slow > 0.0f &&
+			                                  (l.rot_base != 1.0f || l.rot_ramp == YALM_RAMP_TURNS)),
 			       at + "bad rotary rescaling");
 		} else {
 			ARGCHK(false, at + "unknown mixer");
@@ -242,16 +283,18 @@ static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> 
 		} else if (l.ff_kind == YALM_FF_PLAIN) {
 			ARGCHK(l.ff > 0 && l.w_up && l.w_down && (par || ((l.norm2 || !c.pre_norm) && l.norm2b)), at + "bad plain feed-forward");
 		} else if (l.ff_kind == YALM_FF_MOE) {
-			ARGCHK(l.ff > 0 && l.experts > 0 && l.top > 0 && l.top <= l.experts && l.groups > 0 &&
+			ARGCHK(l.ff > 0 && l.experts > 0 && l.top > 0 && l.top <= l.experts + l.identity && l.groups > 0 &&
 			           l.groups <= SEQ_MAX_GROUPS && l.experts % l.groups == 0 && l.groups_keep > 0 &&
-			           l.groups_keep <= l.groups && l.top <= l.groups_keep * (l.experts / l.groups),
+			           l.groups_keep <= l.groups && l.top <= l.groups_keep * (l.experts / l.groups) + l.identity,
 			       at + "bad router sizes");
 			ARGCHK(l.router_kind == YALM_ROUTER_SOFTMAX_TOP || l.router_kind == YALM_ROUTER_SIGMOID_GROUPS ||
-			           (l.router_kind == YALM_ROUTER_TOP_SOFTMAX && l.groups == 1),
-			       at + "unknown router kind (the top-logits router has no groups)");
-			ARGCHK(l.router && l.w_gate && l.w_up && l.w_down && (par || ((l.norm2 || !c.pre_norm) && l.norm2b)), at + "missing expert tensors");
+			           ((l.router_kind == YALM_ROUTER_TOP_SOFTMAX || l.router_kind == YALM_ROUTER_SOFTMAX_NORMED) && l.groups == 1),
+			       at + "unknown router kind (groups belong to the first and third only)");
+			ARGCHK(l.identity >= 0 && (l.identity == 0 || (l.router_kind == YALM_ROUTER_SOFTMAX_NORMED && c.pre_norm)),
+			       at + "identity outputs belong to the softmax router with renormalised weights, in blocks with opening norms");
+			ARGCHK(l.router && l.w_up && l.w_down && (par || ((l.norm2 || !c.pre_norm) && l.norm2b)), at + "missing expert tensors");
 			if (l.shared_ff > 0)
-				ARGCHK(l.ws_gate && l.ws_up && l.ws_down, at + "missing shared expert tensors");
+				ARGCHK((l.ws_gate || !l.w_gate) && l.ws_up && l.ws_down, at + "missing shared expert tensors");
 		} else {
 			ARGCHK(l.ff_kind == YALM_FF_NONE, at + "unknown feed-forward kind");
 		}
@@ -290,7 +333,8 @@ static int att_attr_ct(int rank) {
 // base^(-2i / dims) radians per position; with a rescaling (rot_factor > 0) the pairs that
 // turn fewer than rot_slow times within rot_orig positions turn rot_factor times slower, those
 // that turn more than rot_fast times are left, a linear ramp over the pair index between, and
-// cos / sin are scaled by 0.1 ln(rot_factor) + 1.
+// cos / sin are scaled by 0.1 ln(rot_factor) + 1; or (rot_ramp) a ramp over how often a pair turns within
+// rot_orig positions, cos / sin as they are.
 static int attn_setup(yalm_seq_s *q, int li) {
 	const yalm_seq_layer &l = q->L[li];
 	const int dims = l.rot_dims, half = dims / 2;
@@ -298,7 +342,15 @@ static int attn_setup(yalm_seq_s *q, int li) {
 	double mag = 1.0;
 	for (int i = 0; i < half; ++i)
 		f[i] = std::pow((double)l.rot_base, -2.0 * i / (double)dims);
-	if (l.rot_factor > 0.0f && half > 0) {
+	if (l.rot_factor > 0.0f && l.rot_ramp == YALM_RAMP_TURNS) {
+		for (int i = 0; i < half; ++i) {
+			const double turns = (double)l.rot_orig * f[i] / (2.0 * 3.14159265358979323846), slow = f[i] / (double)l.rot_factor;
+			if (turns > (double)l.rot_fast)
+				continue;
+			const double sh = turns < (double)l.rot_slow ? 0.0 : (turns - l.rot_slow) / std::max((double)l.rot_fast - l.rot_slow, 1e-30);
+			f[i] = (1.0 - std::min(sh, 1.0)) * slow + std::min(sh, 1.0) * f[i];
+		}
+	} else if (l.rot_factor > 0.0f && half > 0) {
 		const double pi = 3.14159265358979323846;
 		auto turn = [&](double t) { return dims * std::log((double)l.rot_orig / (2.0 * pi * t)) / (2.0 * std::log((double)l.rot_base)); };
 		const double lo = std::max(std::floor(turn(l.rot_fast)), 0.0);
@@ -387,8 +439,10 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 	q->cap = std::min(c.max_tokens, (int)SEQ_PORTION_CAP);
 	size_t bw = c.width, arena = 0;
 	int zw = 1, max_e = 1, max_top = 1;
-	for (const yalm_seq_layer &l : q->L) {
-		zw = std::max(zw, in_rows(l));
+	for (int i = 0; i < (int)q->L.size(); ++i) {
+		const yalm_seq_layer &l = q->L[i];
+		const bool joint = i < c.n_layers && q->side_of[i] >= 0 && !q->L[q->side_of[i]].w_in;
+		zw = std::max(zw, in_rows(l) + (joint ? in_rows(q->L[q->side_of[i]]) : 0));
 		if (l.mixer == YALM_MIX_LATENT) {
 			bw = std::max({bw, (size_t)l.heads * (l.dim + l.rot_dim), (size_t)l.heads * (l.kv_rank + l.rot_dim),
 			               (size_t)l.heads * l.vdim, (size_t)l.q_rank});
@@ -398,6 +452,9 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 		} else if (l.mixer == YALM_MIX_ATTN) {
 			// with score mixing a portion's queries span the whole key row
 			bw = std::max({bw, (size_t)l.heads * l.dim * (l.talk ? l.kv_heads : 1), (size_t)l.heads * l.vdim});
+		} else if (l.mixer == YALM_MIX_MEMORY) {
+			bw = std::max(bw, (size_t)l.heads * (l.vdim + 1));
+			arena += memory_state(l);
 		} else if (l.mixer == YALM_MIX_SSM) {
 			const size_t cc = (size_t)l.heads * l.vdim + 2 * (size_t)l.ssm_groups * l.ssm_state;
 			bw = std::max({bw, cc, (size_t)2 * l.heads});
@@ -474,7 +531,7 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 	}
 	q->gen_cap = 1 << 16;
 	STRY(sallocT(q, &q->gen_tokens, q->gen_cap));
-	q->ln = c.norm_kind == YALM_NORM_LAYER;
+	q->nk = c.norm_kind;
 	q->In = c.pre_norm ? q->Hn : q->X;
 	q->Xbase = q->X;
 	if (!c.pre_norm)
@@ -522,6 +579,9 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 			off += l.rec_width;
 			q->conv[i] = q->arena + off;
 			off += (size_t)(l.conv - 1) * l.rec_width;
+		} else if (l.mixer == YALM_MIX_MEMORY) {
+			q->S[i] = q->arena + off;
+			off += memory_state(l);
 		} else if (l.mixer == YALM_MIX_SSM) {
 			const size_t cc = (size_t)l.heads * l.vdim + 2 * (size_t)l.ssm_groups * l.ssm_state;
 			q->S[i] = q->arena + off;
@@ -632,8 +692,8 @@ static int gemm(Seq *q, const GemmArgs &a, int batches = 1, int max_m = -1, bool
 	// output columns past the last multiple of 128 (a few gate rows closing an input projection)
 	// run on the general kernel as a second, narrow product
 	const bool pair = a.W2 != nullptr && (a.epi == EPI_GLU_GELU || a.epi == EPI_GLU_CLAMP || a.epi == EPI_GLU_SILU) && !a.bias;
-	const bool single = !a.W2 && (a.epi == EPI_NONE || a.epi == EPI_GELU || a.epi == EPI_RELU2);
-	const int act1 = a.epi == EPI_GELU ? 1 : (a.epi == EPI_RELU2 ? 2 : 0); // the large-tile door's activation
+	const bool single = !a.W2 && (a.epi == EPI_NONE || a.epi == EPI_GELU || a.epi == EPI_RELU2 || a.epi == EPI_GELU_ERF);
+	const int act1 = a.epi == EPI_GELU ? 1 : (a.epi == EPI_RELU2 ? 2 : (a.epi == EPI_GELU_ERF ? 3 : 0)); // the large-tile door's activation
 	const int n_big = pair ? (a.N % 64 == 0 ? a.N : 0) : (single ? a.N & ~127 : 0);
 	if (q->a16 && batches == 1 && max_m >= 2 * GB_BM && !a.rows && !a.w_sel && a.z_split == 0 && a.ldw == a.K &&
 	    a.K % 64 == 0 && n_big > 0 && (a.N - n_big <= 64 || (!pair && a.N - n_big < 128))) {
@@ -806,16 +866,27 @@ static int mixer_rglru(Seq *q, int li, int n) {
 	return gemm(q, plain(so, W, l.w_o, W, q->Yout, c.width, n, c.width, W));
 }
 
-// The recurrence kernel over a portion: the gated delta rule (ssm = false; gv: one decay per head
-// and key channel) or the state-space walk (ssm = true). K: key / state size, P: value size.
+// The recurrence kernel over a portion: the gated delta rule (gv: one decay per head and key
+// channel), the state-space walk, or the matrix memory (mg: its log gates; scale: on the read-outs).
+// K: key / state size, P: value size (the matrix memory's state has one column more).
+enum { WALK_DELTA, WALK_SSM, WALK_MEMORY };
+struct MemGates {
+	const float *lg; // log gates (or their logits, cap > 0) [t][ld]: input gates, then forget gates
+	int ld;
+	float cap, scale;
+	float *running; // the running maxima
+};
 static int delta_launch(Seq *q, const float *qkv, int ldq, int qo, int ko, int vo, int KH, int K, int H, int P,
-                        const float *bg, const float *gv, const float *dskip, float *state, float *o, int n, bool ssm) {
-	// lanes per column of the state: 16 (twice the workgroups, half the rows per lane) but for the smallest keys
-	const int lpc = K <= 32 ? 8 : 16;
-	const dim3 g(cdiv(P, SEQ_THREADS / lpc), H);
+                        const float *bg, const float *gv, const float *dskip, float *state, float *o, int n, int walk,
+                        const MemGates &mg = MemGates{}) {
+	const dim3 g(delta_blocks(K, walk == WALK_MEMORY ? P + 1 : P), H);
 #define DELTA_LAUNCH(RR, TC, LPC)                                                                                      \
 	do {                                                                                                               \
-		if (ssm)                                                                                                       \
+		if (walk == WALK_MEMORY)                                                                                       \
+			seq_delta_kernel<RR, TC, true, false, LPC, true><<<g, SEQ_THREADS, 0, q->stream>>>(                        \
+			    qkv, ldq, qo, ko, vo, KH, K, H, P, nullptr, nullptr, nullptr, state, o, n, mg.lg, mg.ld, mg.cap,       \
+			    mg.scale, mg.running);                                                                                 \
+		else if (walk == WALK_SSM)                                                                                     \
 			seq_delta_kernel<RR, TC, true, false, LPC><<<g, SEQ_THREADS, 0, q->stream>>>(                              \
 			    qkv, ldq, qo, ko, vo, KH, K, H, P, bg, nullptr, dskip, state, o, n);                                   \
 		else if (gv)                                                                                                   \
@@ -825,7 +896,7 @@ static int delta_launch(Seq *q, const float *qkv, int ldq, int qo, int ko, int v
 			seq_delta_kernel<RR, TC, false, false, LPC><<<g, SEQ_THREADS, 0, q->stream>>>(                             \
 			    qkv, ldq, qo, ko, vo, KH, K, H, P, bg, nullptr, nullptr, state, o, n);                                 \
 	} while (0)
-	if (K <= 32) DELTA_LAUNCH(4, 16, 8);
+	if (K <= 32) DELTA_LAUNCH(4, 16, 8); // the lanes per column are delta_lpc(K)
 	else if (K <= 64) DELTA_LAUNCH(4, 16, 16);
 	else if (K <= 128) DELTA_LAUNCH(8, 16, 16);
 	else DELTA_LAUNCH(16, 8, 16);
@@ -858,7 +929,7 @@ static int mixer_delta(Seq *q, int li, int n) {
 		ldg = CV;
 		gc = 0;
 	}
-	TRY(delta_launch(q, qkv, cc, 0, CQ, 2 * CQ, KH, D, H, V, bg, gv, nullptr, q->S[li], o, n, false));
+	TRY(delta_launch(q, qkv, cc, 0, CQ, 2 * CQ, KH, D, H, V, bg, gv, nullptr, q->S[li], o, n, WALK_DELTA));
 	seq_delta_out_kernel<<<n, SEQ_THREADS, 0, q->stream>>>(o, H, V, l.out_norm, c.norm_eps, gl, ldg, gc, on,
 	                                                       l.gate_act == YALM_GATE_SIGMOID);
 	HIPCHK(hipGetLastError());
@@ -880,18 +951,45 @@ static int mixer_ssm(Seq *q, int li, int n) {
 	seq_ssm_prep_kernel<<<cdiv(n * H, SEQ_THREADS), SEQ_THREADS, 0, q->stream>>>(q->Z, zin, inner + cc, H, l.a_log,
 	                                                                            l.dt_bias, bg, n);
 	HIPCHK(hipGetLastError());
-	TRY(delta_launch(q, xbc, cc, inner + GN, inner, 0, G, N, H, P, bg, nullptr, l.d_skip, q->S[li], y, n, true));
+	TRY(delta_launch(q, xbc, cc, inner + GN, inner, 0, G, N, H, P, bg, nullptr, l.d_skip, q->S[li], y, n, WALK_SSM));
 	seq_gated_part_norm_kernel<<<dim3(n, l.norm_groups), SEQ_THREADS, 0, q->stream>>>(y, inner, l.norm_groups, q->Z, zin, 0,
 	                                                                                  l.out_norm, c.norm_eps, yn);
 	HIPCHK(hipGetLastError());
 	return gemm(q, plain(yn, inner, l.w_o, inner, q->Yout, c.width, n, c.width, inner));
 }
 
+// Matrix memory: one input projection (queries, keys, values, output gate, log-gate logits), the
+// recurrence kernel in its matrix-memory form (a few tokens: the log gates worked out inside it; a
+// long portion: by a launch before it), the divided read-outs normed per head and gated, the output
+// projection.
+static int mixer_memory(Seq *q, int li, int n) {
+	const yalm_seq_layer &l = q->L[li];
+	const yalm_seq_config &c = q->c;
+	const int H = l.heads, D = l.dim, V = l.vdim, zin = in_rows(l), HV = H * V;
+	float *o = q->B[0], *on = q->B[1], *Z = q->Zin ? q->Zin : q->Z;
+	const int ldz = q->Zin ? q->ldz : zin, gcol = 2 * H * D + HV, icol = gcol + HV;
+	if (!q->Zin) {
+		GemmArgs g = plain(q->In, c.width, l.w_in, c.width, Z, zin, n, zin, c.width);
+		g.bias = l.in_bias;
+		TRY(gemm(q, g));
+	}
+	MemGates mg{Z + icol, ldz, l.gate_cap, 1.0f / std::sqrt((float)D), q->S[li] + (size_t)H * D * (V + 1)};
+	if (n > GEMV_MAX_M) {
+		seq_mem_gates_kernel<<<cdiv(n * 2 * H, SEQ_THREADS), SEQ_THREADS, 0, q->stream>>>(Z, ldz, icol, H, l.gate_cap, n);
+		HIPCHK(hipGetLastError());
+		mg.cap = 0.0f;
+	}
+	TRY(delta_launch(q, Z, ldz, 0, H * D, 2 * H * D, H, D, H, V, nullptr, nullptr, nullptr, q->S[li], o, n, WALK_MEMORY, mg));
+	seq_delta_out_kernel<<<n, SEQ_THREADS, 0, q->stream>>>(o, H, V, l.out_norm, c.norm_eps, Z, ldz, gcol, on, 1, V, 1);
+	HIPCHK(hipGetLastError());
+	return gemm(q, plain(on, HV, l.w_o, HV, q->Yout, c.width, n, c.width, HV));
+}
+
 // ---- the closing norm of a single token, owed to the product that reads the stream next
 static int add_norm(Seq *q, const float *wb, const float *w_next, int n, const yalm_seq_layer *moe);
 
 static bool an_foldable(const Seq *q, int n) {
-	return n == 1 && !q->c.pre_norm && !q->dump_on && q->Xalt && q->c.width % 8 == 0 && q->c.width <= 8 * 1024;
+	return n == 1 && !q->c.pre_norm && q->nk != NK_TANH && !q->dump_on && q->Xalt && q->c.width % 8 == 0 && q->c.width <= 8 * 1024;
 }
 static int flush_norm(Seq *q, int n) {
 	if (!q->pend_wb)
@@ -906,7 +1004,7 @@ static int gemv_an_t(Seq *q, const GemmArgs &a) {
 	const dim3 g(cdiv(a.N, (SEQ_THREADS / 64) * GAN_RPW));
 #define GA_LAUNCH(KI)                                                                                                  \
 	seq_gemv_an_kernel<WT, KI><<<g, SEQ_THREADS, (size_t)K * sizeof(float), q->stream>>>(                              \
-	    q->X, q->Y, q->pend_wb, q->c.norm_eps, (int)q->ln, K, q->X == q->Xbase ? q->Xalt : q->Xbase, a.W, a.N, a.C,    \
+	    q->X, q->Y, q->pend_wb, q->c.norm_eps, q->nk, q->c.residual_scale, K, q->X == q->Xbase ? q->Xalt : q->Xbase, a.W, a.N, a.C,    \
 	    a.bias, a.epi)
 	if (ki <= 1) GA_LAUNCH(1);
 	else if (ki <= 2) GA_LAUNCH(2);
@@ -1064,11 +1162,13 @@ static int mixer_attn(Seq *q, int li, int n) {
 	const bool bf = c.weight_dtype == YALM_BF16;
 	const int zin = in_rows(l), H = l.heads, V = l.vdim;
 	float *Q = q->B[0], *gate = q->B[1], *ctx = q->B[2];
+	float *Z = q->Zin ? q->Zin : q->Z;
+	const int ldz = q->Zin ? q->ldz : zin;
 	// per-head gate rows are taken by the projection kernel itself; elementwise gate rows are
 	// ordinary output columns of the input projection
 	const int zmain = zin - (l.out_gate == 1 ? H : 0);
-	{
-		GemmArgs g = plain(q->In, c.width, l.w_in, c.width, q->Z, zin, n, zmain, c.width);
+	if (!q->Zin) {
+		GemmArgs g = plain(q->In, c.width, l.w_in, c.width, Z, zin, n, zmain, c.width);
 		g.bias = l.in_bias;
 		TRY(gemm_in(q, g));
 	}
@@ -1098,6 +1198,8 @@ static int mixer_attn(Seq *q, int li, int n) {
 	a.rel_far = q->rel_far[li];
 	a.q_temp_coef = l.q_temp_coef;
 	a.q_temp_every = l.q_temp_every;
+	a.rot_half = l.rot_pairs == YALM_ROT_HALVES;
+	a.softcap = l.softcap;
 	a.eps = c.norm_eps;
 	// portions: the projection kernel (one workgroup per token) mixes the queries itself
 	a.q_mixed = l.talk && n > GEMV_MAX_M ? 1 : 0;
@@ -1108,17 +1210,17 @@ static int mixer_attn(Seq *q, int li, int n) {
 	const float *gbias = l.in_bias && a.out_gate ? l.in_bias + zmain : nullptr;
 	if (bf)
 		seq_attn_prep_kernel<uint16_t><<<pg, SEQ_THREADS, rot_lds, q->stream>>>(
-		    q->Z, zin, a, q->st, Q, (uint16_t *)q->cache[li], (uint16_t *)q->vcache[li], gate, q->In, c.width,
+		    Z, ldz, a, q->st, Q, (uint16_t *)q->cache[li], (uint16_t *)q->vcache[li], gate, q->In, c.width,
 		    (const uint16_t *)l.w_in + (size_t)zmain * c.width, gbias);
 	else
 		seq_attn_prep_kernel<float><<<pg, SEQ_THREADS, rot_lds, q->stream>>>(
-		    q->Z, zin, a, q->st, Q, (float *)q->cache[li], (float *)q->vcache[li], gate, q->In, c.width,
+		    Z, ldz, a, q->st, Q, (float *)q->cache[li], (float *)q->vcache[li], gate, q->In, c.width,
 		    (const float *)l.w_in + (size_t)zmain * c.width, gbias);
 	HIPCHK(hipGetLastError());
 	const float *gp = a.out_gate ? gate : nullptr;
-	const float *ge = l.out_gate == 2 ? q->Z + (zin - H * V) : nullptr; // elementwise gate logits close the Z rows
-	TRY(bf ? attn_core_t<uint16_t>(q, li, n, a, Q, gp, ctx, nullptr, nullptr, ge, zin)
-	       : attn_core_t<float>(q, li, n, a, Q, gp, ctx, nullptr, nullptr, ge, zin));
+	const float *ge = l.out_gate == 2 ? Z + (zin - H * V) : nullptr; // elementwise gate logits close the mixer's columns
+	TRY(bf ? attn_core_t<uint16_t>(q, li, n, a, Q, gp, ctx, nullptr, nullptr, ge, ldz)
+	       : attn_core_t<float>(q, li, n, a, Q, gp, ctx, nullptr, nullptr, ge, ldz));
 	GemmArgs o = plain(ctx, H * V, l.w_o, H * V, q->Yout, c.width, n, c.width, H * V);
 	o.bias = l.o_bias;
 	return gemm(q, o);
@@ -1241,12 +1343,21 @@ static int mixer_latent_direct(Seq *q, int li, int n) {
 	return gemm(q, o);
 }
 
-// w_down gelu(w_up x)
+// the epilogue of an ungated feed-forward's first product
+static int plain_epi(const yalm_seq_layer &l) {
+	switch (l.ff_act) {
+	case YALM_ACT_RELU2: return EPI_RELU2;
+	case YALM_ACT_GELU_ERF: return EPI_GELU_ERF;
+	default: return EPI_GELU;
+	}
+}
+
+// w_down act(w_up x)
 static int ff_plain(Seq *q, int li, int n, float *out) {
 	const yalm_seq_layer &l = q->L[li];
 	const yalm_seq_config &c = q->c;
 	GemmArgs a = plain(q->In, c.width, l.w_up, c.width, q->B[0], l.ff, n, l.ff, c.width);
-	a.epi = l.ff_act == YALM_ACT_RELU2 ? EPI_RELU2 : EPI_GELU;
+	a.epi = plain_epi(l);
 	TRY(gemm_in(q, a));
 	return gemm(q, plain(q->B[0], l.ff, l.w_down, l.ff, out, c.width, n, c.width, l.ff));
 }
@@ -1275,20 +1386,23 @@ static int ff_dense(Seq *q, int li, int n, float *out) {
 static int ff_moe(Seq *q, int li, int n) {
 	const yalm_seq_layer &l = q->L[li];
 	const yalm_seq_config &c = q->c;
-	const int E = l.experts, top = l.top, ff = l.ff, slots = n * top;
+	const int E = l.experts, ER = E + l.identity, top = l.top, ff = l.ff, slots = n * top;
 	float *hx = q->B[0], *yx = q->B[1], *hs = q->B[2], *ys = q->B[3];
-	seq_router_kernel<<<n, SEQ_THREADS, (2 * E + l.groups) * sizeof(float), q->stream>>>(q->In, c.width, l.router, E, top, l.groups,
+	seq_router_kernel<<<n, SEQ_THREADS, (2 * ER + l.groups) * sizeof(float), q->stream>>>(q->In, c.width, l.router, ER, top, l.groups,
 	                                                                    l.groups_keep, l.router_scale,
 	                                                                    l.shared_ff > 0 ? l.shared_sg : nullptr, q->idx,
 	                                                                    q->wt, q->sgate, l.router_kind, l.router_bias);
 	HIPCHK(hipGetLastError());
-	const int epi = glu_epi(l, EPI_GLU_CLAMP);
+	// experts without gate matrices are plain: one matrix, its activation, the second matrix
+	const bool glu = l.w_gate != nullptr;
+	const int epi = glu ? glu_epi(l, EPI_GLU_CLAMP) : plain_epi(l);
 	if (n <= GEMV_MAX_M) { // one batch per (token, choice): its expert's matrices picked on the device
-		GemmArgs a = plain(q->In, c.width, l.w_gate, c.width, hx, ff, 1, ff, c.width);
-		a.W2 = l.w_up;
+		GemmArgs a = plain(q->In, c.width, glu ? l.w_gate : l.w_up, c.width, hx, ff, 1, ff, c.width);
+		a.W2 = glu ? l.w_up : nullptr;
 		a.a_bs = c.width;
 		a.a_zdiv = top;
 		a.w_sel = q->idx;
+		a.w_count = E;
 		a.w_bs = (long)ff * c.width;
 		a.c_bs = ff;
 		a.epi = epi;
@@ -1297,16 +1411,17 @@ static int ff_moe(Seq *q, int li, int n) {
 		GemmArgs b = plain(hx, ff, l.w_down, ff, yx, c.width, 1, c.width, ff);
 		b.a_bs = ff;
 		b.w_sel = q->idx;
+		b.w_count = E;
 		b.w_bs = (long)c.width * ff;
 		b.c_bs = c.width;
 		TRY(gemm(q, b, slots));
 	} else { // tokens grouped by expert: one batch per expert over its row list
 		seq_fill_int_kernel<<<cdiv(E, 256), 256, 0, q->stream>>>(q->counts, E, 0);
 		seq_moe_lists_kernel<<<cdiv(slots, SEQ_THREADS), SEQ_THREADS, 0, q->stream>>>(q->idx, slots, q->counts, q->lists,
-		                                                                              q->cap);
+		                                                                              q->cap, E);
 		HIPCHK(hipGetLastError());
-		GemmArgs a = plain(q->In, c.width, l.w_gate, c.width, hx, ff, n, ff, c.width);
-		a.W2 = l.w_up;
+		GemmArgs a = plain(q->In, c.width, glu ? l.w_gate : l.w_up, c.width, hx, ff, n, ff, c.width);
+		a.W2 = glu ? l.w_up : nullptr;
 		a.w_bs = (long)ff * c.width;
 		a.rows = q->lists;
 		a.rows_bs = q->cap;
@@ -1323,8 +1438,8 @@ static int ff_moe(Seq *q, int li, int n) {
 		TRY(gemm(q, b, E, n));
 	}
 	if (l.shared_ff > 0) {
-		GemmArgs a = plain(q->In, c.width, l.ws_gate, c.width, hs, l.shared_ff, n, l.shared_ff, c.width);
-		a.W2 = l.ws_up;
+		GemmArgs a = plain(q->In, c.width, glu ? l.ws_gate : l.ws_up, c.width, hs, l.shared_ff, n, l.shared_ff, c.width);
+		a.W2 = glu ? l.ws_up : nullptr;
 		a.epi = epi;
 		a.limit = l.shared_limit;
 		TRY(gemm(q, a));
@@ -1346,9 +1461,10 @@ static int par_close(Seq *q, int li, int n) {
 #define PC_ARGS                                                                                                        \
 	q->X, q->Y, l.ls1, (l.ff_kind != YALM_FF_NONE && !moe) ? q->Y2 : nullptr, l.ls2, moe ? q->B[1] : nullptr, q->wt,    \
 	    moe ? l.top : 0, moe && l.shared_ff > 0 ? q->B[3] : nullptr, gated ? q->sgate : nullptr, dump,                 \
-	    nx ? nx->pre_add : nullptr, c.norm_eps, c.width, nx ? nx->norm1 : nullptr, q->Hn, (int)q->ln,                  \
+	    nx ? nx->pre_add : nullptr, c.norm_eps, c.width, nx ? nx->norm1 : nullptr, q->Hn, q->nk, c.residual_scale,                  \
 	    (nx && nx->ff_kind != YALM_FF_NONE) ? nx->norm2 : nullptr, q->Hn2, joined ? q->Y3 : nullptr, l.join_w,        \
-	    l.side_join_w, l.join_scale
+	    l.side_join_w, l.join_scale, l.side_join_scale, q->idx, l.experts,                                               \
+	    moe && l.identity > 0 ? (l.norm2 ? q->Hn2 : q->Hn) : nullptr
 	if (c.width <= 4 * SEQ_THREADS)
 		seq_par_close_reg_kernel<4><<<n, SEQ_THREADS, 0, q->stream>>>(PC_ARGS);
 	else if (c.width <= 8 * SEQ_THREADS)
@@ -1367,7 +1483,7 @@ static int add_norm(Seq *q, const float *wb, const float *w_next, int n, const y
 	const int w = q->c.width;
 	if (!moe && w <= 16 * SEQ_THREADS) { // the row in registers
 #define AN_LAUNCH(E)                                                                                                   \
-	seq_add_norm_reg_kernel<E><<<n, SEQ_THREADS, 0, q->stream>>>(q->X, q->Y, wb, q->c.norm_eps, w, w_next, q->Hn, (int)q->ln)
+	seq_add_norm_reg_kernel<E><<<n, SEQ_THREADS, 0, q->stream>>>(q->X, q->Y, wb, q->c.norm_eps, w, w_next, q->Hn, q->nk, q->c.residual_scale)
 		if (w <= 4 * SEQ_THREADS) AN_LAUNCH(4);
 		else if (w <= 8 * SEQ_THREADS) AN_LAUNCH(8);
 		else AN_LAUNCH(16);
@@ -1375,7 +1491,8 @@ static int add_norm(Seq *q, const float *wb, const float *w_next, int n, const y
 	} else {
 		seq_add_norm_kernel<<<n, SEQ_THREADS, w * sizeof(float), q->stream>>>(
 		    q->X, q->Y, wb, q->c.norm_eps, w, w_next, q->Hn, moe ? q->B[1] : nullptr, q->wt, moe ? moe->top : 0,
-		    moe && moe->shared_ff > 0 ? q->B[3] : nullptr, q->sgate, (int)q->ln);
+		    moe && moe->shared_ff > 0 ? q->B[3] : nullptr, moe && moe->shared_sg ? q->sgate : nullptr, q->nk,
+		    q->c.residual_scale, q->idx, moe ? moe->experts : 0, moe && moe->identity > 0 ? q->In : nullptr);
 	}
 	HIPCHK(hipGetLastError());
 	return YALM_OK;
@@ -1408,12 +1525,12 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 	if (c.weight_dtype == YALM_F32)
 		seq_embed_kernel<WF32><<<n, SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
 		                                                         c.vocab, c.embed_scale, q->X, first_norm, c.norm_eps,
-		                                                         q->Hn, (int)q->ln, q->L[0].pre_add, q->embed_norm, first_norm2,
+		                                                         q->Hn, q->nk, q->L[0].pre_add, q->embed_norm, first_norm2,
 		                                                         q->Hn2);
 	else
 		seq_embed_kernel<WBF16><<<n, SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
 		                                                          c.vocab, c.embed_scale, q->X, first_norm, c.norm_eps,
-		                                                          q->Hn, (int)q->ln, q->L[0].pre_add, q->embed_norm, first_norm2,
+		                                                          q->Hn, q->nk, q->L[0].pre_add, q->embed_norm, first_norm2,
 		                                                          q->Hn2);
 	HIPCHK(hipGetLastError());
 	auto run_mixer = [&](int mi) {
@@ -1428,6 +1545,8 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 			return mixer_attn(q, mi, n);
 		if (m.mixer == YALM_MIX_SSM)
 			return mixer_ssm(q, mi, n);
+		if (m.mixer == YALM_MIX_MEMORY)
+			return mixer_memory(q, mi, n);
 		return mixer_delta(q, mi, n);
 	};
 	for (int li = 0; li < c.n_layers; ++li) {
@@ -1437,15 +1556,27 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 		if (l.mixer != YALM_MIX_ATTN || side >= 0)
 			TRY(flush_norm(q, n)); // only a lone attention mixer's input projection takes an owed norm
 		q->Yout = q->Y;
-		TRY(run_mixer(li));
-		if (side >= 0) { // the second mixer reads the same input; the two normed results are summed into Y
+		const int own = in_rows(l), joint = side >= 0 && !q->L[side].w_in ? own + in_rows(q->L[side]) : 0;
+		if (joint) { // both mixers' input projections as one product
+			GemmArgs g = plain(q->In, c.width, l.w_in, c.width, q->Z, joint, n, joint, c.width);
+			g.bias = l.in_bias;
+			TRY(gemm(q, g));
+			q->Zin = q->Z;
+			q->ldz = joint;
+		}
+		int rc = run_mixer(li);
+		if (side >= 0 && rc == YALM_OK) { // the second mixer reads the same input; the two results are joined into Y
 			q->Yout = q->Y3;
-			const int rc = run_mixer(side);
+			q->Zin = joint ? q->Z + own : nullptr;
+			rc = run_mixer(side);
 			q->Yout = q->Y;
-			TRY(rc);
+		}
+		q->Zin = nullptr;
+		TRY(rc);
+		if (side >= 0) {
 			if (!par) { // serial blocks: joined here; a parallel block's seam joins them itself
 				seq_pair_join_kernel<<<n, SEQ_THREADS, 0, q->stream>>>(q->Y, q->Y3, l.join_w, l.side_join_w, l.join_scale,
-				                                                       c.norm_eps, c.width);
+				                                                       l.side_join_scale, c.norm_eps, c.width);
 				HIPCHK(hipGetLastError());
 			}
 		}
@@ -1486,10 +1617,15 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 static int enqueue_logits(Seq *q, const int *rows_dev, int n_rows) {
 	const yalm_seq_config &c = q->c;
 	seq_norm_kernel<float><<<n_rows, SEQ_THREADS, 0, q->stream>>>(q->X, c.width, q->final_norm, c.norm_eps, c.width,
-	                                                              q->Hn, c.width, rows_dev, q->st, 0, (int)q->ln,
+	                                                              q->Hn, c.width, rows_dev, q->st, 0, q->nk,
 	                                                              c.logit_scale);
 	HIPCHK(hipGetLastError());
-	return gemm(q, plain(q->Hn, c.width, q->head, c.width, q->logits, c.vocab, n_rows, c.vocab, c.width));
+	GemmArgs a = plain(q->Hn, c.width, q->head, c.width, q->logits, c.vocab, n_rows, c.vocab, c.width);
+	if (c.logit_softcap > 0.0f) {
+		a.epi = EPI_SOFT_CAP;
+		a.limit = c.logit_softcap;
+	}
+	return gemm(q, a);
 }
 
 extern "C" int yalm_seq_step(yalm_seq q, const int *tokens, int n, const int *want, int n_want, float *logits_host) {

@@ -1,7 +1,7 @@
 // seq_attn.h — softmax attention over cached keys and values for the layer-list engine
 // (YALM_MIX_ATTN in include/yalm_hip.h): grouped key/value heads, rotary positions on the
-// first rot_dims entries of a head (interleaved pairs, rescaled frequencies), query / key /
-// value norms, a per-head score temperature, scores mixed across heads, causal / sliding
+// first rot_dims entries of a head (interleaved or half-split pairs, rescaled frequencies), query / key /
+// value norms, a per-head score temperature, scores mixed across heads or capped by a tanh, causal / sliding
 // window / chunked masks, a softmax with an optional zero-score sink, a per-head output gate.
 // Every option is a runtime argument, so another design can combine them differently.
 //
@@ -43,7 +43,19 @@ struct AttnArgs {
 	// q_temp_every > 0: the query at position p times 1 + q_temp_coef ln(floor((p + 1) / q_temp_every) + 1)
 	float q_temp_coef = 0.0f;
 	int q_temp_every = 0;
+	int rot_half = 0;         // rotated pairs: 0: (2i, 2i + 1), 1: (i, i + rot_dims / 2)
+	float softcap = 0.0f;     // > 0: the scaled score s becomes softcap tanh(s / softcap) (before the distance bias)
 };
+
+// The capped score: exact to f32 rounding (the f32 kernels), or through one exp2 and one reciprocal,
+// cap (1 - 2 / (e^(2 s / cap) + 1)), a few f32 roundings of cap off (the matrix-core kernel, whose
+// operands carry 16 bits; c1 = 2 log2(e) / cap).
+__device__ __forceinline__ float attn_cap(float s, float cap) {
+	return cap > 0.0f ? cap * tanhf(s / cap) : s;
+}
+__device__ __forceinline__ float attn_cap_fast(float s, float cap, float c1) {
+	return fmaf(-2.0f * cap, __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(s * c1) + 1.0f), cap);
+}
 
 // The bias of head h's score between a query and a key `dist` positions before it.
 __device__ __forceinline__ float attn_rel_bias(const AttnArgs &a, int h, int dist) {
@@ -194,14 +206,15 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_attn_prep_kernel(const float 
 				if (kind == 2) {
 					v = src[d];
 				} else if (d < a.rot_dims) {
-					const int d0 = d & ~1, d1 = d | 1;
+					const int pr = a.rot_half ? (d < half ? d : d - half) : d >> 1; // the pair, its two entries
+					const int d0 = a.rot_half ? pr : d & ~1, d1 = a.rot_half ? pr + half : d | 1;
 					float u = src[d0], w = src[d1];
 					if (nw) {
 						u = u * rw * nw[d0];
 						w = w * rw * nw[d1];
 					}
-					const float c = rot[d >> 1], sn = rot[half + (d >> 1)];
-					v = (d & 1) ? w * c + u * sn : u * c - w * sn;
+					const float c = rot[pr], sn = rot[half + pr];
+					v = d == d1 ? w * c + u * sn : u * c - w * sn;
 				} else {
 					v = src[d];
 					if (nw)
@@ -534,7 +547,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_attn_kernel(const float *__re
 		for (int r = wave; r < R; r += SEQ_THREADS / 64) {
 			const int j = kt + lane;
 			const bool vis = j >= rlo[r] && j <= rhi[r] && j < k_end;
-			const float sv = vis ? ps[r * SA_KT + lane] + attn_rel_bias(a, h0 + r % Hb, rhi[r] - j) : -FLT_MAX;
+			const float sv = vis ? attn_cap(ps[r * SA_KT + lane], a.softcap) + attn_rel_bias(a, h0 + r % Hb, rhi[r] - j) : -FLT_MAX;
 			const float mold = mrun[r], lold = lrun[r];
 			const float mnew = fmaxf(mold, wave_max(sv));
 			const float p = vis ? expf(sv - mnew) : 0.0f;
@@ -763,7 +776,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_attn_decode_kernel(const floa
 #pragma unroll
 			for (int w = 0; w < NW; ++w)
 				sv += pw[(w * Hb + r) * SA_KT + lane];
-			sv = live ? sv + attn_rel_bias(a, h0 + r, pos - j) : -FLT_MAX;
+			sv = live ? attn_cap(sv, a.softcap) + attn_rel_bias(a, h0 + r, pos - j) : -FLT_MAX;
 			const float mold = mrun[r], lold = lrun[r];
 			const float mnew = fmaxf(mold, wave_max(sv));
 			const float p = live ? expf(sv - mnew) : 0.0f;
@@ -1032,6 +1045,14 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_attn_mfma_kernel(const float 
 					sacc[jt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(qh[sst], kb, sacc[jt], 0, 0, 0);
 					sacc[jt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ql[sst], kb, sacc[jt], 0, 0, 0);
 				}
+			if (a.softcap > 0.0f) {
+				const float c1 = 2.885390081777927f / a.softcap;
+#pragma unroll
+				for (int jt = 0; jt < 2; ++jt)
+#pragma unroll
+					for (int r = 0; r < 4; ++r)
+						sacc[jt][r] = attn_cap_fast(sacc[jt][r], a.softcap, c1);
+			}
 			float al[4];
 #pragma unroll
 			for (int r = 0; r < 4; ++r) {

@@ -28,6 +28,15 @@ __device__ __forceinline__ float sq_softplus(float z) {
 __device__ __forceinline__ float sq_gelu_tanh(float z) {
 	return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
+__device__ __forceinline__ float sq_gelu_erf(float z) { // the exact form, z times the normal distribution function
+	return 0.5f * z * (1.0f + erff(z * 0.7071067811865476f));
+}
+__device__ __forceinline__ float sq_log_sigmoid(float z) {
+	return fminf(z, 0.0f) - log1pf(expf(-fabsf(z)));
+}
+__device__ __forceinline__ float sq_soft_cap(float z, float cap) { // cap tanh(z / cap)
+	return cap * tanhf(z / cap);
+}
 __device__ __forceinline__ uint16_t f2bf(float x) { // round to nearest even
 	const uint32_t u = __builtin_bit_cast(uint32_t, x);
 	return (uint16_t)((u + 0x7FFFu + ((u >> 16) & 1u)) >> 16);
@@ -57,11 +66,16 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
 	return t;
 }
 
-// The two norm kinds (YALM_NORM_*): an rms norm divides a row by sqrt(mean(x^2) + eps); a layer
+// The norm kinds (YALM_NORM_*): an rms norm divides a row by sqrt(mean(x^2) + eps); a layer
 // norm first takes the row's mean off, then divides by sqrt(mean(deviation^2) + eps). Both are
-// followed by a weight and have no bias. Kernels take `ln` (1 = layer norm) and subtract the
-// mean from the entries they hold before the sum of squares (two passes over values already
-// in registers or LDS, so the variance is that of the deviations themselves).
+// followed by a weight and have no bias. Kernels take the kind `nk` and for a layer norm
+// subtract the mean from the entries they hold before the sum of squares (two passes over values
+// already in registers or LDS, so the variance is that of the deviations themselves). A tanh norm
+// has no statistics: tanh(alpha x) w + b per entry, its weight vector being [w: n | b: n | alpha].
+enum { NK_RMS = YALM_NORM_RMS, NK_LAYER = YALM_NORM_LAYER, NK_TANH = YALM_NORM_TANH };
+__device__ __forceinline__ float tanh_norm(const float *__restrict__ w, int n, int i, float x) {
+	return fmaf(tanhf(w[2 * n] * x), w[i], w[n + i]);
+}
 
 // ------------------------------------------------------------------ embedding
 // X[t] = embed[token] * scale (+ the interleaved (sin, cos) position vector of position
@@ -77,7 +91,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
                                                                 const float *__restrict__ inv_freq, int width,
                                                                 int vocab, float scale, float *__restrict__ X,
                                                                 const float *__restrict__ w_next, float eps,
-                                                                float *__restrict__ Hn, int ln,
+                                                                float *__restrict__ Hn, int nk,
                                                                 const float *__restrict__ pre_add = nullptr,
                                                                 const float *__restrict__ e_norm = nullptr,
                                                                 const float *__restrict__ w_next2 = nullptr,
@@ -117,8 +131,17 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 	if (!w_next)
 		return;
 	// the first layer's opening norm in the same launch (each thread re-reads its own entries)
+	if (nk == NK_TANH) {
+		for (int i = threadIdx.x; i < width; i += SEQ_THREADS) {
+			const float v = X[(size_t)t * width + i];
+			Hn[(size_t)t * width + i] = tanh_norm(w_next, width, i, v);
+			if (w_next2)
+				Hn2[(size_t)t * width + i] = tanh_norm(w_next2, width, i, v);
+		}
+		return;
+	}
 	float mu = 0.0f;
-	if (ln) {
+	if (nk == NK_LAYER) {
 		mu = block_sum(sm, red) / (float)width;
 		ss = 0.0f;
 		for (int i = threadIdx.x; i < width; i += SEQ_THREADS) {
@@ -145,12 +168,23 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_norm_kernel(const float *__re
                                                                OT *__restrict__ out, int ld_out,
                                                                const int *__restrict__ rows,
                                                                const StepState *__restrict__ st, int pos_rows,
-                                                               int ln = 0, float post = 1.0f) {
+                                                               int nk = NK_RMS, float post = 1.0f) {
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
 	const float *x = in + (size_t)(rows ? rows[t] : t) * ld_in;
+	OT *o = out + (size_t)(pos_rows ? st->pos + t : t) * ld_out;
+	if (nk == NK_TANH) {
+		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
+			const float v = tanh_norm(w, n, i, x[i]) * post;
+			if constexpr (sizeof(OT) == 2)
+				o[i] = f2bf(v);
+			else
+				o[i] = v;
+		}
+		return;
+	}
 	float mu = 0.0f;
-	if (ln) {
+	if (nk == NK_LAYER) {
 		float sm = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
 			sm += x[i];
@@ -163,7 +197,6 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_norm_kernel(const float *__re
 	}
 	ss = block_sum(ss, red);
 	const float r = post / sqrtf(ss / (float)n + eps);
-	OT *o = out + (size_t)(pos_rows ? st->pos + t : t) * ld_out;
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
 		const float v = (x[i] - mu) * r * w[i];
 		if constexpr (sizeof(OT) == 2)
@@ -205,8 +238,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_norm2_kernel(const float *__r
 	}
 }
 
-// The seam between two sublayers in one launch: X[t] += norm(Y[t]) * wb (the closing norm
-// of the sublayer that produced Y and the residual sum), then, if w_next, Hn[t] =
+// The seam between two sublayers in one launch: X[t] += rs norm(Y[t]) * wb (the closing norm
+// of the sublayer that produced Y and the residual sum, scaled by rs), then, if w_next, Hn[t] =
 // norm(X[t]) * w_next (the opening norm of the next sublayer). Dynamic LDS: n floats.
 // Rows of up to E * SEQ_THREADS entries without a combine: the row of Y, the row of X and both
 // weight vectors are loaded at once (one memory round trip instead of one per pass) and the
@@ -216,7 +249,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
                                                                        const float *__restrict__ Y,
                                                                        const float *__restrict__ wb, float eps, int n,
                                                                        const float *__restrict__ w_next,
-                                                                       float *__restrict__ Hn, int ln) {
+                                                                       float *__restrict__ Hn, int nk, float rs) {
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
 	float y[E], x[E], b[E], wn[E];
@@ -229,7 +262,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 		b[e] = in ? wb[i] : 0.0f;
 		wn[e] = (in && w_next) ? w_next[i] : 0.0f;
 	}
-	if (ln) { // entries past the row's end stay 0
+	if (nk == NK_LAYER) { // entries past the row's end stay 0
 		float sm = 0.0f;
 #pragma unroll
 		for (int e = 0; e < E; ++e)
@@ -240,12 +273,22 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 			if (threadIdx.x + e * SEQ_THREADS < n)
 				y[e] -= mu;
 	}
-	float ss = 0.0f;
+	float r = rs;
+	if (nk == NK_TANH) {
 #pragma unroll
-	for (int e = 0; e < E; ++e)
-		ss = fmaf(y[e], y[e], ss);
-	ss = block_sum(ss, red);
-	const float r = 1.0f / sqrtf(ss / (float)n + eps);
+		for (int e = 0; e < E; ++e) {
+			const int i = threadIdx.x + e * SEQ_THREADS;
+			y[e] = i < n ? tanh_norm(wb, n, i, y[e]) : 0.0f;
+			b[e] = 1.0f;
+		}
+	} else {
+		float ss = 0.0f;
+#pragma unroll
+		for (int e = 0; e < E; ++e)
+			ss = fmaf(y[e], y[e], ss);
+		ss = block_sum(ss, red);
+		r = rs / sqrtf(ss / (float)n + eps);
+	}
 	float s2 = 0.0f, sm2 = 0.0f;
 #pragma unroll
 	for (int e = 0; e < E; ++e) {
@@ -259,7 +302,16 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 	}
 	if (!w_next)
 		return;
-	if (ln) {
+	if (nk == NK_TANH) {
+#pragma unroll
+		for (int e = 0; e < E; ++e) {
+			const int i = threadIdx.x + e * SEQ_THREADS;
+			if (i < n)
+				Hn[(size_t)t * n + i] = tanh_norm(w_next, n, i, x[e]);
+		}
+		return;
+	}
+	if (nk == NK_LAYER) {
 		const float mu = block_sum(sm2, red) / (float)n;
 		s2 = 0.0f;
 #pragma unroll
@@ -279,16 +331,27 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 	}
 }
 
+// Slot k of token t in the routed experts' combine: the row its expert computed (Yx [slot][n]), or,
+// for a choice past the `n_exp` experts (an identity output), the feed-forward's own input row.
+__device__ __forceinline__ const float *combine_row(const float *Yx, const int *idx, int n_exp, const float *hid, int t,
+                                                    int top, int k, int n) {
+	const size_t slot = (size_t)t * top + k;
+	return (hid && idx[slot] >= n_exp) ? hid + (size_t)t * n : Yx + slot * n;
+}
+
 // Yx != null: Y is not read; its row is the routed experts' combine sum_k wt[t][k] Yx[t top + k]
-// (+ sgate[t] Ys[t], the shared expert), summed in slot order.
+// (+ sgate[t] Ys[t], the shared expert; sgate == nullptr: + Ys[t]), summed in slot order; hid: see
+// combine_row (may be Hn itself: every entry is read before it is overwritten).
 __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__restrict__ X, const float *__restrict__ Y,
                                                                    const float *__restrict__ wb, float eps, int n,
                                                                    const float *__restrict__ w_next,
-                                                                   float *__restrict__ Hn,
+                                                                   float *Hn,
                                                                    const float *__restrict__ Yx,
                                                                    const float *__restrict__ wt, int top,
                                                                    const float *__restrict__ Ys,
-                                                                   const float *__restrict__ sgate, int ln) {
+                                                                   const float *__restrict__ sgate, int nk, float rs,
+                                                                   const int *__restrict__ idx = nullptr,
+                                                                   int n_exp = 0, const float *hid = nullptr) {
 	extern __shared__ float row[];
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
@@ -299,9 +362,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		if (Yx) {
 			v = 0.0f;
 			for (int k = 0; k < top; ++k)
-				v = fmaf(wt[(size_t)t * top + k], Yx[((size_t)t * top + k) * n + i], v);
+				v = fmaf(wt[(size_t)t * top + k], combine_row(Yx, idx, n_exp, hid, t, top, k, n)[i], v);
 			if (Ys)
-				v = fmaf(sgate[t], Ys[(size_t)t * n + i], v);
+				v = fmaf(sgate ? sgate[t] : 1.0f, Ys[(size_t)t * n + i], v);
 		} else {
 			v = Y[(size_t)t * n + i];
 		}
@@ -310,7 +373,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		sm += v;
 	}
 	float mu = 0.0f;
-	if (ln) { // each thread re-reads the entries it wrote
+	if (nk == NK_LAYER) { // each thread re-reads the entries it wrote
 		mu = block_sum(sm, red) / (float)n;
 		ss = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
@@ -318,11 +381,12 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 			ss = fmaf(d, d, ss);
 		}
 	}
-	ss = block_sum(ss, red);
-	const float r = 1.0f / sqrtf(ss / (float)n + eps);
+	float r = rs;
+	if (nk != NK_TANH)
+		r = rs / sqrtf(block_sum(ss, red) / (float)n + eps);
 	float s2 = 0.0f, sm2 = 0.0f;
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
-		const float v = x[i] + (row[i] - mu) * r * wb[i];
+		const float v = x[i] + (nk == NK_TANH ? tanh_norm(wb, n, i, row[i]) * r : (row[i] - mu) * r * wb[i]);
 		x[i] = v;
 		row[i] = v;
 		s2 = fmaf(v, v, s2);
@@ -330,8 +394,13 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 	}
 	if (!w_next)
 		return;
+	if (nk == NK_TANH) {
+		for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
+			Hn[(size_t)t * n + i] = tanh_norm(w_next, n, i, row[i]);
+		return;
+	}
 	float mu2 = 0.0f;
-	if (ln) {
+	if (nk == NK_LAYER) {
 		mu2 = block_sum(sm2, red) / (float)n;
 		s2 = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
@@ -345,16 +414,17 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		Hn[(size_t)t * n + i] = (row[i] - mu2) * r2 * w_next[i];
 }
 
-// The seam after a parallel block, one launch: X[t] += s1 * Y1[t] + s2 * Y2[t] (s1, s2 the
-// block's elementwise scales; Y2 == nullptr and Yx == nullptr: no feed-forward). Yx != nullptr:
+// The seam after a parallel block, one launch: X[t] += rs (s1 * Y1[t] + s2 * Y2[t]) (rs the model's
+// residual scale, s1, s2 the block's elementwise scales; Y2 == nullptr and Yx == nullptr: no feed-forward). Yx != nullptr:
 // the feed-forward's row is the routed experts' combine sum_k wt[t][k] Yx[t top + k] (+ sgate[t]
-// Ys[t], the shared expert; sgate == nullptr: + Ys[t]), summed in slot order. dump != nullptr:
-// the row after the sums is also written there (the stream as the block leaves it). Then
+// Ys[t], the shared expert; sgate == nullptr: + Ys[t]), summed in slot order; hid: see combine_row
+// (may be Hn or Hn2: every entry is read before it is overwritten). dump != nullptr: the row after the sums is also written there (the stream as the block leaves it). Then
 // X[t] += add (the vector the next layer adds before its opening norm) and, if w_next, Hn[t]
 // = norm(X[t]) * w_next and, with w_next2, Hn2[t] = norm(X[t]) * w_next2 (the norm the next
 // block's feed-forward reads). s1 / s2 == nullptr: scale 1. Yb != nullptr: the block has two
 // mixers side by side and its mixer row is jscale (rms(Y1[t]) ja + rms(Yb[t]) jb), each row
-// divided by its own root mean square over n (no mean taken off). Dynamic LDS: n floats.
+// divided by its own root mean square over n (no mean taken off), or, ja == nullptr, the plain
+// sum jscale Y1[t] + jscale_b Yb[t]. Dynamic LDS: n floats.
 __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__restrict__ X, const float *__restrict__ Y1,
                                                                     const float *__restrict__ s1,
                                                                     const float *__restrict__ Y2,
@@ -366,19 +436,21 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
                                                                     float *__restrict__ dump,
                                                                     const float *__restrict__ add, float eps, int n,
                                                                     const float *__restrict__ w_next,
-                                                                    float *__restrict__ Hn, int ln,
+                                                                    float *Hn, int nk, float rs,
                                                                     const float *__restrict__ w_next2 = nullptr,
-                                                                    float *__restrict__ Hn2 = nullptr,
+                                                                    float *Hn2 = nullptr,
                                                                     const float *__restrict__ Yb = nullptr,
                                                                     const float *__restrict__ ja = nullptr,
                                                                     const float *__restrict__ jb = nullptr,
-                                                                    float jscale = 1.0f) {
+                                                                    float jscale = 1.0f, float jscale_b = 1.0f,
+                                                                    const int *__restrict__ idx = nullptr,
+                                                                    int n_exp = 0, const float *hid = nullptr) {
 	extern __shared__ float row[];
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
 	float *x = X + (size_t)t * n;
-	float ra = 1.0f, rb = 0.0f;
-	if (Yb) {
+	float ra = jscale, rb = jscale_b;
+	if (Yb && ja) {
 		float sa = 0.0f, sb = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
 			const float a = Y1[(size_t)t * n + i], b = Yb[(size_t)t * n + i];
@@ -392,17 +464,17 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
 		float y1 = Y1[(size_t)t * n + i];
 		if (Yb)
-			y1 = y1 * ra * ja[i] + Yb[(size_t)t * n + i] * rb * jb[i];
-		float v = fmaf(s1 ? s1[i] : 1.0f, y1, x[i]);
+			y1 = y1 * ra * (ja ? ja[i] : 1.0f) + Yb[(size_t)t * n + i] * rb * (ja ? jb[i] : 1.0f);
+		float v = fmaf(rs * (s1 ? s1[i] : 1.0f), y1, x[i]);
 		if (Yx) {
 			float f = 0.0f;
 			for (int k = 0; k < top; ++k)
-				f = fmaf(wt[(size_t)t * top + k], Yx[((size_t)t * top + k) * n + i], f);
+				f = fmaf(wt[(size_t)t * top + k], combine_row(Yx, idx, n_exp, hid, t, top, k, n)[i], f);
 			if (Ys)
 				f = fmaf(sgate ? sgate[t] : 1.0f, Ys[(size_t)t * n + i], f);
-			v = fmaf(s2 ? s2[i] : 1.0f, f, v);
+			v = fmaf(rs * (s2 ? s2[i] : 1.0f), f, v);
 		} else if (Y2) {
-			v = fmaf(s2 ? s2[i] : 1.0f, Y2[(size_t)t * n + i], v);
+			v = fmaf(rs * (s2 ? s2[i] : 1.0f), Y2[(size_t)t * n + i], v);
 		}
 		if (dump)
 			dump[(size_t)t * n + i] = v;
@@ -415,8 +487,16 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
 	}
 	if (!w_next)
 		return;
+	if (nk == NK_TANH) {
+		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
+			Hn[(size_t)t * n + i] = tanh_norm(w_next, n, i, row[i]);
+			if (w_next2)
+				Hn2[(size_t)t * n + i] = tanh_norm(w_next2, n, i, row[i]);
+		}
+		return;
+	}
 	float mu = 0.0f;
-	if (ln) { // each thread re-reads the entries it wrote
+	if (nk == NK_LAYER) { // each thread re-reads the entries it wrote
 		mu = block_sum(sm, red) / (float)n;
 		ss = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
@@ -448,13 +528,15 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
                                                                         float *__restrict__ dump,
                                                                         const float *__restrict__ add, float eps, int n,
                                                                         const float *__restrict__ w_next,
-                                                                        float *__restrict__ Hn, int ln,
+                                                                        float *Hn, int nk, float rs,
                                                                         const float *__restrict__ w_next2 = nullptr,
-                                                                        float *__restrict__ Hn2 = nullptr,
+                                                                        float *Hn2 = nullptr,
                                                                         const float *__restrict__ Yb = nullptr,
                                                                         const float *__restrict__ ja = nullptr,
                                                                         const float *__restrict__ jb = nullptr,
-                                                                        float jscale = 1.0f) {
+                                                                        float jscale = 1.0f, float jscale_b = 1.0f,
+                                                                        const int *__restrict__ idx = nullptr,
+                                                                        int n_exp = 0, const float *hid = nullptr) {
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
 	float x[E], y1[E], a1[E], f[E], a2[E], ad[E], wn[E];
@@ -465,13 +547,19 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 		const bool in = i < n;
 		x[e] = in ? X[(size_t)t * n + i] : 0.0f;
 		y1[e] = in ? Y1[(size_t)t * n + i] : 0.0f;
-		a1[e] = in ? (s1 ? s1[i] : 1.0f) : 0.0f;
-		a2[e] = (in && ff) ? (s2 ? s2[i] : 1.0f) : 0.0f;
+		a1[e] = in ? rs * (s1 ? s1[i] : 1.0f) : 0.0f;
+		a2[e] = (in && ff) ? rs * (s2 ? s2[i] : 1.0f) : 0.0f;
 		ad[e] = (in && add) ? add[i] : 0.0f;
 		wn[e] = (in && w_next) ? w_next[i] : 0.0f;
 		f[e] = (in && Y2 && !Yx) ? Y2[(size_t)t * n + i] : 0.0f;
 	}
-	if (Yb) { // two mixers side by side: the normed rows joined before anything else reads y1
+	if (Yb && !ja) { // two mixers side by side, a plain weighted sum
+#pragma unroll
+		for (int e = 0; e < E; ++e) {
+			const int i = threadIdx.x + e * SEQ_THREADS;
+			y1[e] = i < n ? y1[e] * jscale + Yb[(size_t)t * n + i] * jscale_b : 0.0f;
+		}
+	} else if (Yb) { // two mixers side by side: the normed rows joined before anything else reads y1
 		float yb[E], sa = 0.0f, sb = 0.0f;
 #pragma unroll
 		for (int e = 0; e < E; ++e) {
@@ -492,10 +580,11 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	if (Yx) {
 		for (int k = 0; k < top; ++k) {
 			const float w = wt[(size_t)t * top + k];
+			const float *src = combine_row(Yx, idx, n_exp, hid, t, top, k, n);
 #pragma unroll
 			for (int e = 0; e < E; ++e) {
 				const int i = threadIdx.x + e * SEQ_THREADS;
-				f[e] = fmaf(w, i < n ? Yx[((size_t)t * top + k) * n + i] : 0.0f, f[e]);
+				f[e] = fmaf(w, i < n ? src[i] : 0.0f, f[e]);
 			}
 		}
 		if (Ys) {
@@ -526,7 +615,19 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	}
 	if (!w_next)
 		return;
-	if (ln) {
+	if (nk == NK_TANH) {
+#pragma unroll
+		for (int e = 0; e < E; ++e) {
+			const int i = threadIdx.x + e * SEQ_THREADS;
+			if (i < n) {
+				Hn[(size_t)t * n + i] = tanh_norm(w_next, n, i, x[e]);
+				if (w_next2)
+					Hn2[(size_t)t * n + i] = tanh_norm(w_next2, n, i, x[e]);
+			}
+		}
+		return;
+	}
+	if (nk == NK_LAYER) {
 		const float mu = block_sum(sm, red) / (float)n;
 		ss = 0.0f;
 #pragma unroll
@@ -550,15 +651,21 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 }
 
 // Two mixers side by side: Ya[t] <- scale (rms(Ya[t]) wa + rms(Yb[t]) wb), each row divided by
-// its own root mean square over n (no mean taken off). One workgroup per token.
+// its own root mean square over n (no mean taken off); wa == nullptr: scale Ya[t] + scale_b Yb[t].
+// One workgroup per token.
 __global__ __launch_bounds__(SEQ_THREADS) void seq_pair_join_kernel(float *__restrict__ Ya, const float *__restrict__ Yb,
                                                                     const float *__restrict__ wa,
-                                                                    const float *__restrict__ wb, float scale, float eps,
-                                                                    int n) {
+                                                                    const float *__restrict__ wb, float scale, float scale_b,
+                                                                    float eps, int n) {
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
 	float *a = Ya + (size_t)t * n;
 	const float *b = Yb + (size_t)t * n;
+	if (!wa) {
+		for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
+			a[i] = a[i] * scale + b[i] * scale_b;
+		return;
+	}
 	float sa = 0.0f, sb = 0.0f;
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
 		sa = fmaf(a[i], a[i], sa);
@@ -582,7 +689,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gate_mul_kernel(float *__rest
 }
 
 // ------------------------------------------------------------------ matrix products
-enum { EPI_NONE = 0, EPI_GLU_GELU = 1, EPI_GLU_CLAMP = 2, EPI_SIGMOID = 3, EPI_GELU = 4, EPI_GLU_SILU = 5, EPI_RELU2 = 6 };
+enum { EPI_NONE = 0, EPI_GLU_GELU = 1, EPI_GLU_CLAMP = 2, EPI_SIGMOID = 3, EPI_GELU = 4, EPI_GLU_SILU = 5, EPI_RELU2 = 6,
+       EPI_GELU_ERF = 7, EPI_SOFT_CAP = 8 /* limit tanh(. / limit) */ };
 
 // C[c_row(m)][n] = epi(sum_k A[a_row(m)][k] W[n][k]) for every batch z = blockIdx.z.
 struct GemmArgs {
@@ -594,6 +702,7 @@ struct GemmArgs {
 	int ldw = 0;
 	long w_bs = 0;
 	const int *w_sel = nullptr; // != null: batch z reads matrix w_sel[z]
+	int w_count = 0;            // w_sel with w_count > 0: a batch whose w_sel[z] >= w_count has no rows
 	float *C = nullptr;
 	int ldc = 0;
 	long c_bs = 0;
@@ -630,6 +739,8 @@ __device__ __forceinline__ float epi_apply(const GemmArgs &a, float v, float v2,
 		const float r = fmaxf(v + b, 0.0f);
 		return r * r;
 	}
+	case EPI_GELU_ERF: return sq_gelu_erf(v + b);
+	case EPI_SOFT_CAP: return sq_soft_cap(v + b, a.limit);
 	default: return v + b;
 	}
 }
@@ -650,14 +761,17 @@ __device__ __forceinline__ GemmBatch gemm_batch(const GemmArgs &a, int z) {
 		z -= a.z_split;
 	const long za = a.a_zdiv > 0 ? z / a.a_zdiv : z;
 	b.A = a.A + za * a.a_bs;
-	const long zw = a.w_sel ? a.w_sel[z] : z;
+	long zw = a.w_sel ? a.w_sel[z] : z;
+	const bool none = a.w_sel && a.w_count > 0 && zw >= a.w_count;
+	if (none)
+		zw = 0;
 	b.W = (const char *)(second ? a.W_b : a.W) + zw * a.w_bs * WT::BYTES;
 	b.W2 = a.W2 ? (const char *)a.W2 + zw * a.w_bs * WT::BYTES : nullptr;
 	b.C = (second ? a.C_b : a.C) + (long)z * a.c_bs;
 	const float *bias = second ? a.bias_b : a.bias;
 	b.bias = bias ? bias + (long)z * a.bias_bs : nullptr;
 	b.rows = a.rows ? a.rows + (long)z * a.rows_bs : nullptr;
-	b.M = a.counts ? a.counts[z] : a.M;
+	b.M = none ? 0 : (a.counts ? a.counts[z] : a.M);
 	return b;
 }
 
@@ -798,7 +912,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 	}
 }
 
-// ---- one token, the previous sublayer's closing norm folded in: x' = x + norm(y) wb is what
+// ---- one token, the previous sublayer's closing norm (rms or layer) folded in: x' = x + rs norm(y) wb is what
 // the product reads when sublayers read the stream itself. Every workgroup rebuilds x' once
 // (a thread KI groups of 4 entries, the row's statistics over the workgroup) into LDS, while
 // its waves' first weight rows are already in flight; then each wave multiplies RPW weight
@@ -808,7 +922,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 #define GAN_RPW 2
 template <class WT, int KI>
 __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_an_kernel(const float *__restrict__ X, const float *__restrict__ Y,
-                                                                  const float *__restrict__ wb, float eps, int ln, int K,
+                                                                  const float *__restrict__ wb, float eps, int nk, float rs,
+                                                                  int K,
                                                                   float *__restrict__ Xout, const void *__restrict__ W,
                                                                   int N, float *__restrict__ C,
                                                                   const float *__restrict__ bias, int epi) {
@@ -841,7 +956,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_an_kernel(const float *_
 		b[i] = in ? *(const float4_t *)(wb + k) : float4_t{0, 0, 0, 0};
 		sm += (y[i][0] + y[i][1]) + (y[i][2] + y[i][3]);
 	}
-	if (ln) { // entries past the row's end stay 0
+	if (nk == NK_LAYER) { // entries past the row's end stay 0
 		const float mu = block_sum(sm, red) / (float)K;
 #pragma unroll
 		for (int i = 0; i < KI; ++i)
@@ -856,7 +971,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_an_kernel(const float *_
 #pragma unroll
 		for (int e = 0; e < 4; ++e)
 			ss = fmaf(y[i][e], y[i][e], ss);
-	const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)K + eps);
+	const float r = rs / sqrtf(block_sum(ss, red) / (float)K + eps);
 #pragma unroll
 	for (int i = 0; i < KI; ++i) {
 		const int k = 4 * (tid + SEQ_THREADS * i);
@@ -1448,6 +1563,22 @@ __device__ __forceinline__ float sum_lanes(float v) { // over aligned groups of 
 	return v;
 }
 
+// A matrix memory's log gates from their logits: cap tanh(z / cap), for the forget gate its log sigmoid.
+__device__ __forceinline__ float mem_log_gate(float z, float cap, bool forget) {
+	const float c = sq_soft_cap(z, cap);
+	return forget ? sq_log_sigmoid(c) : c;
+}
+// The same for all tokens of a long portion, in place: Z columns gcol .. + H (input), + 2 H (forget).
+__global__ __launch_bounds__(SEQ_THREADS) void seq_mem_gates_kernel(float *__restrict__ Z, int ldz, int gcol, int H,
+                                                                    float cap, int T) {
+	const int i = blockIdx.x * SEQ_THREADS + threadIdx.x;
+	if (i >= T * 2 * H)
+		return;
+	const int t = i / (2 * H), c = i - t * 2 * H;
+	float *z = Z + (size_t)t * ldz + gcol + c;
+	*z = mem_log_gate(*z, cap, c >= H);
+}
+
 // The recurrence itself. The columns of a head's [dim][vdim] state never mix, so one group
 // of LPC (8 or 16) lanes owns one column (each lane a contiguous slice of R dim entries, in
 // registers; LPC R >= dim) and walks the portion's tokens in order:
@@ -1459,37 +1590,50 @@ __device__ __forceinline__ float sum_lanes(float v) { // over aligned groups of 
 // and double the workgroups of a walk that fills a fraction of the chip.
 // SSM: the state-space form of the same walk, S *= g; S += k (beta v); o = S.q + dskip[h] v
 // (no prediction S.k is taken off the write; k, q, v, beta are the layer's B, C, x and dt).
+// MEM (with SSM): the matrix memory's walk. Its factors come from log gates: LG row t holds the log
+// input gates of the heads, then their log forget gates (gcap > 0: still raw, see mem_log_gates);
+// with the running maximum m <- max(lf + m', li) (m' the one before) g = exp(lf + m' - m) and
+// beta = exp(li - m). A chunk's maxima are a prefix scan over its tokens, taken by the first wave
+// as it stages the chunk. The state has one more column, written with v = 1 (the normaliser): the
+// read-outs O [t][H][V + 1] are oscale S.q, in the last column max(|oscale S.q|, exp(-m)) + 1e-6, the
+// divisor of the others. mst [H][gridDim.x]: the running maximum, one copy per workgroup of a head
+// (each reads and writes its own).
 // GVEC: g is a vector over the key channels, GV [T][H D], instead of one number per head.
 // QKV [T][ldq]: key/query head kh's q at column qo + kh D, its k at ko + kh D, head h's v at vo + h V.
-template <int R, int TC, bool SSM, bool GVEC, int LPC>
+template <int R, int TC, bool SSM, bool GVEC, int LPC, bool MEM = false>
 __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__restrict__ QKV, int ldq, int qo_, int ko_,
                                                                 int vo_, int KH, int D, int H, int V,
                                                                 const float *__restrict__ BG,
                                                                 const float *__restrict__ GV,
                                                                 const float *__restrict__ dskip,
                                                                 float *__restrict__ state, float *__restrict__ O,
-                                                                int T) {
+                                                                int T, const float *__restrict__ LG = nullptr,
+                                                                int ldlg = 0, float gcap = 0.0f,
+                                                                float oscale = 1.0f, float *__restrict__ mst = nullptr) {
 	constexpr int DP = LPC * R;                    // padded key dimension
 	constexpr int NS = GVEC ? 3 : 2;               // staged rows per token: k | q (| g)
 	constexpr int NKQ = TC * NS * DP / SEQ_THREADS; // staged values per thread and chunk
 	constexpr int COLS = SEQ_THREADS / LPC, NV = (TC * COLS + SEQ_THREADS - 1) / SEQ_THREADS;
 	static_assert((LPC == 8 || LPC == 16) && (TC * NS * DP) % SEQ_THREADS == 0, "staging assumes whole passes of the workgroup");
 	__shared__ __attribute__((aligned(16))) float kq[2][TC][NS * DP];
-	__shared__ float vs[2][TC][COLS], bgs[2][TC][2];
+	static_assert(!MEM || (SSM && !GVEC && TC <= 16), "the matrix memory walks as the state-space form, at most 16 tokens a chunk");
+	__shared__ float vs[2][TC][COLS], bgs[2][TC][MEM ? 3 : 2];
 	const int tid = threadIdx.x;
 	const int h = blockIdx.y, kh = h / (H / KH);
 	const int c0 = blockIdx.x * COLS, col = c0 + tid / LPC, sub = tid % LPC;
-	const bool live = col < V;
+	const int VS = MEM ? V + 1 : V; // columns of the state
+	const bool live = col < VS;
 	const int d0 = sub * R; // this lane's slice of the key dimension: d0 .. d0 + R - 1
 	float S[R];
-	float *sp = state + (size_t)h * D * V;
+	float *sp = state + (size_t)h * D * VS;
 #pragma unroll
 	for (int i = 0; i < R; ++i)
-		S[i] = (live && d0 + i < D) ? sp[(size_t)(d0 + i) * V + col] : 0.0f;
+		S[i] = (live && d0 + i < D) ? sp[(size_t)(d0 + i) * VS + col] : 0.0f;
 	const int qo = qo_ + kh * D, ko = ko_ + kh * D, vo = vo_ + h * V;
 	const float dsk = (SSM && dskip) ? dskip[h] : 0.0f;
 	// a chunk of TC tokens: global -> registers (in flight while the previous chunk is applied) -> LDS
-	float rkq[NKQ], rv[NV], rbg = 0.0f;
+	float rkq[NKQ], rv[NV], rbg = 0.0f, rlf = 0.0f;
+	float mrun = MEM ? mst[(size_t)h * gridDim.x + blockIdx.x] : 0.0f; // kept by the first wave
 	auto fetch = [&](int t0) {
 #pragma unroll
 		for (int i = 0; i < NKQ; ++i) {
@@ -1510,8 +1654,20 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 			const int idx = tid + i * SEQ_THREADS;
 			const int tt = idx / COLS, cc = idx % COLS, t = t0 + tt;
 			rv[i] = (tt < TC && t < T && c0 + cc < V) ? QKV[(size_t)t * ldq + vo + c0 + cc] : 0.0f;
+			if (MEM && c0 + cc == V)
+				rv[i] = 1.0f;
 		}
-		if (tid < 2 * TC) {
+		if constexpr (MEM) {
+			if (tid < TC) { // identities of the scan past the portion's end
+				const int t = t0 + tid;
+				rbg = t < T ? LG[(size_t)t * ldlg + h] : -1e30f;
+				rlf = t < T ? LG[(size_t)t * ldlg + H + h] : 0.0f;
+				if (gcap > 0.0f && t < T) {
+					rbg = mem_log_gate(rbg, gcap, false);
+					rlf = mem_log_gate(rlf, gcap, true);
+				}
+			}
+		} else if (tid < 2 * TC) {
 			const int t = t0 + (tid >> 1);
 			rbg = t < T ? BG[(size_t)t * 2 * H + (tid & 1) * H + h] : 0.0f;
 		}
@@ -1528,8 +1684,32 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 			if (idx < TC * COLS)
 				vs[buf][idx / COLS][idx % COLS] = rv[i];
 		}
-		if (tid < 2 * TC)
+		if constexpr (MEM) {
+			if (tid < 64) {
+				// m after token tt = max(m0 + A, B) with (A, B) the inclusive scan of (lf, li) over the chunk
+				const int tt = tid & 15;
+				const float li = tt < TC ? __shfl(rbg, tt) : -1e30f, lf = tt < TC ? __shfl(rlf, tt) : 0.0f;
+				float A = lf, B = li;
+#pragma unroll
+				for (int d = 1; d < 16; d <<= 1) {
+					const float pa = __shfl_up(A, d, 16), pb = __shfl_up(B, d, 16);
+					if (tt >= d) {
+						B = fmaxf(pb + A, B);
+						A += pa;
+					}
+				}
+				const float m = fmaxf(mrun + A, B), up = __shfl_up(m, 1, 16);
+				const float before = tt == 0 ? mrun : up;
+				if (tid < TC) {
+					bgs[buf][tid][0] = expf(li - m);
+					bgs[buf][tid][1] = expf(lf + before - m);
+					bgs[buf][tid][2] = expf(-m);
+				}
+				mrun = __shfl(m, 15);
+			}
+		} else if (tid < 2 * TC) {
 			bgs[buf][tid >> 1][tid & 1] = rbg;
+		}
 	};
 	fetch(0);
 	stash(0);
@@ -1544,7 +1724,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 		// turn), so that the LDS round trip runs under the previous token's dependent chain.
 		struct Tok {
 			float k[R], q[R], gv[GVEC ? R : 1];
-			float v, beta, g;
+			float v, beta, g, em;
 		};
 		auto load = [&](int tt, Tok &x) {
 			if constexpr (R % 4 == 0) {
@@ -1576,6 +1756,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 			x.v = vs[buf][tt][tid / LPC];
 			x.beta = bgs[buf][tt][0];
 			x.g = bgs[buf][tt][1];
+			if constexpr (MEM)
+				x.em = bgs[buf][tt][2];
 		};
 		auto apply = [&](int tt, const Tok &x) {
 			float dd0 = 0.0f, dd1 = 0.0f;
@@ -1607,10 +1789,15 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 					o0 = fmaf(S[i], x.q[i], o0);
 			}
 			float o = sum_lanes<LPC>(o0 + o1);
-			if constexpr (SSM)
+			if constexpr (MEM) {
+				o *= oscale;
+				if (col == V)
+					o = fmaxf(fabsf(o), x.em) + 1e-6f;
+			} else if constexpr (SSM) {
 				o = fmaf(dsk, x.v, o);
+			}
 			if (sub == 0 && live)
-				O[(size_t)(t0 + tt) * H * V + h * V + col] = o;
+				O[(size_t)(t0 + tt) * H * VS + h * VS + col] = o;
 		};
 		Tok xa, xb;
 		load(0, xa);
@@ -1633,30 +1820,36 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 #pragma unroll
 		for (int i = 0; i < R; ++i)
 			if (d0 + i < D)
-				sp[(size_t)(d0 + i) * V + col] = S[i];
+				sp[(size_t)(d0 + i) * VS + col] = S[i];
 	}
+	if (MEM && tid == 0)
+		mst[(size_t)h * gridDim.x + blockIdx.x] = mrun;
 }
 
-// Each head's read-out divided by its root mean square over vdim, times the shared weight,
-// times the output gate: silu (sig == 0) or sigmoid (sig != 0) of the gate logits Gl [t][ldg],
+// Each head's read-out divided by its root mean square over vdim, times the weight (shared by the
+// heads, or wstride = vdim: one per head), times the output gate: silu (sig == 0) or sigmoid (sig != 0) of the gate logits Gl [t][ldg],
 // head h's at column gcol + h V (out may alias Gl when both rows have the same layout: every
-// entry is read before the same entry is written). One workgroup per token, a wave per head.
+// entry is read before the same entry is written). divided: O rows hold vdim + 1 entries per head, the
+// last one a divisor of the others. One workgroup per token, a wave per head.
 __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_out_kernel(const float *__restrict__ O, int H, int V,
                                                                     const float *__restrict__ w, float eps,
                                                                     const float *Gl, int ldg, int gcol,
-                                                                    float *out, int sig = 0) {
+                                                                    float *out, int sig = 0, int wstride = 0,
+                                                                    int divided = 0) {
 	const int t = blockIdx.x;
 	const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
 	for (int h = wave; h < H; h += SEQ_THREADS / 64) {
-		const float *o = O + (size_t)t * H * V + (size_t)h * V;
+		const int VS = V + (divided ? 1 : 0);
+		const float *o = O + ((size_t)t * H + h) * VS;
+		const float dv = divided ? 1.0f / o[V] : 1.0f;
 		float ss = 0.0f;
 		for (int i = lane; i < V; i += 64)
-			ss = fmaf(o[i], o[i], ss);
+			ss = fmaf(o[i] * dv, o[i] * dv, ss);
 		ss = wave_sum(ss);
-		const float r = 1.0f / sqrtf(ss / (float)V + eps);
+		const float r = dv / sqrtf(ss / (float)V + eps);
 		for (int i = lane; i < V; i += 64) {
 			const float gl = Gl[(size_t)t * ldg + gcol + h * V + i];
-			out[(size_t)t * H * V + (size_t)h * V + i] = o[i] * r * w[i] * (sig ? sq_sigmoid(gl) : sq_silu(gl));
+			out[(size_t)t * H * V + (size_t)h * V + i] = o[i] * r * w[h * wstride + i] * (sig ? sq_sigmoid(gl) : sq_silu(gl));
 		}
 	}
 }
@@ -2052,7 +2245,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_latent_attn_mfma_kernel(const
 // renormalised. kind 1: the `top` largest logits win (ties: the lower index), weights =
 // softmax over the chosen logits only. kind 2: scores sigmoid(logit); the choice ranks score +
 // bias: a group by the sum of its two largest, the `top` largest within the `keep` best groups
-// win (ties: the lower index); weight = score * rscale, without the bias, not renormalised.
+// win (ties: the lower index); weight = score * rscale, without the bias, not renormalised. kind 3:
+// scores = softmax over all E; the `top` largest score + bias win (ties: the lower index, no groups);
+// weight = score / (sum of the chosen scores + 1e-20) * rscale.
 // Also the shared expert's gate sigmoid(w_sg . h). Dynamic LDS: 2 E + G floats.
 #define SEQ_MAX_GROUPS 64
 __global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__restrict__ Hn, int width,
@@ -2086,7 +2281,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__
 		a = wave_sum(a);
 		if (lane == 0) {
 			if (e < E)
-				sc[e] = a + ((bias && kind != 2) ? bias[e] : 0.0f);
+				sc[e] = a + ((bias && kind < 2) ? bias[e] : 0.0f);
 			else
 				sgate[t] = sq_sigmoid(a);
 		}
@@ -2118,6 +2313,57 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__
 	}
 	float *gsc = sc + E; // [G]
 	__shared__ float red[SEQ_THREADS / 64];
+	if (kind == 3) { // one wave: a lane owns experts lane, lane + 64, ... and only touches their entries
+		if (wave != 0)
+			return;
+		float *sv = gsc + G; // [E] the scores (the weights); sc becomes the choice scores
+		float mx = -FLT_MAX, sum = 0.0f;
+		for (int e = lane; e < E; e += 64)
+			mx = fmaxf(mx, sc[e]);
+		mx = wave_max(mx);
+		for (int e = lane; e < E; e += 64) {
+			sv[e] = expf(sc[e] - mx);
+			sum += sv[e];
+		}
+		const float inv = 1.0f / wave_sum(sum);
+		for (int e = lane; e < E; e += 64) {
+			sv[e] *= inv;
+			sc[e] = sv[e] + (bias ? bias[e] : 0.0f);
+		}
+		float chosen = 0.0f; // sum of the chosen scores
+		for (int k = 0; k < top; ++k) {
+			float bv = -INFINITY;
+			int best = E; // above every index; a taken expert (-inf) never wins while another is left
+			for (int e = lane; e < E; e += 64)
+				if (sc[e] > bv) {
+					bv = sc[e];
+					best = e;
+				}
+#pragma unroll
+			for (int d = 32; d > 0; d >>= 1) {
+				const float ov = __shfl_xor(bv, d);
+				const int oe = __shfl_xor(best, d);
+				if (ov > bv || (ov == bv && oe < best)) {
+					bv = ov;
+					best = oe;
+				}
+			}
+			best = min(best, E - 1);
+			const bool mine = (best & 63) == lane;
+			const float score = __shfl(mine ? sv[best] : 0.0f, best & 63);
+			chosen += score;
+			if (mine) {
+				sc[best] = -INFINITY;
+				idx[(size_t)t * top + k] = best;
+				wt[(size_t)t * top + k] = score;
+			}
+		}
+		const float f = rscale / (chosen + 1e-20f);
+		__threadfence_block(); // the weights written by other lanes of this wave
+		for (int k = lane; k < top; k += 64)
+			wt[(size_t)t * top + k] *= f;
+		return;
+	}
 	if (kind == 2) { // sc holds the logits (no bias added above)
 		if (threadIdx.x != 0)
 			return;
@@ -2217,14 +2463,17 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__
 }
 
 // Slot s = t * top + k goes onto its expert's list (any order: every slot's rows are
-// computed independently of their neighbours in the list).
+// computed independently of their neighbours in the list); choices past the n_exp experts
+// (identity outputs) go nowhere.
 __global__ __launch_bounds__(SEQ_THREADS) void seq_moe_lists_kernel(const int *__restrict__ idx, int n_slots,
                                                                     int *__restrict__ counts, int *__restrict__ lists,
-                                                                    int cap) {
+                                                                    int cap, int n_exp) {
 	const int s = blockIdx.x * SEQ_THREADS + threadIdx.x;
 	if (s >= n_slots)
 		return;
 	const int e = idx[s];
+	if (e >= n_exp)
+		return;
 	const int p = atomicAdd(&counts[e], 1);
 	lists[(size_t)e * cap + p] = s;
 }

@@ -8,9 +8,11 @@ a packer that turns its checkpoint tensors into the engine's per-layer tensors
 experts). ``Sinulorn`` (latent attention, recurrences, routed experts), ``Lenuzen``
 (windowed / chunked softmax attention, plain feed-forwards), ``Mirorax`` (parallel
 blocks with layer scales, a looped run of layers, gated attention, latent attention with a
-rotated key part, a window and a learned sink) and ``Lifenex`` (parallel blocks with a norm
+rotated key part, a window and a learned sink), ``Lifenex`` (parallel blocks with a norm
 per sublayer, a selective state-space mixer, attention with a distance bias beside a delta
-rule with per-channel decays, grouped sigmoid routing) are such designs.
+rule with per-channel decays, grouped sigmoid routing) and ``Faguzen`` (norms without
+statistics, score-capped attention beside a matrix memory, ungated experts with identity
+outputs, a looped run) are such designs.
 
 Checkpoints are folders with ``config.json`` and ``model.safetensors`` (bf16
 matrices; read with yalmfile.read_yalm, the same container the .yalm files use).
@@ -26,14 +28,16 @@ import numpy as np
 
 from . import models as M
 
-MIX_LATENT, MIX_RGLRU, MIX_DELTA, MIX_ATTN, MIX_SSM = 0, 1, 2, 3, 4
+MIX_LATENT, MIX_RGLRU, MIX_DELTA, MIX_ATTN, MIX_SSM, MIX_MEMORY = 0, 1, 2, 3, 4, 5
 FF_NONE, FF_DENSE, FF_MOE, FF_PLAIN = 0, 1, 2, 3
-NORM_RMS, NORM_LAYER = 0, 1
+NORM_RMS, NORM_LAYER, NORM_TANH = 0, 1, 2
 MASK_CAUSAL, MASK_WINDOW, MASK_CHUNK = 0, 1, 2
 QK_NONE, QK_HEAD_UNIT, QK_WHOLE, QK_HEAD_W = 0, 1, 2, 3
 BLOCK_SERIAL, BLOCK_PARALLEL = 0, 1
-ACT_DEFAULT, ACT_GELU, ACT_CLAMP, ACT_SILU, ACT_RELU2 = 0, 1, 2, 3, 4
-ROUTER_SOFTMAX_TOP, ROUTER_TOP_SOFTMAX, ROUTER_SIGMOID_GROUPS = 0, 1, 2
+ACT_DEFAULT, ACT_GELU, ACT_CLAMP, ACT_SILU, ACT_RELU2, ACT_GELU_ERF = 0, 1, 2, 3, 4, 5
+ROUTER_SOFTMAX_TOP, ROUTER_TOP_SOFTMAX, ROUTER_SIGMOID_GROUPS, ROUTER_SOFTMAX_NORMED = 0, 1, 2, 3
+ROT_INTERLEAVED, ROT_HALVES = 0, 1
+RAMP_INDEX, RAMP_TURNS = 0, 1
 DELTA_GATE_SILU, DELTA_GATE_SIGMOID = 0, 1
 GATE_NONE, GATE_HEAD, GATE_ELEMENT = 0, 1, 2
 
@@ -104,10 +108,23 @@ class LayerSpec:
     q_temp_every: int = 0
     rel_rows: int = 0
     rel_max: float = 0.0
+    # rotated pairs (2i, 2i + 1) or (i, i + rot_dims / 2); frequency rescaling by pair index or by turns
+    rot_pairs: int = ROT_INTERLEAVED
+    rot_ramp: int = RAMP_INDEX
+    softcap: float = 0.0        # scores s -> softcap tanh(s / softcap)
+    # matrix memory: cap of the log gates' logits
+    gate_cap: float = 0.0
+    # routed experts: identity outputs after the experts; experts without gate matrices (ff_act of one matrix)
+    identity: int = 0
+    ungated: bool = False
     # a second mixer beside this one (a LayerSpec whose mixer fields alone are used); the two
-    # results are rms-normed with join_w / side_join_w, summed and scaled by join_scale
+    # results are rms-normed with join_w / side_join_w, summed and scaled by join_scale, or
+    # (join_normed False) join_scale a + side_join_scale b
     side: "LayerSpec" = None
     join_scale: float = 1.0
+    join_normed: bool = True
+    side_join_scale: float = 1.0
+    side_shares_in: bool = False  # the second mixer's input projection follows this one's in w_in (and in_bias)
     # parallel blocks: the feed-forward reads its own norm (norm2) of the stream; no layer scales
     ff_normed: bool = False
     layer_scaled: bool = True
@@ -126,6 +143,8 @@ class LayerSpec:
             return self.heads * self.dim + self.kv_heads * (self.dim + self.vdim) + gate
         if self.mixer == MIX_SSM:
             return 2 * self.heads * self.vdim + 2 * self.ssm_groups * self.ssm_state + self.heads
+        if self.mixer == MIX_MEMORY:
+            return 2 * self.heads * (self.dim + self.vdim + 1)
         return (2 * self.kv_heads * self.dim + self.heads * self.vdim + (self.gate_rank or self.heads * self.vdim)
                 + self.heads + (self.decay_rank or self.heads))
 
@@ -152,15 +171,23 @@ class LayeredConfig:
     tied_head: bool = False   # the logits read the embedding table
     block_kind: int = BLOCK_SERIAL  # BLOCK_PARALLEL: x += ls1 * mixer(norm1(x)) + ls2 * ff(norm1(x))
     embed_normed: bool = False  # the embedding row is rms-normed (weight embed_norm) before it becomes the stream
+    residual_scale: float = 1.0  # every sublayer's result times this as it joins the stream
+    logit_softcap: float = 0.0   # logits z -> logit_softcap tanh(z / logit_softcap)
 
     def with_(self, **kw) -> "LayeredConfig":
         return dataclasses.replace(self, **kw)
 
 
-def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False) -> dict:
+def norm_shape(c: LayeredConfig) -> tuple:
+    """Shape of a norm's vector: the weight, or (tanh norms) weight | bias | alpha."""
+    return (2 * c.width + 1,) if c.norm_kind == NORM_TANH else (c.width,)
+
+
+def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False, shared_in: bool = False) -> dict:
     """field -> (shape, kind) of one layer's engine tensors; kind "w": a matrix of the
-    model's weight dtype, "f": f32. side: l is a layer's second mixer (its mixer tensors only)."""
-    W = c.width
+    model's weight dtype, "f": f32. side: l is a layer's second mixer (its mixer tensors only;
+    shared_in: its input projection is part of the first mixer's)."""
+    W, N = c.width, norm_shape(c)
     out = {}
     if l.pre_added:
         out["pre_add"] = ((W,), "f")
@@ -169,25 +196,27 @@ def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False) -> dict:
     if side:
         pass
     elif c.block_kind == BLOCK_PARALLEL:
-        out["norm1"] = ((W,), "f")
+        out["norm1"] = (N, "f")
         if l.layer_scaled:
             out["ls1"] = ((W,), "f")
         if l.ff_kind != FF_NONE:
             if l.layer_scaled:
                 out["ls2"] = ((W,), "f")
             if l.ff_normed:
-                out["norm2"] = ((W,), "f")
+                out["norm2"] = (N, "f")
     else:
-        out["norm1b"] = ((W,), "f")
+        out["norm1b"] = (N, "f")
         if c.pre_norm:
-            out["norm1"] = ((W,), "f")
+            out["norm1"] = (N, "f")
         if l.ff_kind != FF_NONE:
-            out["norm2b"] = ((W,), "f")
+            out["norm2b"] = (N, "f")
             if c.pre_norm:
-                out["norm2"] = ((W,), "f")
-    if l.side is not None:
+                out["norm2"] = (N, "f")
+    if l.side is not None and l.join_normed:
         out["join_w"] = out["side_join_w"] = ((W,), "f")
-    out["w_in"] = ((l.in_rows, W), "w")
+    in_rows = l.in_rows + (l.side.in_rows if l.side_shares_in else 0)
+    if not shared_in:
+        out["w_in"] = ((in_rows, W), "w")
     out["w_o"] = ((W, l.mix_out), "w")
     if l.o_biased:
         out["o_bias"] = ((W,), "f")
@@ -213,7 +242,7 @@ def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False) -> dict:
         )
     elif l.mixer == MIX_ATTN:
         if l.in_biased:
-            out["in_bias"] = ((l.in_rows,), "f")
+            out["in_bias"] = ((in_rows,), "f")
         if l.qk_norm == QK_WHOLE:
             out.update(q_norm=((l.heads * l.dim,), "f"), kv_norm=((l.kv_heads * l.dim,), "f"))
         if l.head_temps:
@@ -224,6 +253,10 @@ def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False) -> dict:
             out.update(q_norm=((l.dim,), "f"), kv_norm=((l.dim,), "f"))
         if l.rel_rows:
             out["rel"] = ((l.rel_rows, l.heads), "f")
+    elif l.mixer == MIX_MEMORY:
+        if l.in_biased:
+            out["in_bias"] = ((in_rows,), "f")
+        out["out_norm"] = ((l.heads * l.vdim,), "f")
     elif l.mixer == MIX_SSM:
         inner, cc = l.heads * l.vdim, l.heads * l.vdim + 2 * l.ssm_groups * l.ssm_state
         out.update(conv_w=((cc, l.conv), "f"), conv_b=((cc,), "f"), a_log=((l.heads,), "f"), dt_bias=((l.heads,), "f"),
@@ -241,13 +274,16 @@ def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False) -> dict:
     if l.ff_kind == FF_DENSE:
         out.update(w_gate=((l.ff, W), "w"), w_up=((l.ff, W), "w"), w_down=((W, l.ff), "w"))
     elif l.ff_kind == FF_MOE:
-        out.update(router=((l.experts, W), "f"), w_gate=((l.experts, l.ff, W), "w"),
-                   w_up=((l.experts, l.ff, W), "w"), w_down=((l.experts, W, l.ff), "w"))
+        out.update(router=((l.experts + l.identity, W), "f"), w_up=((l.experts, l.ff, W), "w"),
+                   w_down=((l.experts, W, l.ff), "w"))
+        if not l.ungated:
+            out["w_gate"] = ((l.experts, l.ff, W), "w")
         if l.router_biased:
-            out["router_bias"] = ((l.experts,), "f")
+            out["router_bias"] = ((l.experts + l.identity,), "f")
         if l.shared_ff:
-            out.update(ws_gate=((l.shared_ff, W), "w"), ws_up=((l.shared_ff, W), "w"),
-                       ws_down=((W, l.shared_ff), "w"))
+            out.update(ws_up=((l.shared_ff, W), "w"), ws_down=((W, l.shared_ff), "w"))
+            if not l.ungated:
+                out["ws_gate"] = ((l.shared_ff, W), "w")
             if l.shared_gated:
                 out["shared_sg"] = ((W,), "f")
     return out
@@ -626,6 +662,19 @@ def unroll_loop(layers: list, loop) -> list:
     return runs + [(i, None) for i in range(b, n)]
 
 
+def _unrolled(cfg: dict, make) -> list:
+    """The layer runs of a config.json with a loop: make(layer entry) -> LayerSpec for each, a
+    repeated run naming the run of its first pass, the first run of a pass taking a vector."""
+    first, runs = {}, []
+    for i, step in unroll_loop(cfg["layers"], cfg.get("loop")):
+        s = make(cfg["layers"][i])
+        s.pre_added = step is not None
+        s.shares = first.get(i, -1)
+        first.setdefault(i, len(runs))
+        runs.append(s)
+    return runs
+
+
 def _mirorax_layer(e: dict) -> LayerSpec:
     m = e["mixer"]
     if e["type"] == "attention":
@@ -660,16 +709,8 @@ def mirorax_config(cfg: dict, max_tokens: int = 4096, weight_dtype: int = M.BF16
     """config.json of a Mirorax checkpoint -> LayeredConfig whose layers are the layer RUNS (the
     looped run unrolled; a repeated run shares the tensors of its first pass). Every size and
     every constant that can differ between models of the design is read from cfg."""
-    first = {}
-    runs = []
-    for i, step in unroll_loop(cfg["layers"], cfg.get("loop")):
-        s = _mirorax_layer(cfg["layers"][i])
-        s.pre_added = step is not None
-        s.shares = first.get(i, -1)
-        first.setdefault(i, len(runs))
-        runs.append(s)
     return LayeredConfig(
-        arch="Mirorax", width=cfg["width"], vocab=cfg["vocab"], layers=runs, embed_scale=1.0,
+        arch="Mirorax", width=cfg["width"], vocab=cfg["vocab"], layers=_unrolled(cfg, _mirorax_layer), embed_scale=1.0,
         norm_eps=float(cfg["norm"]["eps"]), max_tokens=max_tokens, weight_dtype=weight_dtype, norm_kind=NORM_RMS,
         pre_norm=True, pos_embed=False, block_kind=BLOCK_PARALLEL,
     )
@@ -1018,11 +1059,190 @@ def lifenex_random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, **sizes)
     return out
 
 
+# ------------------------------------------------------------------ Faguzen
+# x = E[token]. Every layer is a parallel block with two tanh norms of the same stream, both results
+# scaled by one constant: x += m (mix(n1(x)) + ff(n2(x))), n(x) = tanh(alpha x) w + b. A run of layers
+# [start, stop) is walked `times` times with the same weights, pass t first adding row t of loop.step
+# to the stream; every pass has caches and states of its own. One mixer kind:
+#   "parallel": a left + c right on the same input: left, causal softmax attention with grouped
+#               key/value heads, biased q / k / v / o, the first dims entries of queries and keys
+#               rotated in half-split pairs (frequencies rescaled by turns), scores capped by a tanh,
+#               the concatenated heads times sigmoid(W_g h); right, a matrix memory with exponential
+#               gates (log gates capped by a tanh), read through its normaliser, rms-normed per head,
+#               times sigmoid(W_g h).
+# Feed-forward "moe": experts W_down gelu(W_up h) (exact gelu), softmax scores over experts and
+# identity outputs, the choice by score + correction, weights the chosen scores over their sum; plus a
+# shared expert. Logits: cap tanh(head n(x) / cap).
+def _faguzen_layer(e: dict) -> LayerSpec:
+    m = e["mixer"]
+    if e["type"] != "parallel":
+        raise ValueError(f"unknown mixer type {e['type']!r}")
+    a, d = m["left"], m["right"]
+    rot = a.get("rot") or {"dims": 0, "base": 1.0}
+    sc = rot.get("scaling") or {}
+    s = LayerSpec(MIX_ATTN, heads=a["heads"], kv_heads=a.get("kv_heads", a["heads"]), dim=a["dim"], vdim=a["vdim"],
+                  attn_scale=float(a["scale"]), mask_kind=MASK_CAUSAL, softcap=float(a.get("softcap") or 0.0),
+                  out_gate=GATE_ELEMENT, in_biased=True, o_biased=True, rot_dims=int(rot["dims"]),
+                  rot_base=float(rot["base"]), rot_pairs=ROT_HALVES, rot_ramp=RAMP_TURNS,
+                  rot_factor=float(sc.get("factor", 0.0)), rot_orig=int(sc.get("original", 0)),
+                  rot_fast=float(sc.get("high", 0.0)), rot_slow=float(sc.get("low", 0.0)),
+                  join_normed=False, join_scale=float(m["left_scale"]), side_join_scale=float(m["right_scale"]),
+                  side_shares_in=True, ff_normed=True, layer_scaled=False)
+    s.side = LayerSpec(MIX_MEMORY, heads=d["heads"], dim=d["dim"], vdim=d["vdim"], gate_cap=float(d["gate_cap"]))
+    mlp = e.get("mlp")
+    if mlp:
+        if mlp["kind"] != "moe":
+            raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+        r = mlp["router"]
+        s.ff_kind, s.ff, s.ff_act, s.ungated = FF_MOE, mlp["expert"]["ff"], ACT_GELU_ERF, True
+        s.experts, s.top, s.identity = r["experts"], r["top"], int(r.get("identity") or 0)
+        s.router_kind, s.router_biased = ROUTER_SOFTMAX_NORMED, True
+        if mlp.get("shared"):
+            s.shared_ff, s.shared_gated = mlp["shared"]["ff"], False
+    return s
+
+
+def faguzen_config(cfg: dict, max_tokens: int = 4096, weight_dtype: int = M.BF16) -> LayeredConfig:
+    """config.json of a Faguzen checkpoint -> LayeredConfig whose layers are the layer RUNS (the
+    looped run unrolled; a repeated run shares the tensors of its first pass). Every size and every
+    constant that can differ between models of the design is read from cfg."""
+    return LayeredConfig(
+        arch="Faguzen", width=cfg["width"], vocab=cfg["vocab"], layers=_unrolled(cfg, _faguzen_layer), embed_scale=1.0,
+        norm_eps=float(cfg["norm"]["eps"]), max_tokens=max_tokens, weight_dtype=weight_dtype, norm_kind=NORM_TANH,
+        pre_norm=True, pos_embed=False, block_kind=BLOCK_PARALLEL, residual_scale=float(cfg["residual_mult"]),
+        logit_softcap=float(cfg.get("logit_softcap") or 0.0),
+    )
+
+
+def faguzen_tensor_shapes(cfg: dict) -> dict:
+    """Checkpoint tensor name -> shape for a Faguzen config.json."""
+    W = cfg["width"]
+    out = {"embed": (cfg["vocab"], W), "head": (cfg["vocab"], W)}
+    if cfg.get("loop"):
+        out["loop.step"] = (cfg["loop"]["times"], W)
+
+    def norm(name):
+        out[name] = out[name + ".b"] = (W,)
+        out[name + ".alpha"] = ()
+
+    norm("final.norm")
+    for i, e in enumerate(cfg["layers"]):
+        p = f"l{i}."
+        a, d = e["mixer"]["left"], e["mixer"]["right"]
+        norm(p + "norm1")
+        H, G, D, V = a["heads"], a.get("kv_heads", a["heads"]), a["dim"], a["vdim"]
+        x = p + "mix.left."
+        for n, rows in (("q", H * D), ("k", G * D), ("v", G * V)):
+            out[x + n], out[x + n + ".b"] = (rows, W), (rows,)
+        out[x + "g"], out[x + "o"], out[x + "o.b"] = (H * V, W), (W, H * V), (W,)
+        H, D, V = d["heads"], d["dim"], d["vdim"]
+        x = p + "mix.right."
+        for n, rows in (("q", H * D), ("k", H * D), ("v", H * V), ("g", H * V), ("i", H), ("f", H)):
+            out[x + n] = (rows, W)
+        out[x + "i.b"] = out[x + "f.b"] = (H,)
+        out[x + "norm"], out[x + "o"] = (H * V,), (W, H * V)
+        mlp = e.get("mlp")
+        if not mlp:
+            continue
+        norm(p + "norm2")
+        f, ff, E = p + "mlp.", mlp["expert"]["ff"], mlp["router"]["experts"]
+        for k in range(E):
+            out[f"{f}e{k}.up"], out[f"{f}e{k}.down"] = (ff, W), (W, ff)
+        ER = E + int(mlp["router"].get("identity") or 0)
+        out[f + "router"], out[f + "correction"] = (ER, W), (ER,)
+        if mlp.get("shared"):
+            sf = mlp["shared"]["ff"]
+            out[f + "shared.up"], out[f + "shared.down"] = (sf, W), (W, sf)
+    return out
+
+
+def faguzen_pack(c: LayeredConfig, t: dict, cfg: dict) -> dict:
+    """Checkpoint tensors -> the engine's tensors (see sinulorn_pack), one dict per layer run; a
+    repeated run holds the very arrays of its first pass (uploaded once) and its own pre_add. Both
+    mixers' input projections are one w_in (attention q | k | v | gate, memory q | k | v | gate | i | f)
+    with one bias vector (zeros where the design has none); a norm is weight | bias | alpha."""
+    dt = c.weight_dtype
+
+    def w(*names):
+        parts = [_as_weight(t[n], dt) for n in names]
+        return parts[0] if len(parts) == 1 else np.ascontiguousarray(np.concatenate(parts, axis=0))
+
+    def f(name):
+        return np.ascontiguousarray(_as_f32(t[name]))
+
+    def norm(name):
+        return np.concatenate([f(name), f(name + ".b"), f(name + ".alpha").reshape(1)])
+
+    runs = []
+    for r, (l, (i, step)) in enumerate(zip(c.layers, unroll_loop(cfg["layers"], cfg.get("loop")))):
+        own = {}
+        if step is not None:
+            own["pre_add"] = np.ascontiguousarray(f("loop.step")[step])
+        if l.shares >= 0:
+            d = {k: v for k, v in runs[l.shares].items() if k != "pre_add"}
+            d.update(own)
+            runs.append(d)
+            continue
+        p, m = f"l{i}.", f"l{i}.mlp."
+        y, z = p + "mix.left.", p + "mix.right."
+        none = np.zeros
+        d = dict(own, norm1=norm(p + "norm1"),
+                 w_in=w(*[y + n for n in ("q", "k", "v", "g")], *[z + n for n in ("q", "k", "v", "g", "i", "f")]),
+                 in_bias=np.concatenate([f(y + "q.b"), f(y + "k.b"), f(y + "v.b"), none(l.heads * l.vdim, np.float32),
+                                         none(l.side.in_rows - 2 * l.side.heads, np.float32), f(z + "i.b"), f(z + "f.b")]),
+                 w_o=w(y + "o"), o_bias=f(y + "o.b"))
+        sd = {"out_norm": f(z + "norm"), "w_o": w(z + "o")}
+        if l.ff_kind != FF_NONE:
+            d.update(norm2=norm(p + "norm2"), router=f(m + "router"), router_bias=f(m + "correction"))
+            for k in ("up", "down"):
+                d["w_" + k] = np.ascontiguousarray(
+                    np.stack([_as_weight(t[f"{m}e{e}.{k}"], dt) for e in range(l.experts)]))
+            if l.shared_ff:
+                d.update(ws_up=w(m + "shared.up"), ws_down=w(m + "shared.down"))
+        _check_packed(f"layer {i}", packed_shapes(c, l), d)
+        _check_packed(f"layer {i}, second mixer", packed_shapes(c, l.side, side=True, shared_in=True), sd)
+        d["side"] = sd
+        runs.append(d)
+    return {"embed": w("embed"), "final_norm": norm("final.norm"), "head": w("head"), "layers": runs}
+
+
+def faguzen_random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0) -> dict:
+    """Random checkpoint tensors for a Faguzen config.json, as float32 arrays already rounded to
+    bf16 values (the f32 and bf16 engines and a float64 restatement see the same weights)."""
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in faguzen_tensor_shapes(cfg).items():
+        leaf = name.split(".")[-1]
+        if leaf in ("norm1", "norm2", "norm"):
+            a = 1.0 + 0.2 * rng.standard_normal(shape)
+        elif leaf == "alpha":
+            a = rng.uniform(0.4, 1.2, shape)
+        elif name.endswith(".f.b"):  # forget gates between nearly closed and nearly open
+            a = rng.uniform(-1.0, 5.0, shape)
+        elif leaf == "b":
+            a = 0.3 * rng.standard_normal(shape)
+        elif leaf == "correction":
+            a = 0.1 * rng.standard_normal(shape)
+        elif leaf == "step":
+            a = 0.3 * rng.standard_normal(shape)
+        elif leaf == "embed":
+            a = 0.7 * rng.standard_normal(shape)
+        else:
+            a = gain * rng.standard_normal(shape) / np.sqrt(shape[-1])
+        out[name] = bf16_to_f32(f32_to_bf16(np.asarray(a, np.float32))).reshape(shape)
+    return out
+
+
 # ------------------------------------------------------------------ registry
-# design name (config.json "architecture") -> (config reader, weight packer)
-DESIGNS = {"Sinulorn": (sinulorn_config, sinulorn_pack), "Lenuzen": (lenuzen_config, lenuzen_pack),
-           "Mirorax": (mirorax_config, lambda c, t, cfg=None: mirorax_pack(c, t, cfg)),
-           "Lifenex": (lifenex_config, lifenex_pack)}
+# design name (config.json "architecture") -> (config reader, weight packer). A reader takes (cfg,
+# max_tokens, weight_dtype, shapes of the checkpoint's tensors), a packer (LayeredConfig, tensors, cfg).
+DESIGNS = {
+    "Sinulorn": (lambda cfg, n, dt, shapes: sinulorn_config(cfg, n, dt), lambda c, t, cfg: sinulorn_pack(c, t)),
+    "Lenuzen": (lambda cfg, n, dt, shapes: lenuzen_config(cfg, n, dt), lambda c, t, cfg: lenuzen_pack(c, t)),
+    "Mirorax": (lambda cfg, n, dt, shapes: mirorax_config(cfg, n, dt), mirorax_pack),
+    "Lifenex": (lifenex_config, lambda c, t, cfg: lifenex_pack(c, t)),
+    "Faguzen": (lambda cfg, n, dt, shapes: faguzen_config(cfg, n, dt), faguzen_pack),
+}
 
 
 def read_checkpoint(path: str, max_tokens: int = 4096, weight_dtype: int = M.BF16):
@@ -1038,11 +1258,8 @@ def read_checkpoint(path: str, max_tokens: int = 4096, weight_dtype: int = M.BF1
     reader, packer = DESIGNS[arch]
     yd = read_yalm(os.path.join(path, "model.safetensors"))
     try:
-        if arch == "Lifenex":  # some sizes are the tensors' own
-            c = reader(cfg, max_tokens, weight_dtype, {k: tuple(v.shape) for k, v in yd.tensors.items()})
-        else:
-            c = reader(cfg, max_tokens, weight_dtype)
+        c = reader(cfg, max_tokens, weight_dtype, {k: tuple(v.shape) for k, v in yd.tensors.items()})
         t = {k: np.asarray(v.data).reshape(v.shape) for k, v in yd.tensors.items()}
-        return c, (packer(c, t, cfg) if arch == "Mirorax" else packer(c, t))
+        return c, packer(c, t, cfg)
     finally:
         yd.close()

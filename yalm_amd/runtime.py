@@ -158,7 +158,8 @@ class SeqLayer(ctypes.Structure):
         + [(n, c_float) for n in ("rot_base", "rot_factor", "rot_fast", "rot_slow")]
         + [(n, c_int) for n in ("ssm_state", "ssm_groups", "norm_groups", "decay_rank", "gate_rank", "gate_act")]
         + [("q_temp_coef", c_float), ("q_temp_every", c_int), ("rel_rows", c_int), ("rel_max", c_float),
-           ("join_scale", c_float)]
+           ("join_scale", c_float), ("side_join_scale", c_float), ("rot_pairs", c_int), ("rot_ramp", c_int),
+           ("softcap", c_float), ("gate_cap", c_float), ("identity", c_int)]
         + [(n, c_void_p) for n in PTRS]
     )
 
@@ -166,7 +167,8 @@ class SeqLayer(ctypes.Structure):
 class SeqConfig(ctypes.Structure):
     _fields_ = [("width", c_int), ("vocab", c_int), ("n_layers", c_int), ("max_tokens", c_int),
                 ("embed_scale", c_float), ("norm_eps", c_float), ("weight_dtype", c_int), ("norm_kind", c_int),
-                ("pre_norm", c_int), ("pos_embed", c_int), ("logit_scale", c_float), ("block_kind", c_int)]
+                ("pre_norm", c_int), ("pos_embed", c_int), ("logit_scale", c_float), ("block_kind", c_int),
+                ("residual_scale", c_float), ("logit_softcap", c_float)]
 
 
 class SeqWeights(ctypes.Structure):
@@ -727,15 +729,15 @@ class SeqModel:
             return p
 
         self.ptrs["embed"] = make("embed", (cfg.vocab, cfg.width), "w", fan_in=100.0)
-        self.ptrs["final_norm"] = make("final_norm", (cfg.width,), "f")
+        self.ptrs["final_norm"] = make("final_norm", layered.norm_shape(cfg), "f")
         self.ptrs["head"] = self.ptrs["embed"] if cfg.tied_head else make("head", (cfg.vocab, cfg.width), "w")
         if cfg.embed_normed:
             self.ptrs["embed_norm"] = make("embed_norm", (cfg.width,), "f")
         for i, l in enumerate(cfg.layers):
             ptrs = {k: make(f"l{i}.{k}", shape, kind) for k, (shape, kind) in layered.packed_shapes(cfg, l).items()}
-            if l.side is not None:
+            if l.side is not None and l.shares < 0:
                 ptrs["side"] = {k: make(f"l{i}.side.{k}", shape, kind)
-                                for k, (shape, kind) in layered.packed_shapes(cfg, l.side, side=True).items()}
+                                for k, (shape, kind) in layered.packed_shapes(cfg, l.side, side=True, shared_in=l.side_shares_in).items()}
             if l.shares >= 0:  # a repeated run: the first pass's tensors, its own pre_add
                 ptrs = {**{k: v for k, v in self.layer_ptrs[l.shares].items() if k != "pre_add"}, **ptrs}
             self.layer_ptrs.append(ptrs)
@@ -767,7 +769,7 @@ class SeqModel:
         arr._sides = sides  # kept alive with the layer array
         sc = SeqConfig(cfg.width, cfg.vocab, len(cfg.layers), cfg.max_tokens, cfg.embed_scale, cfg.norm_eps,
                        cfg.weight_dtype, cfg.norm_kind, int(cfg.pre_norm), int(cfg.pos_embed), cfg.logit_scale,
-                       cfg.block_kind)
+                       cfg.block_kind, cfg.residual_scale, cfg.logit_softcap)
         sw = SeqWeights(self.ptrs["embed"], self.ptrs["final_norm"], self.ptrs["head"], arr, self.ptrs.get("embed_norm"))
         return sc, sw, arr
 
