@@ -79,7 +79,7 @@ def parse():
                          "(Sinulorn-shaped stacks, random bf16 weights) at a few real layer sizes, each beside a "
                          "Llama-shaped decoder of equal width, depth and feed-forward size; one JSON line")
     ap.add_argument("--layered-sizes", default="1024,2048,4096", help="model widths of the --layered legs")
-    ap.add_argument("--layered-design", default="sinulorn", choices=["sinulorn", "lenuzen", "mirorax", "lifenex"],
+    ap.add_argument("--layered-design", default="sinulorn", choices=["sinulorn", "lenuzen", "mirorax", "lifenex", "faguzen"],
                     help="which layer-list design the --layered stack is shaped like")
     return ap.parse_args()
 
@@ -610,6 +610,32 @@ def lifenex_stack(Ly, M, width, max_tokens):
                             logit_scale=0.25, tied_head=True, block_kind=Ly.BLOCK_PARALLEL, embed_normed=True)
 
 
+def faguzen_stack(Ly, M, width, max_tokens):
+    """A Faguzen-shaped stack at a real layer size, six layer runs, every one a pair (score-capped
+    attention beside a matrix memory) + routed experts: two layers walked twice with the same
+    weights, then two more. Attention heads of 128 with four query heads per key/value head, half of
+    a head rotated with rescaled frequencies, elementwise output gate; memory heads of 128 x 128, as many
+    as the Lifenex-shaped stack's delta rule has; ungated experts and shared expert of the Lifenex-
+    shaped stack's hidden sizes, four identity outputs, top 4."""
+    heads = width // 128
+    ff = width * 7 // 2
+    kw = dict(heads=heads, kv_heads=max(heads // 4, 1), dim=128, vdim=128, attn_scale=128 ** -0.5, mask_kind=Ly.MASK_CAUSAL,
+              softcap=50.0, out_gate=Ly.GATE_ELEMENT, in_biased=True, o_biased=True, rot_dims=64, rot_base=500000.0,
+              rot_pairs=Ly.ROT_HALVES, rot_ramp=Ly.RAMP_TURNS, rot_factor=8.0, rot_orig=8192, rot_fast=4.0, rot_slow=1.0,
+              join_normed=False, join_scale=0.8, side_join_scale=0.6, side_shares_in=True, ff_normed=True,
+              layer_scaled=False, ff_kind=Ly.FF_MOE, ff=ff // 8, ff_act=Ly.ACT_GELU_ERF, ungated=True, experts=16, top=4,
+              identity=4, shared_ff=ff // 2, shared_gated=False, router_kind=Ly.ROUTER_SOFTMAX_NORMED, router_biased=True)
+
+    def run(**loop):
+        side = Ly.LayerSpec(Ly.MIX_MEMORY, heads=max(heads // 2, 1), dim=128, vdim=128, gate_cap=15.0)
+        return Ly.LayerSpec(Ly.MIX_ATTN, side=side, **kw, **loop)
+
+    layers = [run(pre_added=True), run(), run(pre_added=True, shares=0), run(shares=1), run(), run()]
+    return Ly.LayeredConfig("Faguzen", width, 32000, layers, embed_scale=1.0, norm_eps=1e-6, max_tokens=max_tokens,
+                            weight_dtype=M.BF16, norm_kind=Ly.NORM_TANH, pre_norm=True, pos_embed=False,
+                            block_kind=Ly.BLOCK_PARALLEL, residual_scale=0.5, logit_softcap=30.0)
+
+
 def layered_bench(args, out_file):
     """--layered: tokens/s of a prompt portion (n = 2048 at position 0) and of single-token
     decoding (the device greedy loop at context ~1024) for the layer-list engine, and for a
@@ -623,8 +649,8 @@ def layered_bench(args, out_file):
     n_pf, ctx, steps = 2048, 1024, max(args.steps if args.steps != 256 else 64, 8)
     legs = []
     for width in [int(x) for x in args.layered_sizes.split(",")]:
-        make = {"lenuzen": lenuzen_stack, "mirorax": mirorax_stack, "lifenex": lifenex_stack}.get(args.layered_design,
-                                                                                                   layered_stack)
+        make = {"lenuzen": lenuzen_stack, "mirorax": mirorax_stack, "lifenex": lifenex_stack,
+                "faguzen": faguzen_stack}.get(args.layered_design, layered_stack)
 
         def timed(cfg):
             model = runtime.SeqModel.synthetic(cfg, seed=3)
@@ -645,11 +671,13 @@ def layered_bench(args, out_file):
         leg = {"width": width, "layers": len(cfg.layers), "prefill_tokens": n_pf, "prefill_ms": round(pf_ms, 3),
                "prefill_tok_s": round(n_pf / pf_ms * 1e3, 1), "decode_context": ctx, "decode_steps": steps,
                "decode_ms_per_token": round(dt / steps * 1e3, 4), "decode_tok_s": round(steps / dt, 2)}
-        if args.layered_design == "lifenex":
-            # the closest layer-list design (delta rule, a linear recurrence, grouped routed experts with a
-            # gated shared expert, attention) at the same width, depth and feed-forward size
-            npf, ndt = timed(layered_stack(Ly, M, width, n_pf + 64))
-            leg.update(near_design="Sinulorn", near_prefill_ms=round(npf, 3), near_prefill_tok_s=round(n_pf / npf * 1e3, 1),
+        # the closest layer-list design at the same width, depth and feed-forward size: Sinulorn for Lifenex
+        # (delta rule, a linear recurrence, grouped routed experts with a gated shared expert, attention),
+        # Lifenex for Faguzen (attention and a recurrence side by side, routed experts)
+        near = {"lifenex": ("Sinulorn", layered_stack), "faguzen": ("Lifenex", lifenex_stack)}.get(args.layered_design)
+        if near:
+            npf, ndt = timed(near[1](Ly, M, width, n_pf + 64))
+            leg.update(near_design=near[0], near_prefill_ms=round(npf, 3), near_prefill_tok_s=round(n_pf / npf * 1e3, 1),
                        near_decode_ms_per_token=round(ndt / steps * 1e3, 4), near_decode_tok_s=round(steps / ndt, 2))
         ref = M.ModelConfig(dim=width, hidden_dim=width * 7 // 2, head_dim=128, n_layers=len(cfg.layers),
                             n_heads=width // 128, n_kv_heads=max(width // 512, 1), vocab_size=32000,

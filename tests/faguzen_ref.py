@@ -129,19 +129,23 @@ def memory_gates(h, w, pre, cap):
     return i, f
 
 
-def memory_scan(q, k, v, i, f, start_max=0.0):
+def normaliser(nq, m):
+    return max(abs(nq), np.exp(-m)) + 1e-6
+
+
+def memory_scan(q, k, v, i, f):
     """q, k [T, H, D], v [T, H, V], i, f [T, H]: the read-outs [T, H, V]."""
     T, H, D = q.shape
     o = np.zeros((T, H, v.shape[2]), F)
     for h in range(H):
-        S, n, m = np.zeros((D, v.shape[2]), F), np.zeros(D, F), start_max
+        S, n, m = np.zeros((D, v.shape[2]), F), np.zeros(D, F), 0.0
         for t in range(T):
             new = max(f[t, h] + m, i[t, h])
             keep, put = np.exp(f[t, h] + m - new), np.exp(i[t, h] - new)
             m = new
             S = keep * S + put * np.outer(k[t, h], v[t, h])
             n = keep * n + put * k[t, h]
-            o[t, h] = S.T @ q[t, h] / (max(abs(n @ q[t, h]), np.exp(-m)) + 1e-6)
+            o[t, h] = S.T @ q[t, h] / normaliser(n @ q[t, h], m)
     return o
 
 

@@ -296,7 +296,8 @@ def test_bench_stacks_are_valid_layer_list_configurations():
     import bench
 
     for width in (1024, 2048, 4096):
-        for make in (bench.layered_stack, bench.lenuzen_stack, bench.mirorax_stack, bench.lifenex_stack):
+        for make in (bench.layered_stack, bench.lenuzen_stack, bench.mirorax_stack, bench.lifenex_stack,
+                     bench.faguzen_stack):
             c = make(Ly, M, width, 2112)
             assert c.width == width and len(c.layers) == 6
             for l in c.layers:
@@ -304,10 +305,12 @@ def test_bench_stacks_are_valid_layer_list_configurations():
                 if l.shares >= 0:  # a repeated run of a loop owns its pre_add only
                     assert set(shapes) <= {"pre_add"} and c.layers[l.shares].mixer == l.mixer
                     continue
-                assert shapes["w_in"][0] == (l.in_rows, width) and shapes["w_o"][0] == (width, l.mix_out)
+                joint = l.side.in_rows if l.side_shares_in else 0  # a pair's one projection
+                assert shapes["w_in"][0] == (l.in_rows + joint, width) and shapes["w_o"][0] == (width, l.mix_out)
                 if l.side is not None:
-                    side = Ly.packed_shapes(c, l.side, side=True)
-                    assert side["w_in"][0] == (l.side.in_rows, width) and "norm1" not in side and "join_w" in shapes
+                    side = Ly.packed_shapes(c, l.side, side=True, shared_in=bool(joint))
+                    assert ("w_in" not in side) if joint else side["w_in"][0] == (l.side.in_rows, width)
+                    assert "norm1" not in side and ("join_w" in shapes) == l.join_normed
                 if l.mixer == Ly.MIX_ATTN:
                     assert l.heads % l.kv_heads == 0 and l.rot_dims <= l.dim
                     if l.talking:
@@ -428,3 +431,154 @@ def test_lifenex_restatement_mechanisms():
     assert np.allclose(g, [[3 / np.sqrt(12.5), 4 / np.sqrt(12.5), 0.0, np.sqrt(2.0)]])
     y = LR.causal_conv(np.array([[1.0], [2.0], [3.0]]), np.array([[10.0, 1.0]]), np.array([0.5]))
     assert np.allclose(y[:, 0], [1.5, 12.5, 23.5])
+
+
+# ------------------------------------------------------------------ Faguzen
+def test_faguzen_config_reads_every_size_and_constant():
+    import faguzen_cases as FC
+
+    cfg = FC.MIXED
+    c = Ly.faguzen_config(cfg, max_tokens=77, weight_dtype=M.F32)
+    assert (c.arch, c.width, c.vocab, c.max_tokens, c.weight_dtype) == ("Faguzen", 96, 211, 77, M.F32)
+    assert (c.norm_kind, c.block_kind, c.pre_norm, c.pos_embed, c.tied_head, c.embed_normed) == (
+        Ly.NORM_TANH, Ly.BLOCK_PARALLEL, True, False, False, False)
+    assert (c.norm_eps, c.residual_scale, c.logit_softcap) == (1e-5, 0.8, 9.0)
+    # layers 1 and 2 run three times: a repeated run names its first pass, a pass opens with a vector
+    assert [l.shares for l in c.layers] == [-1, -1, -1, 1, 2, 1, 2, -1]
+    assert [l.pre_added for l in c.layers] == [False, True, False, True, False, True, False, False]
+    s, e = c.layers[0], cfg["layers"][0]
+    a, d, r = e["mixer"]["left"], e["mixer"]["right"], e["mlp"]["router"]
+    assert (s.mixer, s.heads, s.kv_heads, s.dim, s.vdim, s.attn_scale, s.softcap) == (
+        Ly.MIX_ATTN, a["heads"], a["kv_heads"], a["dim"], a["vdim"], a["scale"], a["softcap"])
+    assert (s.rot_dims, s.rot_base, s.rot_factor, s.rot_slow, s.rot_fast, s.rot_orig) == (8, 500.0, 4.0, 1.0, 3.0, 40)
+    assert (s.rot_pairs, s.rot_ramp, s.mask_kind, s.out_gate, s.in_biased, s.o_biased) == (
+        Ly.ROT_HALVES, Ly.RAMP_TURNS, Ly.MASK_CAUSAL, Ly.GATE_ELEMENT, True, True)
+    assert (s.join_normed, s.join_scale, s.side_join_scale, s.side_shares_in) == (False, 0.9, 0.7, True)
+    assert (s.side.mixer, s.side.heads, s.side.dim, s.side.vdim, s.side.gate_cap) == (
+        Ly.MIX_MEMORY, d["heads"], d["dim"], d["vdim"], d["gate_cap"])
+    assert (s.ff_kind, s.ff, s.ff_act, s.ungated, s.experts, s.top, s.identity) == (
+        Ly.FF_MOE, 40, Ly.ACT_GELU_ERF, True, r["experts"], r["top"], r["identity"])
+    assert (s.router_kind, s.router_biased, s.shared_ff, s.shared_gated) == (Ly.ROUTER_SOFTMAX_NORMED, True, 24, False)
+    assert c.layers[1].rot_factor == 0.0 and c.layers[1].shared_ff == 0 and c.layers[2].ff_kind == Ly.FF_NONE
+    assert c.layers[2].rot_dims == 0 and c.layers[7].identity == 3
+    # rows of the input projections
+    assert s.in_rows == 4 * 24 + 2 * (24 + 40) + 4 * 40 and s.side.in_rows == 2 * 3 * 16 + 2 * 3 * 24 + 2 * 3
+    one = {k: v for k, v in FC.ONLY_MOE.items() if k != "logit_softcap"}
+    assert Ly.faguzen_config(one).logit_softcap == 0.0 and [l.shares for l in Ly.faguzen_config(one).layers] == [-1]
+
+
+def test_faguzen_unknown_names_are_refused():
+    import faguzen_cases as FC
+
+    bad = {**FC.ONLY_PAIR, "layers": [{"type": "attention", "mixer": FC.pair(), "mlp": None}]}
+    with pytest.raises(ValueError):
+        Ly.faguzen_config(bad)
+    bad = {**FC.ONLY_PAIR, "layers": [{"type": "parallel", "mixer": FC.pair(), "mlp": {"kind": "dense", "ff": 8}}]}
+    with pytest.raises(ValueError):
+        Ly.faguzen_config(bad)
+    bad = {**FC.ONLY_PAIR, "loop": {"start": 1, "stop": 3, "times": 2}}
+    with pytest.raises(ValueError):
+        Ly.faguzen_config(bad)
+
+
+def test_faguzen_pack_joins_projections_and_norms():
+    import faguzen_cases as FC
+
+    cfg = FC.MIXED
+    t = Ly.faguzen_random_tensors(cfg, seed=3)
+    assert set(t) == set(Ly.faguzen_tensor_shapes(cfg)) and t["l0.norm1.alpha"].shape == ()
+    for wdt in (M.F32, M.BF16):
+        c = Ly.faguzen_config(cfg, weight_dtype=wdt)
+        p = Ly.faguzen_pack(c, t, cfg)
+        f = (lambda a: a) if wdt == M.F32 else Ly.bf16_to_f32
+        W = cfg["width"]
+        for packed, name in ((p["final_norm"], "final.norm"), (p["layers"][0]["norm1"], "l0.norm1"),
+                             (p["layers"][0]["norm2"], "l0.norm2")):
+            assert packed.dtype == np.float32 and packed.shape == (2 * W + 1,)
+            assert np.array_equal(packed[:W], t[name]) and np.array_equal(packed[W:-1], t[name + ".b"])
+            assert packed[-1] == t[name + ".alpha"]
+        assert np.array_equal(f(p["head"]), t["head"]) and np.array_equal(f(p["embed"]), t["embed"])
+        d = p["layers"][0]
+        names = [f"l0.mix.left.{n}" for n in "qkvg"] + [f"l0.mix.right.{n}" for n in "qkvgif"]
+        assert np.array_equal(f(d["w_in"]), np.concatenate([t[n] for n in names]))
+        biases = [t[n + ".b"] if n + ".b" in t else np.zeros(len(t[n]), np.float32) for n in names]
+        assert np.array_equal(d["in_bias"], np.concatenate(biases))
+        assert {n for n in names if n + ".b" in t} == {"l0.mix.left.q", "l0.mix.left.k", "l0.mix.left.v", "l0.mix.right.i",
+                                                       "l0.mix.right.f"}
+        assert np.array_equal(f(d["w_up"][5]), t["l0.mlp.e5.up"]) and d["router"].shape == (8, W)
+        assert np.array_equal(d["router_bias"], t["l0.mlp.correction"]) and "w_gate" not in d and "join_w" not in d
+        assert np.array_equal(d["side"]["out_norm"], t["l0.mix.right.norm"]) and "w_in" not in d["side"]
+        # every later pass holds the first pass's arrays and its own vector
+        for r, first, step in ((3, 1, 1), (5, 1, 2), (4, 2, None)):
+            for k, a in p["layers"][r].items():
+                assert k == "pre_add" or a is p["layers"][first][k]
+            assert step is None or np.array_equal(p["layers"][r]["pre_add"], t["loop.step"][step])
+        for l, d in zip(c.layers, p["layers"]):
+            assert l.shares >= 0 or set(Ly.packed_shapes(c, l)) == set(d) - {"side"}
+
+
+def test_faguzen_checkpoint_folder_is_read(tmp_path):
+    """The registry picks the design by config.json's name; scalar tensors survive the container."""
+    import json
+
+    import faguzen_cases as FC
+    from yalm_amd.yalmfile import write_yalm
+
+    cfg = FC.ODD
+    t = Ly.faguzen_random_tensors(cfg, seed=4)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    write_yalm(str(tmp_path / "model.safetensors"), {k: Ly.f32_to_bf16(v).reshape(v.shape) for k, v in t.items()}, {},
+               {k: "BF16" for k in t})
+    c, p = Ly.read_checkpoint(str(tmp_path), 50, M.F32)
+    q = Ly.faguzen_pack(c, t, cfg)
+    assert c.arch == "Faguzen" and c.max_tokens == 50 and len(p["layers"]) == 3
+    for a, b in zip(p["layers"], q["layers"]):
+        assert all(np.array_equal(a[k], b[k]) for k in b if k != "side")
+        assert all(np.array_equal(a["side"][k], b["side"][k]) for k in b["side"])
+
+
+def test_faguzen_restatement_mechanisms():
+    """The restatement itself: causality; the norm; the rotation's three frequency ranges and its
+    pairing; the memory against the sum it stands for; the router's weights and identity outputs; the
+    loop's order."""
+    import faguzen_cases as FC
+    import faguzen_ref as FR
+
+    cfg = FC.MIXED
+    w = {k: v.astype(np.float64) for k, v in Ly.faguzen_random_tensors(cfg, seed=4).items()}
+    a = FC.tokens(cfg, 40, 1)
+    b = list(a)
+    b[30] = (b[30] + 1) % cfg["vocab"]
+    ra, rb = FR.forward(cfg, w, a), FR.forward(cfg, w, b)
+    assert np.array_equal(ra[:30], rb[:30]) and not np.allclose(ra[30], rb[30]) and not np.allclose(ra[39], rb[39])
+    assert np.abs(ra).max() < cfg["logit_softcap"]
+    assert FR.run_order(cfg) == [(0, None), (1, 0), (2, None), (1, 1), (2, None), (1, 2), (2, None), (3, None)]
+    n = FR.tanh_norm(np.array([[-2.0, 0.0, 9.0]]), {"n": np.array([1.0, 2.0, 3.0]), "n.b": np.array([0.5, 0.5, -0.5]),
+                                                    "n.alpha": np.float64(0.5)}, "n")
+    assert np.allclose(n, [[0.5 - np.tanh(1.0), 0.5, 3 * np.tanh(4.5) - 0.5]])
+    # base 4, four pairs: 100 positions hold 15.9, 11.3, 8.0, 5.6 turns; low 7, high 12
+    f = FR.rotation_frequencies(8, 4.0, {"factor": 10.0, "low": 7.0, "high": 12.0, "original": 100})
+    turns = 100 * 4.0 ** (-np.arange(4) / 4) / (2 * np.pi)
+    s = (turns - 7.0) / 5.0
+    base = 4.0 ** (-np.arange(4) / 4)
+    assert np.allclose(f, [base[0], base[1] * (0.1 * (1 - s[1]) + s[1]), base[2] * (0.1 * (1 - s[2]) + s[2]), base[3] / 10])
+    x = np.zeros((2, 1, 5))
+    x[1, 0] = [1.0, 0.0, 0.0, 2.0, 7.0]
+    r = FR.rotate_halves(x, np.array([0.3, 0.5]))
+    assert np.allclose(r[1, 0], [np.cos(0.3), -2 * np.sin(0.5), np.sin(0.3), 2 * np.cos(0.5), 7.0])
+    # the memory is sum_s exp(i_s + f_{s+1} + .. + f_t) (q.k_s) v_s over max(|the same with v = 1|, 1), up to 1e-6
+    rng = np.random.default_rng(2)
+    q, k, v = rng.standard_normal((12, 1, 3)), rng.standard_normal((12, 1, 3)), rng.standard_normal((12, 1, 2))
+    i, fg = rng.standard_normal((12, 1)), -rng.uniform(0, 1, (12, 1))
+    o = FR.memory_scan(q, k, v, i, fg)
+    for t in range(12):
+        wt = [np.exp(i[s_, 0] + fg[s_ + 1:t + 1, 0].sum()) * (q[t, 0] @ k[s_, 0]) for s_ in range(t + 1)]
+        assert np.allclose(o[t, 0], np.array(wt) @ v[:t + 1, 0] / max(abs(sum(wt)), 1.0), atol=1e-4)
+    idx, wt = FR.route(np.log(np.array([0.1, 0.4, 0.3, 0.2])), np.array([0.0, 0.0, -0.2, 0.05]), 2)
+    assert idx.tolist() == [1, 3] and np.allclose(wt, [2 / 3, 1 / 3])
+    z = np.array([-1.0, 0.0, 2.0])
+    assert np.allclose(FR.gelu_erf(z), [-0.15865525, 0.0, 1.95449974])
+    one = {"r.router": np.array([[-5.0, 0.0], [5.0, 0.0]]), "r.correction": np.zeros(2), "r.e0.up": np.ones((1, 2)),
+           "r.e0.down": np.ones((2, 1))}
+    h = np.array([[1.0, -4.0]])  # the identity output wins: the input itself
+    assert np.allclose(FR.feed_forward(one, "r.", h, {"router": {"experts": 1, "identity": 1, "top": 1}}), h)

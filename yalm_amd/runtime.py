@@ -737,7 +737,8 @@ class SeqModel:
             ptrs = {k: make(f"l{i}.{k}", shape, kind) for k, (shape, kind) in layered.packed_shapes(cfg, l).items()}
             if l.side is not None and l.shares < 0:
                 ptrs["side"] = {k: make(f"l{i}.side.{k}", shape, kind)
-                                for k, (shape, kind) in layered.packed_shapes(cfg, l.side, side=True, shared_in=l.side_shares_in).items()}
+                                for k, (shape, kind) in layered.packed_shapes(
+                                    cfg, l.side, side=True, shared_in=l.side_shares_in).items()}
             if l.shares >= 0:  # a repeated run: the first pass's tensors, its own pre_add
                 ptrs = {**{k: v for k, v in self.layer_ptrs[l.shares].items() if k != "pre_add"}, **ptrs}
             self.layer_ptrs.append(ptrs)
