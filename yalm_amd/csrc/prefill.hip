@@ -114,10 +114,11 @@ int pf_alloc(yalm_decoder_s *d, void **p, size_t bytes) {
 }
 
 // BN for a GEMM of M x N (n_eff = B rows: 2 x hidden for the GLU); 0 = none fits. A
-// forced width that does not divide N falls back to the automatic choice.
-int pick_bn(const PfForms &f, int kind, int M, int n_eff, bool glu) {
+// forced width that does not divide N falls back to the automatic choice. ragged: no width needs to
+// divide N (BRowsRagged), the last tile counts whole.
+int pick_bn(const PfForms &f, int kind, int M, int n_eff, bool glu, bool ragged = false) {
 	static const int cands[4] = {128, 192, 256, 320};
-	auto fits = [&](int bn) { return n_eff % bn == 0 && (!glu || bn == 128 || bn == 256); };
+	auto fits = [&](int bn) { return (n_eff % bn == 0 || (ragged && bn <= 256)) && (!glu || bn == 128 || bn == 256); };
 	const int form = f.g16[kind];
 	if (form > 0 && fits(form) && (form == 128 || form == 192 || form == 256 || form == 320))
 		return form;
@@ -128,7 +129,7 @@ int pick_bn(const PfForms &f, int kind, int M, int n_eff, bool glu) {
 	for (int bn : cands) {
 		if (!fits(bn))
 			continue;
-		const long rounds = (tiles_m * (n_eff / bn) + ncu - 1) / ncu;
+		const long rounds = (tiles_m * ((n_eff + bn - 1) / bn) + ncu - 1) / ncu;
 		// an 8-phase tile (widths 192, 256) costs 3/4 of a 2-phase tile of the same
 		// width (Llama-3B T 4096, one process: Wo / W2 at 256 in the 8-phase kernel beat
 		// 192 in the 2-phase one, profiles/r3_prefill_8phase.txt)
@@ -175,7 +176,7 @@ int launch_g16_t(const PfForms &f, const uint16_t *A, int lda, int M, int K, int
 			return launch_g8p<EPI, BMAP, 2, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
 		if constexpr (BN == 192 && WM == 2)
 			return launch_g8p<EPI, BMAP, 2, 1>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
-		if constexpr (BN == 128 && std::is_same<BMAP, pf::BRowsPlain>::value) // GLU rows pair per 64-col wave
+		if constexpr (BN == 128 && BMAP::COLS_PER_TILE_DIV == 1) // GLU rows pair per 64-col wave
 			return launch_g8p<EPI, BMAP, 1, 1>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
 	}
 	auto kern = pf::gemm16_kernel<EPI, BMAP, BN, WM>;
@@ -192,22 +193,27 @@ int launch_g16_t(const PfForms &f, const uint16_t *A, int lda, int M, int K, int
 }
 
 // C = A · W^T through the large-tile kernel at width bn (pick_bn; 0: no width fits)
-template <class EPI>
-int launch_plain(const PfForms &f, int bn, const uint16_t *A, int lda, int M, int K, int kb, const pf::BSrc &b,
-                 int N, const EPI &epi, hipStream_t st, int c0 = 0) {
-	pf::BRowsPlain bm{b};
+template <class EPI, class BMAP>
+int launch_rows(const PfForms &f, int bn, const uint16_t *A, int lda, int M, int K, int kb, const BMAP &bm, int N,
+                const EPI &epi, hipStream_t st, int c0 = 0) {
 	switch (bn) {
 	case 128:
-		return launch_g16_t<EPI, pf::BRowsPlain, 128, 4>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
+		return launch_g16_t<EPI, BMAP, 128, 4>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
 	case 192:
-		return launch_g16_t<EPI, pf::BRowsPlain, 192, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
+		return launch_g16_t<EPI, BMAP, 192, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
 	case 256:
-		return launch_g16_t<EPI, pf::BRowsPlain, 256, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
+		return launch_g16_t<EPI, BMAP, 256, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
 	case 320:
-		return launch_g16_t<EPI, pf::BRowsPlain, 320, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
+		return launch_g16_t<EPI, BMAP, 320, 2>(f, A, lda, M, K, kb, bm, N, epi, st, c0);
 	}
 	set_err("prefill GEMM: no 256-row tile width (128 / 192 / 256 / 320) divides N, or the forced one does not");
 	return YALM_ERR_UNSUPPORTED;
+}
+
+template <class EPI>
+int launch_plain(const PfForms &f, int bn, const uint16_t *A, int lda, int M, int K, int kb, const pf::BSrc &b,
+                 int N, const EPI &epi, hipStream_t st, int c0 = 0) {
+	return launch_rows(f, bn, A, lda, M, K, kb, pf::BRowsPlain{b}, N, epi, st, c0);
 }
 
 // ---- short prompts (T <= SK_MAX_T): split-K skinny GEMMs (prefill_skinny.h)
@@ -758,15 +764,17 @@ extern "C" int yalm_prefill_time(yalm_decoder d, int n, int iters, float *avg_ms
 }
 
 // The layer-list engine's door to the large-tile GEMM (seq.hip; device pointers, asynchronous
-// on st): C [M][ldc] f32 = act(A [M][lda] bf16 . W [N][K]^T bf16 (+ bias[n])), act 1 = gelu. Same tiles, phases
-// and tile-width choice as the f16 prefill GEMMs; YALM_ERR_UNSUPPORTED (nothing launched)
-// when the shape does not fit them: K % 64, no tile width dividing N, rows not 16-byte aligned.
+// on st): C [M][ldc] f32 = act(A [M][lda] bf16 . W [N][K]^T bf16 (+ bias[n])), act: E16StoreF32B. Same tiles, phases
+// and tile-width choice as the f16 prefill GEMMs (an N that is no multiple of 128 takes a last tile that
+// reaches past it); YALM_ERR_UNSUPPORTED (nothing launched) when the shape does not fit them: K % 64,
+// N below one tile, rows not 16-byte aligned.
 int pf_gemm_bf16(const uint16_t *A, int lda, int M, int K, const uint16_t *W, int N, float *C, int ldc,
                  const float *bias, int act, hipStream_t st) {
 	static const PfForms f = pf_forms_default();
 	if (M <= 0 || K % pf::BK != 0 || lda % 8 != 0 || ((size_t)A | (size_t)W) % 16 != 0)
 		return YALM_ERR_UNSUPPORTED;
-	const int bn = pick_bn(f, PG_TEST, M, N, false);
+	const bool ragged = N % 128 != 0;
+	const int bn = N < 128 ? 0 : pick_bn(f, PG_TEST, M, N, false, ragged);
 	if (!bn)
 		return YALM_ERR_UNSUPPORTED;
 	pf::E16StoreF32B e;
@@ -774,8 +782,9 @@ int pf_gemm_bf16(const uint16_t *A, int lda, int M, int K, const uint16_t *W, in
 	e.bias = bias;
 	e.ldc = ldc;
 	e.M = M;
+	e.N = N;
 	e.act = act;
-	return launch_plain(f, bn, A, lda, M, K, K, one(W, N), N, e, st);
+	return launch_rows(f, bn, A, lda, M, K, K, pf::BRowsRagged{W, N}, (N + bn - 1) / bn * bn, e, st);
 }
 
 // The same door for a gated pair: C [M][ldc] f32 = act(A Wg^T) (.) (A Wu^T) over `hidden` units

@@ -74,6 +74,17 @@ struct BRowsPlain { // W rows n0 + r from up to 3 row-major [rows][K] matrices l
 	}
 };
 
+// One matrix of `rows` rows that need not be a multiple of the tile's width: the last tile's rows past
+// the end repeat the last row, and the epilogue leaves their columns out.
+struct BRowsRagged {
+	const uint16_t *w;
+	int rows;
+	static constexpr int COLS_PER_TILE_DIV = 1;
+	__device__ __forceinline__ const uint16_t *row(int n0, int r, int K) const {
+		return w + (size_t)min(n0 + r, rows - 1) * K;
+	}
+};
+
 // GLU: a tile covers BN / 2 hidden columns h0 .. ; wave column wc's TN B rows are
 // TN / 2 W1 rows then the same TN / 2 W3 rows (h0 + wc * TN / 2 + ..).
 template <int TN>
@@ -121,14 +132,15 @@ struct E16StoreF32B {
 	float *red = nullptr;
 	float *c;
 	const float *bias;
-	int ldc, M;
+	int ldc, M, N; // N: columns that exist (the last tile may reach past them)
 	int act = 0;
 	template <int FI, int FJ>
 	__device__ __forceinline__ void apply(f32x4_t (&acc)[FI][FJ], int m0, int n0, int lane, int, int) const {
 #pragma unroll
 		for (int j = 0; j < FJ; ++j) {
 			const int n = n0 + 16 * j + (lane & 15);
-			const float b = bias ? bias[n] : 0.0f;
+			const bool in = n < N;
+			const float b = bias && in ? bias[n] : 0.0f;
 #pragma unroll
 			for (int i = 0; i < FI; ++i)
 #pragma unroll
@@ -141,7 +153,7 @@ struct E16StoreF32B {
 						v = fmaxf(v, 0.0f) * fmaxf(v, 0.0f);
 					else if (act == 3)
 						v = 0.5f * v * (1.0f + erff(v * 0.7071067811865476f));
-					if (m < M)
+					if (m < M && in)
 						c[(size_t)m * ldc + n] = v;
 				}
 		}

@@ -661,7 +661,7 @@ template <class WT>
 static int gemm_t(Seq *q, const GemmArgs &a, int batches, int max_m) {
 	const bool glu = a.W2 != nullptr;
 	if (max_m <= GEMV_MAX_M) {
-		const dim3 g(cdiv(a.N, SEQ_THREADS / 64), 1, batches);
+		const dim3 g(cdiv(a.own_b ? std::max(a.N, a.N_b) : a.N, SEQ_THREADS / 64), 1, batches);
 		if (glu)
 			seq_gemv_kernel<WT, true><<<g, SEQ_THREADS, 0, q->stream>>>(a);
 		else
@@ -688,15 +688,12 @@ static int gemm(Seq *q, const GemmArgs &a, int batches = 1, int max_m = -1, bool
 		max_m = a.M;
 	if (f32w || q->c.weight_dtype == YALM_F32)
 		return gemm_t<WF32>(q, a, batches, max_m);
-	// plain products of long portions whose shape fits the large-tile GEMM of the prefill unit;
-	// output columns past the last multiple of 128 (a few gate rows closing an input projection)
-	// run on the general kernel as a second, narrow product
+	// plain products of long portions whose shape fits the large-tile GEMM of the prefill unit
 	const bool pair = a.W2 != nullptr && (a.epi == EPI_GLU_GELU || a.epi == EPI_GLU_CLAMP || a.epi == EPI_GLU_SILU) && !a.bias;
 	const bool single = !a.W2 && (a.epi == EPI_NONE || a.epi == EPI_GELU || a.epi == EPI_RELU2 || a.epi == EPI_GELU_ERF);
 	const int act1 = a.epi == EPI_GELU ? 1 : (a.epi == EPI_RELU2 ? 2 : (a.epi == EPI_GELU_ERF ? 3 : 0)); // the large-tile door's activation
-	const int n_big = pair ? (a.N % 64 == 0 ? a.N : 0) : (single ? a.N & ~127 : 0);
 	if (q->a16 && batches == 1 && max_m >= 2 * GB_BM && !a.rows && !a.w_sel && a.z_split == 0 && a.ldw == a.K &&
-	    a.K % 64 == 0 && n_big > 0 && (a.N - n_big <= 64 || (!pair && a.N - n_big < 128))) {
+	    a.K % 64 == 0 && (pair ? a.N % 64 == 0 : (single && a.N >= 128))) {
 		const size_t n8 = (size_t)a.M * (a.K / 8);
 		seq_to_bf16_kernel<<<(unsigned)std::min<size_t>((n8 + SEQ_THREADS - 1) / SEQ_THREADS, 4096), SEQ_THREADS, 0,
 		                     q->stream>>>(a.A, a.lda, a.M, a.K, q->a16);
@@ -704,25 +701,7 @@ static int gemm(Seq *q, const GemmArgs &a, int batches = 1, int max_m = -1, bool
 		const int rc =
 		    pair ? pf_gemm_glu_bf16(q->a16, a.K, a.M, a.K, (const uint16_t *)a.W, (const uint16_t *)a.W2, a.N, a.C, a.ldc,
 		                            a.epi == EPI_GLU_GELU ? 1 : (a.epi == EPI_GLU_CLAMP ? 2 : 3), a.limit, q->stream)
-		         : pf_gemm_bf16(q->a16, a.K, a.M, a.K, (const uint16_t *)a.W, n_big, a.C, a.ldc, a.bias,
-		                        act1, q->stream);
-		if (rc == YALM_OK && !pair && n_big < a.N && a.N >= 128) {
-			// the last 128 columns as one more large tile: it computes the columns below n_big a
-			// second time (the same kernel on the same operands: the same values) and the tail
-			const int c0 = a.N - 128;
-			const int rc2 = pf_gemm_bf16(q->a16, a.K, a.M, a.K, (const uint16_t *)a.W + (size_t)c0 * a.ldw, 128, a.C + c0,
-			                             a.ldc, a.bias ? a.bias + c0 : nullptr, act1, q->stream);
-			if (rc2 != YALM_ERR_UNSUPPORTED)
-				return rc2;
-		}
-		if (rc == YALM_OK && n_big < a.N) {
-			GemmArgs t = a;
-			t.W = (const uint16_t *)a.W + (size_t)n_big * a.ldw;
-			t.C = a.C + n_big;
-			t.bias = a.bias ? a.bias + n_big : nullptr;
-			t.N = a.N - n_big;
-			return gemm_t<WBF16>(q, t, 1, max_m);
-		}
+		         : pf_gemm_bf16(q->a16, a.K, a.M, a.K, (const uint16_t *)a.W, a.N, a.C, a.ldc, a.bias, act1, q->stream);
 		if (rc != YALM_ERR_UNSUPPORTED)
 			return rc;
 	}
@@ -1388,7 +1367,10 @@ static int ff_moe(Seq *q, int li, int n) {
 	const yalm_seq_config &c = q->c;
 	const int E = l.experts, ER = E + l.identity, top = l.top, ff = l.ff, slots = n * top;
 	float *hx = q->B[0], *yx = q->B[1], *hs = q->B[2], *ys = q->B[3];
-	seq_router_kernel<<<n, SEQ_THREADS, (2 * ER + l.groups) * sizeof(float), q->stream>>>(q->In, c.width, l.router, ER, top, l.groups,
+	// the renormalised softmax router's choice is one wave's work: more waves for its logits
+	auto router = l.router_kind == YALM_ROUTER_SOFTMAX_NORMED ? seq_router_kernel<1024> : seq_router_kernel<SEQ_THREADS>;
+	const int rth = l.router_kind == YALM_ROUTER_SOFTMAX_NORMED ? 1024 : SEQ_THREADS;
+	router<<<n, rth, (2 * ER + l.groups) * sizeof(float), q->stream>>>(q->In, c.width, l.router, ER, top, l.groups,
 	                                                                    l.groups_keep, l.router_scale,
 	                                                                    l.shared_ff > 0 ? l.shared_sg : nullptr, q->idx,
 	                                                                    q->wt, q->sgate, l.router_kind, l.router_bias);
@@ -1396,7 +1378,10 @@ static int ff_moe(Seq *q, int li, int n) {
 	// experts without gate matrices are plain: one matrix, its activation, the second matrix
 	const bool glu = l.w_gate != nullptr;
 	const int epi = glu ? glu_epi(l, EPI_GLU_CLAMP) : plain_epi(l);
-	if (n <= GEMV_MAX_M) { // one batch per (token, choice): its expert's matrices picked on the device
+	// a few tokens: one batch per (token, choice), its expert's matrices picked on the device; the shared
+	// expert is the last batch
+	if (n <= GEMV_MAX_M) {
+		const bool shared = l.shared_ff > 0;
 		GemmArgs a = plain(q->In, c.width, glu ? l.w_gate : l.w_up, c.width, hx, ff, 1, ff, c.width);
 		a.W2 = glu ? l.w_up : nullptr;
 		a.a_bs = c.width;
@@ -1407,14 +1392,29 @@ static int ff_moe(Seq *q, int li, int n) {
 		a.c_bs = ff;
 		a.epi = epi;
 		a.limit = l.limit;
-		TRY(gemm(q, a, slots));
 		GemmArgs b = plain(hx, ff, l.w_down, ff, yx, c.width, 1, c.width, ff);
 		b.a_bs = ff;
 		b.w_sel = q->idx;
 		b.w_count = E;
 		b.w_bs = (long)c.width * ff;
 		b.c_bs = c.width;
-		TRY(gemm(q, b, slots));
+		if (shared) {
+			a.own_b = b.own_b = true;
+			a.z_split = b.z_split = slots;
+			a.M_b = b.M_b = n;
+			a.A_b = q->In;
+			a.W_b = glu ? l.ws_gate : l.ws_up;
+			a.W2_b = glu ? l.ws_up : nullptr;
+			a.C_b = hs;
+			b.A_b = hs;
+			a.N_b = b.K_b = l.shared_ff;
+			a.K_b = b.N_b = c.width;
+			a.limit_b = l.shared_limit;
+			b.W_b = l.ws_down;
+			b.C_b = ys;
+		}
+		TRY(gemm(q, a, slots + (shared ? 1 : 0)));
+		return gemm(q, b, slots + (shared ? 1 : 0));
 	} else { // tokens grouped by expert: one batch per expert over its row list
 		seq_fill_int_kernel<<<cdiv(E, 256), 256, 0, q->stream>>>(q->counts, E, 0);
 		seq_moe_lists_kernel<<<cdiv(slots, SEQ_THREADS), SEQ_THREADS, 0, q->stream>>>(q->idx, slots, q->counts, q->lists,
@@ -1465,7 +1465,10 @@ static int par_close(Seq *q, int li, int n) {
 	    (nx && nx->ff_kind != YALM_FF_NONE) ? nx->norm2 : nullptr, q->Hn2, joined ? q->Y3 : nullptr, l.join_w,        \
 	    l.side_join_w, l.join_scale, l.side_join_scale, q->idx, l.experts,                                               \
 	    moe && l.identity > 0 ? (l.norm2 ? q->Hn2 : q->Hn) : nullptr
-	if (c.width <= 4 * SEQ_THREADS)
+	// without row statistics (tanh norms, a plain join) the seam is elementwise: a row spreads over workgroups
+	if (q->nk == NK_TANH && !(joined && l.join_w))
+		seq_par_close_reg_kernel<1><<<dim3(n, cdiv(c.width, SEQ_THREADS)), SEQ_THREADS, 0, q->stream>>>(PC_ARGS);
+	else if (c.width <= 4 * SEQ_THREADS)
 		seq_par_close_reg_kernel<4><<<n, SEQ_THREADS, 0, q->stream>>>(PC_ARGS);
 	else if (c.width <= 8 * SEQ_THREADS)
 		seq_par_close_reg_kernel<8><<<n, SEQ_THREADS, 0, q->stream>>>(PC_ARGS);
@@ -1522,13 +1525,14 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 		}
 		return add_norm(q, wb, w_next, n, moe);
 	};
+	const int eb = q->nk == NK_TANH && !q->embed_norm ? cdiv(c.width, SEQ_THREADS) : 1; // no row statistics: elementwise
 	if (c.weight_dtype == YALM_F32)
-		seq_embed_kernel<WF32><<<n, SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
+		seq_embed_kernel<WF32><<<dim3(n, eb), SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
 		                                                         c.vocab, c.embed_scale, q->X, first_norm, c.norm_eps,
 		                                                         q->Hn, q->nk, q->L[0].pre_add, q->embed_norm, first_norm2,
 		                                                         q->Hn2);
 	else
-		seq_embed_kernel<WBF16><<<n, SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
+		seq_embed_kernel<WBF16><<<dim3(n, eb), SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
 		                                                          c.vocab, c.embed_scale, q->X, first_norm, c.norm_eps,
 		                                                          q->Hn, q->nk, q->L[0].pre_add, q->embed_norm, first_norm2,
 		                                                          q->Hn2);
@@ -1616,7 +1620,8 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 // Final norm of the asked rows and their logits into q->logits ([n_rows][vocab], n_rows <= LOGIT_ROWS).
 static int enqueue_logits(Seq *q, const int *rows_dev, int n_rows) {
 	const yalm_seq_config &c = q->c;
-	seq_norm_kernel<float><<<n_rows, SEQ_THREADS, 0, q->stream>>>(q->X, c.width, q->final_norm, c.norm_eps, c.width,
+	const dim3 ng(n_rows, q->nk == NK_TANH ? cdiv(c.width, SEQ_THREADS) : 1);
+	seq_norm_kernel<float><<<ng, SEQ_THREADS, 0, q->stream>>>(q->X, c.width, q->final_norm, c.norm_eps, c.width,
 	                                                              q->Hn, c.width, rows_dev, q->st, 0, q->nk,
 	                                                              c.logit_scale);
 	HIPCHK(hipGetLastError());

@@ -101,8 +101,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 	int tok = tokens ? tokens[t] : st->token;
 	tok = min(max(tok, 0), vocab - 1);
 	const float p = (float)(st->pos + t);
+	// tanh norms without an embedding norm: the workgroups of a token (gridDim.y) share its entries
+	const int i0 = blockIdx.y * SEQ_THREADS + threadIdx.x, istep = gridDim.y * SEQ_THREADS;
 	float ss = 0.0f, sm = 0.0f;
-	for (int i = threadIdx.x; i < width; i += SEQ_THREADS) {
+	for (int i = i0; i < width; i += istep) {
 		float pe = 0.0f;
 		if (inv_freq) {
 			const float ang = p * inv_freq[i >> 1];
@@ -112,6 +114,11 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 		if (pre_add && !e_norm)
 			v += pre_add[i];
 		X[(size_t)t * width + i] = v;
+		if (nk == NK_TANH && !e_norm && w_next) {
+			Hn[(size_t)t * width + i] = tanh_norm(w_next, width, i, v);
+			if (w_next2)
+				Hn2[(size_t)t * width + i] = tanh_norm(w_next2, width, i, v);
+		}
 		ss = fmaf(v, v, ss);
 		sm += v;
 	}
@@ -128,7 +135,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 			sm += v;
 		}
 	}
-	if (!w_next)
+	if (!w_next || (nk == NK_TANH && !e_norm))
 		return;
 	// the first layer's opening norm in the same launch (each thread re-reads its own entries)
 	if (nk == NK_TANH) {
@@ -173,8 +180,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_norm_kernel(const float *__re
 	const int t = blockIdx.x;
 	const float *x = in + (size_t)(rows ? rows[t] : t) * ld_in;
 	OT *o = out + (size_t)(pos_rows ? st->pos + t : t) * ld_out;
-	if (nk == NK_TANH) {
-		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
+	if (nk == NK_TANH) { // the workgroups of a row (gridDim.y) share its entries
+		for (int i = blockIdx.y * SEQ_THREADS + threadIdx.x; i < n; i += gridDim.y * SEQ_THREADS) {
 			const float v = tanh_norm(w, n, i, x[i]) * post;
 			if constexpr (sizeof(OT) == 2)
 				o[i] = f2bf(v);
@@ -514,8 +521,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
 	}
 }
 
-// The same seam with the row in registers (rows of up to E * SEQ_THREADS entries): every
-// operand row and vector is loaded at once, one memory round trip instead of one per pass.
+// The same seam with the row in registers (rows of up to E * SEQ_THREADS entries; where nothing needs a
+// row's statistics gridDim.y workgroups of E * SEQ_THREADS entries share it): every operand row
+// and vector is loaded at once, one memory round trip instead of one per pass.
 template <int E>
 __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *__restrict__ X, const float *__restrict__ Y1,
                                                                         const float *__restrict__ s1,
@@ -538,12 +546,14 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
                                                                         const int *__restrict__ idx = nullptr,
                                                                         int n_exp = 0, const float *hid = nullptr) {
 	__shared__ float red[SEQ_THREADS / 64];
-	const int t = blockIdx.x;
+	const int t = blockIdx.x, c0 = blockIdx.y * E * SEQ_THREADS + threadIdx.x;
 	float x[E], y1[E], a1[E], f[E], a2[E], ad[E], wn[E];
+	float wn2[E], nb[E] = {}, nb2[E] = {}, al = 0.0f, al2 = 0.0f; // nb, al: biases and alphas of tanh norms
+	const bool tn = nk == NK_TANH && w_next;
 	const bool ff = Yx || Y2;
 #pragma unroll
 	for (int e = 0; e < E; ++e) {
-		const int i = threadIdx.x + e * SEQ_THREADS;
+		const int i = c0 + e * SEQ_THREADS;
 		const bool in = i < n;
 		x[e] = in ? X[(size_t)t * n + i] : 0.0f;
 		y1[e] = in ? Y1[(size_t)t * n + i] : 0.0f;
@@ -552,18 +562,27 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 		ad[e] = (in && add) ? add[i] : 0.0f;
 		wn[e] = (in && w_next) ? w_next[i] : 0.0f;
 		f[e] = (in && Y2 && !Yx) ? Y2[(size_t)t * n + i] : 0.0f;
+		wn2[e] = (in && w_next && w_next2) ? w_next2[i] : 0.0f;
+		if (tn && in) {
+			nb[e] = w_next[n + i];
+			nb2[e] = w_next2 ? w_next2[n + i] : 0.0f;
+		}
+	}
+	if (tn) {
+		al = w_next[2 * n];
+		al2 = w_next2 ? w_next2[2 * n] : 0.0f;
 	}
 	if (Yb && !ja) { // two mixers side by side, a plain weighted sum
 #pragma unroll
 		for (int e = 0; e < E; ++e) {
-			const int i = threadIdx.x + e * SEQ_THREADS;
+			const int i = c0 + e * SEQ_THREADS;
 			y1[e] = i < n ? y1[e] * jscale + Yb[(size_t)t * n + i] * jscale_b : 0.0f;
 		}
 	} else if (Yb) { // two mixers side by side: the normed rows joined before anything else reads y1
 		float yb[E], sa = 0.0f, sb = 0.0f;
 #pragma unroll
 		for (int e = 0; e < E; ++e) {
-			const int i = threadIdx.x + e * SEQ_THREADS;
+			const int i = c0 + e * SEQ_THREADS;
 			yb[e] = i < n ? Yb[(size_t)t * n + i] : 0.0f;
 			sa = fmaf(y1[e], y1[e], sa);
 			sb = fmaf(yb[e], yb[e], sb);
@@ -572,26 +591,38 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 		const float rb = jscale / sqrtf(block_sum(sb, red) / (float)n + eps);
 #pragma unroll
 		for (int e = 0; e < E; ++e) {
-			const int i = threadIdx.x + e * SEQ_THREADS;
+			const int i = c0 + e * SEQ_THREADS;
 			if (i < n)
 				y1[e] = y1[e] * ra * ja[i] + yb[e] * rb * jb[i];
 		}
 	}
 	if (Yx) {
-		for (int k = 0; k < top; ++k) {
-			const float w = wt[(size_t)t * top + k];
-			const float *src = combine_row(Yx, idx, n_exp, hid, t, top, k, n);
+		constexpr int KB = 4; // choices whose rows are in flight together
+		for (int k0 = 0; k0 < top; k0 += KB) {
+			float w[KB], v[KB][E];
 #pragma unroll
-			for (int e = 0; e < E; ++e) {
-				const int i = threadIdx.x + e * SEQ_THREADS;
-				f[e] = fmaf(w, i < n ? src[i] : 0.0f, f[e]);
+			for (int u = 0; u < KB; ++u) {
+				const int k = min(k0 + u, top - 1);
+				w[u] = k0 + u < top ? wt[(size_t)t * top + k] : 0.0f;
+				const float *src = combine_row(Yx, idx, n_exp, hid, t, top, k, n);
+#pragma unroll
+				for (int e = 0; e < E; ++e) {
+					const int i = c0 + e * SEQ_THREADS;
+					v[u][e] = i < n ? src[i] : 0.0f;
+				}
 			}
+#pragma unroll
+			for (int u = 0; u < KB; ++u)
+				if (k0 + u < top)
+#pragma unroll
+					for (int e = 0; e < E; ++e)
+						f[e] = fmaf(w[u], v[u][e], f[e]);
 		}
 		if (Ys) {
 			const float w = sgate ? sgate[t] : 1.0f;
 #pragma unroll
 			for (int e = 0; e < E; ++e) {
-				const int i = threadIdx.x + e * SEQ_THREADS;
+				const int i = c0 + e * SEQ_THREADS;
 				f[e] = fmaf(w, i < n ? Ys[(size_t)t * n + i] : 0.0f, f[e]);
 			}
 		}
@@ -599,7 +630,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	float ss = 0.0f, sm = 0.0f;
 #pragma unroll
 	for (int e = 0; e < E; ++e) {
-		const int i = threadIdx.x + e * SEQ_THREADS;
+		const int i = c0 + e * SEQ_THREADS;
 		float v = fmaf(a1[e], y1[e], x[e]);
 		if (ff)
 			v = fmaf(a2[e], f[e], v);
@@ -615,14 +646,14 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	}
 	if (!w_next)
 		return;
-	if (nk == NK_TANH) {
+	if (tn) {
 #pragma unroll
 		for (int e = 0; e < E; ++e) {
-			const int i = threadIdx.x + e * SEQ_THREADS;
+			const int i = c0 + e * SEQ_THREADS;
 			if (i < n) {
-				Hn[(size_t)t * n + i] = tanh_norm(w_next, n, i, x[e]);
+				Hn[(size_t)t * n + i] = fmaf(tanhf(al * x[e]), wn[e], nb[e]);
 				if (w_next2)
-					Hn2[(size_t)t * n + i] = tanh_norm(w_next2, n, i, x[e]);
+					Hn2[(size_t)t * n + i] = fmaf(tanhf(al2 * x[e]), wn2[e], nb2[e]);
 			}
 		}
 		return;
@@ -632,7 +663,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 		ss = 0.0f;
 #pragma unroll
 		for (int e = 0; e < E; ++e)
-			if (threadIdx.x + e * SEQ_THREADS < n) {
+			if (c0 + e * SEQ_THREADS < n) {
 				x[e] -= mu;
 				ss = fmaf(x[e], x[e], ss);
 			}
@@ -641,11 +672,11 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	const float r = 1.0f / sqrtf(ss / (float)n + eps);
 #pragma unroll
 	for (int e = 0; e < E; ++e) {
-		const int i = threadIdx.x + e * SEQ_THREADS;
+		const int i = c0 + e * SEQ_THREADS;
 		if (i < n) {
 			Hn[(size_t)t * n + i] = x[e] * r * wn[e];
 			if (w_next2)
-				Hn2[(size_t)t * n + i] = x[e] * r * w_next2[i];
+				Hn2[(size_t)t * n + i] = x[e] * r * wn2[e];
 		}
 	}
 }
@@ -722,14 +753,21 @@ struct GemmArgs {
 	const void *W_b = nullptr;
 	float *C_b = nullptr;
 	const float *bias_b = nullptr;
+	// own_b (the GEMV kernel only): the second product is one batch of its own shape, M_b rows A_b
+	// [K_b], matrices W_b (, W2_b) [N_b][K_b], results C_b [N_b], rows contiguous, clamp limit_b
+	bool own_b = false;
+	const float *A_b = nullptr;
+	const void *W2_b = nullptr;
+	int M_b = 0, N_b = 0, K_b = 0;
+	float limit_b = 0.0f;
 };
 
-__device__ __forceinline__ float epi_apply(const GemmArgs &a, float v, float v2, float b) {
+__device__ __forceinline__ float epi_apply(const GemmArgs &a, float v, float v2, float b, float limit) {
 	switch (a.epi) {
 	case EPI_GLU_GELU: return sq_gelu_tanh(v) * v2;
 	case EPI_GLU_CLAMP: {
-		const float g = fminf(v, a.limit);
-		const float u = fminf(fmaxf(v2, -a.limit), a.limit);
+		const float g = fminf(v, limit);
+		const float u = fminf(fmaxf(v2, -limit), limit);
 		return g * sq_sigmoid(1.702f * g) * (u + 1.0f);
 	}
 	case EPI_GLU_SILU: return sq_silu(v) * v2;
@@ -740,7 +778,7 @@ __device__ __forceinline__ float epi_apply(const GemmArgs &a, float v, float v2,
 		return r * r;
 	}
 	case EPI_GELU_ERF: return sq_gelu_erf(v + b);
-	case EPI_SOFT_CAP: return sq_soft_cap(v + b, a.limit);
+	case EPI_SOFT_CAP: return sq_soft_cap(v + b, limit);
 	default: return v + b;
 	}
 }
@@ -751,14 +789,21 @@ struct GemmBatch {
 	float *C;
 	const float *bias;
 	const int *rows;
-	int M;
+	int M, N, K, lda, ldw, ldc;
+	float limit;
 };
 template <class WT>
 __device__ __forceinline__ GemmBatch gemm_batch(const GemmArgs &a, int z) {
 	GemmBatch b;
+	b.N = a.N;
+	b.K = a.K;
+	b.lda = a.lda;
+	b.ldw = a.ldw;
+	b.ldc = a.ldc;
+	b.limit = a.limit;
 	const bool second = a.z_split > 0 && z >= a.z_split;
 	if (second)
-		z -= a.z_split;
+		z = a.own_b ? 0 : z - a.z_split;
 	const long za = a.a_zdiv > 0 ? z / a.a_zdiv : z;
 	b.A = a.A + za * a.a_bs;
 	long zw = a.w_sel ? a.w_sel[z] : z;
@@ -780,10 +825,22 @@ __device__ __forceinline__ GemmBatch gemm_batch(const GemmArgs &a, int z) {
 #define GEMV_MAX_M 8
 template <class WT, bool GLU>
 __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
-	const GemmBatch b = gemm_batch<WT>(a, blockIdx.z);
+	GemmBatch b = gemm_batch<WT>(a, blockIdx.z);
+	if (a.own_b && (int)blockIdx.z == a.z_split) {
+		b.A = a.A_b;
+		b.W = (const char *)a.W_b;
+		b.W2 = (const char *)a.W2_b;
+		b.C = a.C_b;
+		b.bias = nullptr;
+		b.rows = nullptr;
+		b.M = a.M_b;
+		b.N = b.ldc = a.N_b;
+		b.K = b.lda = b.ldw = a.K_b;
+		b.limit = a.limit_b;
+	}
 	const int lane = threadIdx.x & 63;
 	const int n = blockIdx.x * (SEQ_THREADS / 64) + (threadIdx.x >> 6);
-	if (n >= a.N || b.M <= 0)
+	if (n >= b.N || b.M <= 0)
 		return;
 	const int M = min(b.M, GEMV_MAX_M);
 	const float *ar[GEMV_MAX_M];
@@ -792,21 +849,21 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 	for (int m = 0; m < GEMV_MAX_M; ++m) {
 		const int mm = min(m, M - 1);
 		const int s = b.rows ? b.rows[mm] : mm;
-		ar[m] = b.A + (size_t)(b.rows ? s / a.a_div : s) * a.lda;
+		ar[m] = b.A + (size_t)(b.rows ? s / a.a_div : s) * b.lda;
 		crow[m] = (b.rows && !a.c_dense) ? s : mm;
 	}
 	float acc[GEMV_MAX_M] = {}, acc2[GEMV_MAX_M] = {};
-	const char *w = b.W + (size_t)n * a.ldw * WT::BYTES;
-	const char *w2 = GLU ? b.W2 + (size_t)n * a.ldw * WT::BYTES : nullptr;
+	const char *w = b.W + (size_t)n * b.ldw * WT::BYTES;
+	const char *w2 = GLU ? b.W2 + (size_t)n * b.ldw * WT::BYTES : nullptr;
 	constexpr int E = 8; // elements per lane and pass
-	const bool vec = (a.ldw % E == 0) && (((size_t)b.W | (size_t)(GLU ? b.W2 : b.W)) % 16 == 0) && (a.lda % 4 == 0) &&
+	const bool vec = (b.ldw % E == 0) && (((size_t)b.W | (size_t)(GLU ? b.W2 : b.W)) % 16 == 0) && (b.lda % 4 == 0) &&
 	                 ((size_t)b.A % 16 == 0);
 	int kbeg = lane * E;
-	if (M == 1 && vec && a.K % E == 0) {
+	if (M == 1 && vec && b.K % E == 0) {
 		// one token, whole aligned rows: four 512-element steps of the weight row (non-temporal:
 		// read once per token) and of the activation row in flight before the first FMA
 		constexpr int U = 4;
-		for (; kbeg + (U - 1) * 64 * E < a.K; kbeg += U * 64 * E) {
+		for (; kbeg + (U - 1) * 64 * E < b.K; kbeg += U * 64 * E) {
 			u32x4_t wv[U][WT::BYTES == 2 ? 1 : 2], wv2[U][WT::BYTES == 2 ? 1 : 2];
 			float4_t xv[U][2];
 #pragma unroll
@@ -852,9 +909,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 			}
 		}
 	}
-	for (int k0 = kbeg; k0 < a.K; k0 += 64 * E) {
+	for (int k0 = kbeg; k0 < b.K; k0 += 64 * E) {
 		float wf[E], wf2[E];
-		const bool full = vec && k0 + E <= a.K;
+		const bool full = vec && k0 + E <= b.K;
 		if (full) {
 			if constexpr (WT::BYTES == 2) {
 				WT::unpack(load16(w + (size_t)k0 * 2), wf);
@@ -871,9 +928,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 		} else {
 #pragma unroll
 			for (int e = 0; e < E; ++e) {
-				wf[e] = k0 + e < a.K ? wload<WT>(w, k0 + e) : 0.0f;
+				wf[e] = k0 + e < b.K ? wload<WT>(w, k0 + e) : 0.0f;
 				if constexpr (GLU)
-					wf2[e] = k0 + e < a.K ? wload<WT>(w2, k0 + e) : 0.0f;
+					wf2[e] = k0 + e < b.K ? wload<WT>(w2, k0 + e) : 0.0f;
 			}
 		}
 #pragma unroll
@@ -890,7 +947,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 				} else {
 #pragma unroll
 					for (int e = 0; e < E; ++e)
-						x[e] = k0 + e < a.K ? ar[m][k0 + e] : 0.0f;
+						x[e] = k0 + e < b.K ? ar[m][k0 + e] : 0.0f;
 				}
 #pragma unroll
 				for (int e = 0; e < E; ++e) {
@@ -907,7 +964,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 			const float v = wave_sum(acc[m]);
 			const float v2 = GLU ? wave_sum(acc2[m]) : 0.0f;
 			if (lane == 0)
-				b.C[(size_t)crow[m] * a.ldc + n] = epi_apply(a, v, v2, b.bias ? b.bias[n] : 0.0f);
+				b.C[(size_t)crow[m] * b.ldc + n] = epi_apply(a, v, v2, b.bias ? b.bias[n] : 0.0f, b.limit);
 		}
 	}
 }
@@ -1131,7 +1188,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_kernel(GemmArgs a) {
 				const int ml = wm + (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
 				const int rc = crow[ml];
 				if (rc >= 0)
-					b.C[(size_t)rc * a.ldc + n] = epi_apply(a, acc[r], GLU ? acc2[r] : 0.0f, bias);
+					b.C[(size_t)rc * a.ldc + n] = epi_apply(a, acc[r], GLU ? acc2[r] : 0.0f, bias, b.limit);
 			}
 		}
 	} else {
@@ -1180,7 +1237,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_kernel(GemmArgs a) {
 				const int n = n0 + tx * 4 + j;
 				if (n < a.N)
 					b.C[(size_t)rc * a.ldc + n] =
-					    epi_apply(a, acc[i][j], GLU ? acc2[i][j] : 0.0f, b.bias ? b.bias[n] : 0.0f);
+					    epi_apply(a, acc[i][j], GLU ? acc2[i][j] : 0.0f, b.bias ? b.bias[n] : 0.0f, b.limit);
 			}
 		}
 	}
@@ -1345,7 +1402,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_bf16_kernel(GemmArgs a) 
 				const int ml = wm + 32 * i + (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
 				const int rc = crow[ml];
 				if (rc >= 0)
-					b.C[(size_t)rc * a.ldc + n] = epi_apply(a, acc[i][j][r], GLU ? acc2[i][j][r] : 0.0f, bias);
+					b.C[(size_t)rc * a.ldc + n] = epi_apply(a, acc[i][j][r], GLU ? acc2[i][j][r] : 0.0f, bias, b.limit);
 			}
 	}
 }
@@ -2248,9 +2305,11 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_latent_attn_mfma_kernel(const
 // win (ties: the lower index); weight = score * rscale, without the bias, not renormalised. kind 3:
 // scores = softmax over all E; the `top` largest score + bias win (ties: the lower index, no groups);
 // weight = score / (sum of the chosen scores + 1e-20) * rscale.
+// NT threads (kind 0: SEQ_THREADS).
 // Also the shared expert's gate sigmoid(w_sg . h). Dynamic LDS: 2 E + G floats.
 #define SEQ_MAX_GROUPS 64
-__global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__restrict__ Hn, int width,
+template <int NT>
+__global__ __launch_bounds__(NT) void seq_router_kernel(const float *__restrict__ Hn, int width,
                                                                  const float *__restrict__ Wr, int E, int top, int G,
                                                                  int keep, float rscale,
                                                                  const float *__restrict__ w_sg, int *__restrict__ idx,
@@ -2260,7 +2319,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__
 	const int t = blockIdx.x;
 	const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
 	const float *h = Hn + (size_t)t * width;
-	for (int e = wave; e < E + (w_sg ? 1 : 0); e += SEQ_THREADS / 64) {
+	for (int e = wave; e < E + (w_sg ? 1 : 0); e += NT / 64) {
 		const float *w = e < E ? Wr + (size_t)e * width : w_sg;
 		float a = 0.0f;
 		if (width % 4 == 0 && ((size_t)w | (size_t)h) % 16 == 0) {
@@ -2411,54 +2470,56 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_router_kernel(const float *__
 		}
 		return;
 	}
-	float mx = -FLT_MAX;
-	for (int e = threadIdx.x; e < E; e += SEQ_THREADS)
-		mx = fmaxf(mx, sc[e]);
-	mx = wave_max(mx);
-	if (lane == 0)
-		red[wave] = mx;
-	__syncthreads();
-	mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
-	float sum = 0.0f;
-	for (int e = threadIdx.x; e < E; e += SEQ_THREADS) {
-		const float v = expf(sc[e] - mx);
-		sc[e] = v;
-		sum += v;
-	}
-	sum = block_sum(sum, red);
-	const float inv = 1.0f / sum;
-	const int gs = E / G;
-	for (int g = threadIdx.x; g < G; g += SEQ_THREADS) {
-		float m = -1.0f;
-		for (int e = g * gs; e < (g + 1) * gs; ++e)
-			m = fmaxf(m, sc[e]);
-		gsc[g] = m;
-	}
-	__syncthreads();
-	if (threadIdx.x != 0)
-		return;
-	unsigned long long allowed = 0ull; // groups that may be chosen from (G <= 64)
-	for (int k = 0; k < keep; ++k) {
-		int best = -1;
-		float bv = -2.0f;
-		for (int g = 0; g < G; ++g)
-			if (!((allowed >> g) & 1ull) && gsc[g] > bv) {
-				bv = gsc[g];
-				best = g;
-			}
-		allowed |= 1ull << best;
-	}
-	for (int k = 0; k < top; ++k) {
-		int best = 0;
-		float bv = -1.0f;
-		for (int e = 0; e < E; ++e)
-			if (((allowed >> (e / gs)) & 1ull) && sc[e] > bv) {
-				bv = sc[e];
-				best = e;
-			}
-		idx[(size_t)t * top + k] = best;
-		wt[(size_t)t * top + k] = bv * inv * rscale;
-		sc[best] = -1.0f; // taken
+	if constexpr (NT == SEQ_THREADS) { // kind 0
+		float mx = -FLT_MAX;
+		for (int e = threadIdx.x; e < E; e += SEQ_THREADS)
+			mx = fmaxf(mx, sc[e]);
+		mx = wave_max(mx);
+		if (lane == 0)
+			red[wave] = mx;
+		__syncthreads();
+		mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+		float sum = 0.0f;
+		for (int e = threadIdx.x; e < E; e += SEQ_THREADS) {
+			const float v = expf(sc[e] - mx);
+			sc[e] = v;
+			sum += v;
+		}
+		sum = block_sum(sum, red);
+		const float inv = 1.0f / sum;
+		const int gs = E / G;
+		for (int g = threadIdx.x; g < G; g += SEQ_THREADS) {
+			float m = -1.0f;
+			for (int e = g * gs; e < (g + 1) * gs; ++e)
+				m = fmaxf(m, sc[e]);
+			gsc[g] = m;
+		}
+		__syncthreads();
+		if (threadIdx.x != 0)
+			return;
+		unsigned long long allowed = 0ull; // groups that may be chosen from (G <= 64)
+		for (int k = 0; k < keep; ++k) {
+			int best = -1;
+			float bv = -2.0f;
+			for (int g = 0; g < G; ++g)
+				if (!((allowed >> g) & 1ull) && gsc[g] > bv) {
+					bv = gsc[g];
+					best = g;
+				}
+			allowed |= 1ull << best;
+		}
+		for (int k = 0; k < top; ++k) {
+			int best = 0;
+			float bv = -1.0f;
+			for (int e = 0; e < E; ++e)
+				if (((allowed >> (e / gs)) & 1ull) && sc[e] > bv) {
+					bv = sc[e];
+					best = e;
+				}
+			idx[(size_t)t * top + k] = best;
+			wt[(size_t)t * top + k] = bv * inv * rscale;
+			sc[best] = -1.0f; // taken
+		}
 	}
 }
 
