@@ -2,7 +2,8 @@
 HIPCC ?= /opt/rocm/bin/hipcc
 CXX ?= g++
 ARCH ?= gfx950
-HIPFLAGS = --offload-arch=$(ARCH) -O3 -std=c++17 -fPIC -Wall
+# no packed-FP32 VALU forms: the compiler would make v_pk_*_f32 of ordinary float code by itself
+HIPFLAGS = --offload-arch=$(ARCH) -O3 -std=c++17 -fPIC -Wall -Xclang -target-feature -Xclang -packed-fp32-ops
 CSRC = yalm_amd/csrc
 HIP_SRCS = $(CSRC)/shim.hip $(CSRC)/yalm_hip.hip $(CSRC)/prefill.hip $(CSRC)/seq.hip
 HIP_OBJS = $(patsubst $(CSRC)/%.hip,build/%.o,$(HIP_SRCS))
@@ -24,9 +25,6 @@ yalm_amd/libyalm_seq.so: build/shim.o build/seq.o
 # S^T accumulators are touched by VALU (softmax, rescale), and the AGPR form copied all 64 O
 # registers out and back on every key tile (260 registers -> 1 wave per SIMD; 175 without)
 build/prefill.o: HIPFLAGS += -mllvm -amdgpu-mfma-vgpr-form
-
-# the newer units are built without packed-FP32 VALU forms
-build/shim.o build/seq.o: HIPFLAGS += -Xclang -target-feature -Xclang -packed-fp32-ops
 
 build/%.o: $(CSRC)/%.hip $(HIP_HDRS)
 	@mkdir -p build
@@ -52,6 +50,6 @@ clean:
 TOOLS = stream_bench launch_bench persist_bench mall_bench concurrency_check wg_timeline
 tools: $(addprefix tools/,$(TOOLS))
 tools/%: tools/%.hip $(HIP_HDRS)
-	$(HIPCC) --offload-arch=$(ARCH) -O3 -std=c++17 -o $@ $<
+	$(HIPCC) --offload-arch=$(ARCH) -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops -o $@ $<
 
 .PHONY: all seq oracle host clean resource-usage tools

@@ -18,7 +18,7 @@ fi
 mkdir -p "$root/yalm_amd/ab"
 for f in yalm_hip prefill; do  # EXTRA_DEFS: more -D flags for the A/B build
   extra=""; [ $f = prefill ] && extra="-mllvm -amdgpu-mfma-vgpr-form"
-  /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC $def ${EXTRA_DEFS:-} $extra -c -o "$tmp/$f.o" "$tmp/yalm_amd/csrc/$f.hip" &
+  /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -Xclang -target-feature -Xclang -packed-fp32-ops $def ${EXTRA_DEFS:-} $extra -c -o "$tmp/$f.o" "$tmp/yalm_amd/csrc/$f.hip" &
 done
 wait
 /opt/rocm/bin/hipcc --offload-arch=gfx950 -O3 -std=c++17 -fPIC -shared -o "$root/yalm_amd/ab/libyalm_hip_$rev$suf.so" \
