@@ -422,16 +422,17 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 }
 
 // The seam after a parallel block, one launch: X[t] += rs (s1 * Y1[t] + s2 * Y2[t]) (rs the model's
-// residual scale, s1, s2 the block's elementwise scales; Y2 == nullptr and Yx == nullptr: no feed-forward). Yx != nullptr:
-// the feed-forward's row is the routed experts' combine sum_k wt[t][k] Yx[t top + k] (+ sgate[t]
-// Ys[t], the shared expert; sgate == nullptr: + Ys[t]), summed in slot order; hid: see combine_row
-// (may be Hn or Hn2: every entry is read before it is overwritten). dump != nullptr: the row after the sums is also written there (the stream as the block leaves it). Then
-// X[t] += add (the vector the next layer adds before its opening norm) and, if w_next, Hn[t]
-// = norm(X[t]) * w_next and, with w_next2, Hn2[t] = norm(X[t]) * w_next2 (the norm the next
-// block's feed-forward reads). s1 / s2 == nullptr: scale 1. Yb != nullptr: the block has two
-// mixers side by side and its mixer row is jscale (rms(Y1[t]) ja + rms(Yb[t]) jb), each row
-// divided by its own root mean square over n (no mean taken off), or, ja == nullptr, the plain
-// sum jscale Y1[t] + jscale_b Yb[t]. Dynamic LDS: n floats.
+// residual scale, s1, s2 the block's elementwise scales, nullptr: 1; Y2 == nullptr and Yx == nullptr:
+// no feed-forward). Yx != nullptr: the feed-forward's row is the routed experts' combine
+// sum_k wt[t][k] Yx[t top + k] (+ sgate[t] Ys[t], the shared expert; sgate == nullptr: + Ys[t]), summed
+// in slot order; hid: see combine_row (may be Hn or Hn2: every entry is read before it is
+// overwritten). dump != nullptr: the row after the sums is also written there (the stream as the
+// block leaves it). Then X[t] += add (the vector the next layer adds before its opening norm) and,
+// if w_next, Hn[t] = norm(X[t]) * w_next and, with w_next2, Hn2[t] = norm(X[t]) * w_next2 (the norm
+// the next block's feed-forward reads). Yb != nullptr: the block has two mixers side by side and its
+// mixer row is jscale (rms(Y1[t]) ja + rms(Yb[t]) jb), each row divided by its own root mean square
+// over n (no mean taken off), or, ja == nullptr, the plain sum jscale Y1[t] + jscale_b Yb[t].
+// Dynamic LDS: n floats.
 __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__restrict__ X, const float *__restrict__ Y1,
                                                                     const float *__restrict__ s1,
                                                                     const float *__restrict__ Y2,
