@@ -313,16 +313,18 @@ int yalm_set_prefill_forms(yalm_decoder d, const char *spec);
  * another: every layer names a token mixer (latent attention over a cached low-rank
  * key/value latent, a real-gated linear recurrence, a gated delta rule, softmax attention
  * over cached keys and values with a window or chunk mask, a selective state-space layer, a
- * matrix memory with exponential gates; or two of them side by side on the same input) and a feed-forward (none, dense
+ * matrix memory with exponential gates, a gated linear attention; or two of them side by side on the same input) and a feed-forward (none, dense
  * GLU, routed experts with an optional shared expert, a plain two-matrix one), each with
  * its own sizes and constants. Serial blocks (block_kind = YALM_BLOCK_SERIAL): around every
  * sublayer x += norm_b(f(norm(x))) (pre_norm = 1) or x += norm_b(f(x)) (pre_norm = 0).
  * Parallel blocks (YALM_BLOCK_PARALLEL): h = norm1(x), x += ls1 * mixer(h) + ls2 * ff(h), one
  * norm read by both sublayers, each result scaled elementwise by its own vector (NULL: 1); a
- * layer of such a block that has norm2 feeds its feed-forward norm2(x) of the same x. Every
- * sublayer's result is also scaled by residual_scale. The norms are rms norms or mean-subtracting
- * layer norms (both with a weight and no bias), or YALM_NORM_TANH: tanh(alpha x) w + b elementwise, no
- * statistics, its vector [2 width + 1] holding w, b and alpha one after the other (norm_kind).
+ * layer of such a block that has norm2 feeds its feed-forward norm2(x) of the same x. Post-norm
+ * blocks (YALM_BLOCK_POST, pre_norm = 0): around every sublayer x <- norm_b(stream_scale * x + f(x)),
+ * the sublayers reading the stream itself. Every sublayer's result is also scaled by residual_scale. The norms are rms norms or mean-subtracting
+ * layer norms (both with a weight and no bias), YALM_NORM_LAYER_BIAS: a layer norm with a bias, its
+ * vector [2 width] holding weight and bias one after the other, or YALM_NORM_TANH: tanh(alpha x) w + b
+ * elementwise, no statistics, its vector [2 width + 1] holding w, b and alpha (norm_kind).
  * The layer array is the order the layers RUN in: a block of layers that is walked several
  * times with the same weights is passed unrolled, its entries naming the same tensors, and
  * every entry has its own caches and states; pre_add is a vector added to the stream before
@@ -336,10 +338,10 @@ int yalm_set_prefill_forms(yalm_decoder d, const char *spec);
  * weight-streaming GEMVs for single tokens) or YALM_F32 (true f32 products).
  * Matrices are row-major [out][in]. */
 enum { YALM_MIX_LATENT = 0, YALM_MIX_RGLRU = 1, YALM_MIX_DELTA = 2, YALM_MIX_ATTN = 3, YALM_MIX_SSM = 4,
-	   YALM_MIX_MEMORY = 5 };
+	   YALM_MIX_MEMORY = 5, YALM_MIX_GLA = 6 };
 enum { YALM_FF_NONE = 0, YALM_FF_DENSE = 1, YALM_FF_MOE = 2, YALM_FF_PLAIN = 3 };
-enum { YALM_NORM_RMS = 0, YALM_NORM_LAYER = 1, YALM_NORM_TANH = 2 };
-enum { YALM_BLOCK_SERIAL = 0, YALM_BLOCK_PARALLEL = 1 };
+enum { YALM_NORM_RMS = 0, YALM_NORM_LAYER = 1, YALM_NORM_TANH = 2, YALM_NORM_LAYER_BIAS = 3 };
+enum { YALM_BLOCK_SERIAL = 0, YALM_BLOCK_PARALLEL = 1, YALM_BLOCK_POST = 2 };
 /* gated feed-forwards: y = w_down (act(w_gate x) (.) w_up x) */
 enum { YALM_ACT_DEFAULT = 0, /* dense: gelu; experts and shared expert: clamp */
 	   YALM_ACT_GELU = 1,  /* gelu_tanh(g) u */
@@ -353,9 +355,11 @@ enum { YALM_ROUTER_SOFTMAX_TOP = 0, /* softmax over all experts, best groups, to
 	   YALM_ROUTER_SIGMOID_GROUPS = 2, /* scores sigmoid(logit); the choice ranks score + router_bias: a group by the sum of
 	                                    its two largest, the `top` largest within the groups_keep best groups win (ties: the
 	                                    lower index); weight = score * router_scale (without the bias, not renormalised) */
-	   YALM_ROUTER_SOFTMAX_NORMED = 3 /* scores softmax over experts and identity outputs; the `top` largest score + router_bias
+	   YALM_ROUTER_SOFTMAX_NORMED = 3, /* scores softmax over experts and identity outputs; the `top` largest score + router_bias
 	                                    win (ties: the lower index, no groups); weight = score (without the bias) divided by the
-	                                    chosen scores' sum + 1e-20, times router_scale */ };
+	                                    chosen scores' sum + 1e-20, times router_scale */
+	   YALM_ROUTER_SIGMOID_TOP = 4 /* the `top` largest logits + router_bias win (ties: the lower index, no groups); weight =
+	                                  sigmoid(logit) * router_scale (without the bias, not renormalised) */ };
 /* attn: which earlier positions j <= i a position i sees */
 enum { YALM_MASK_CAUSAL = 0, /* all of them */
 	   YALM_MASK_WINDOW = 1, /* i - j < mask_size */
@@ -367,12 +371,12 @@ enum { YALM_QK_NONE = 0,
 	   YALM_QK_HEAD_W = 3 /* every head rms-normed over dim, times q_norm / kv_norm [dim] shared by all heads (no rotation) */ };
 /* attn, latent: which entries of a head's first rot_dims turn together */
 enum { YALM_ROT_INTERLEAVED = 0, /* (2i, 2i + 1) */
-	   YALM_ROT_HALVES = 1 /* (i, i + rot_dims / 2) (attn) */ };
+	   YALM_ROT_HALVES = 1 /* (i, i + rot_dims / 2) */ };
 /* attn: how rot_factor > 0 rescales the frequencies */
 enum { YALM_RAMP_INDEX = 0, /* a linear ramp over the pair index; cos and sin scaled, see rot_factor */
 	   YALM_RAMP_TURNS = 1 /* by t, the times a pair turns within rot_orig positions: f kept for t > rot_fast, f / rot_factor
 	                          for t < rot_slow, between (1 - s) f / rot_factor + s f with s = (t - slow) / (fast - slow) */ };
-/* delta: activation of the output gate */
+/* delta, gla: activation of the output gate */
 enum { YALM_GATE_SILU = 0, YALM_GATE_SIGMOID = 1 };
 
 typedef struct yalm_seq_layer {
@@ -381,12 +385,14 @@ typedef struct yalm_seq_layer {
 	                                  queries / keys shared by heads / kv_heads value heads of vdim; attn: heads
 	                                  query heads of dim, kv_heads key (dim) / value (vdim) heads, query head h
 	                                  reads key/value head h / (heads / kv_heads) */
-	int kv_rank, q_rank, kv_from;  /* latent: ranks; kv_from >= 0: read that layer's latent cache (no own w_in rows);
+	int kv_rank, q_rank, kv_from;  /* latent: ranks; kv_from >= 0: read that layer's latent cache (no latent rows and, with
+	                                  q_rank = 0, no rotated key rows of its own in w_in; the rotated key part is shared too);
 	                                  q_rank = 0: the queries are projected from the input directly */
 	int rot_dim;                   /* latent with q_rank = 0: every query head is [dim plain | rot_dim rotated] entries and
 	                                  w_in's last rot_dim rows give one rotated key part shared by all heads (not normed),
 	                                  score = (q_plain . W_uk c + q_rot . k_rot) * attn_scale; rotation as rot_dims / rot_base
-	                                  below (rot_dims <= rot_dim); mask_kind / mask_size / sink / sink_w apply */
+	                                  below (rot_dims <= rot_dim); mask_kind / mask_size / sink / sink_w apply, and out_gate 0 or 2
+	                                  (the gate rows close w_in) */
 	float attn_scale;              /* latent, attn: score = q.k * attn_scale */
 	int rec_width, blocks;         /* rglru: channels, diagonal gate blocks */
 	int conv;                      /* rglru, delta: taps of the causal per-channel convolution */
@@ -433,7 +439,7 @@ typedef struct yalm_seq_layer {
 	float rel_max;
 	float join_scale;              /* side != NULL: mixer result = join_scale (rms(a) join_w + rms(b) side_join_w) */
 	float side_join_scale;         /* side != NULL with join_w NULL: mixer result = join_scale a + side_join_scale b */
-	int rot_pairs, rot_ramp;       /* attn: YALM_ROT_*, YALM_RAMP_* */
+	int rot_pairs, rot_ramp;       /* attn, latent (rot_pairs): YALM_ROT_*, YALM_RAMP_* */
 	float softcap;                 /* attn: > 0: the scaled score s becomes softcap tanh(s / softcap), before mask and softmax */
 	/* memory (YALM_MIX_MEMORY, the matrix memory of xLSTM): heads heads of dim keys and vdim values; w_in rows [q: heads
 	   dim | k: heads dim | v: heads vdim | output gate: heads vdim | i: heads | f: heads] (+ in_bias); per head the log
@@ -444,6 +450,12 @@ typedef struct yalm_seq_layer {
 	float gate_cap;
 	int identity;                  /* moe: identity outputs after the experts (router and router_bias have experts +
 	                                  identity rows): a chosen one adds the feed-forward's input times its weight */
+	/* gla (YALM_MIX_GLA, gated linear attention): heads heads of dim keys and vdim values; w_in rows [q: heads dim | k: heads
+	   dim | v: heads vdim | output gate: heads vdim | decay: decay_rank]; one decay per head and key channel, a = sigmoid(w_a2
+	   (decay rows) + dt_bias)^(1 / decay_tau), w_a2 [heads dim][decay_rank], dt_bias [heads dim]; S <- diag(a) S + k v^T,
+	   o = S^T (q dim^-1/2); o rms-normed per head, times out_norm [vdim], times gate_act(output gate); then w_o */
+	float decay_tau;
+	int expert_in_weighted;        /* moe: 1: a choice's weight multiplies its expert's INPUT, the outputs are summed as they are */
 	/* f32 vectors */
 	const float *norm1, *norm1b, *norm2, *norm2b; /* [width] each; norm2* unused without a feed-forward; parallel blocks: norm1 only */
 	const float *ls1, *ls2;         /* parallel blocks: [width] scales of the mixer's and the feed-forward's result */
@@ -458,11 +470,12 @@ typedef struct yalm_seq_layer {
 	const float *conv_w, *conv_b;   /* [channels][conv] (last column = current token); rglru bias [rec_width] */
 	const float *gate_a, *gate_a_b, *gate_i, *gate_i_b; /* rglru: [blocks][bs][bs], [rec_width] (bs = rec_width / blocks) */
 	const float *lam;               /* rglru: [rec_width] */
-	const float *a_log, *dt_bias, *out_norm; /* delta: [heads], [heads] ([heads dim] with decay_rank), [vdim]; ssm: [heads], [heads], [heads vdim]; memory: -, -, [heads vdim] */
+	const float *a_log, *dt_bias, *out_norm; /* delta: [heads], [heads] ([heads dim] with decay_rank), [vdim]; ssm: [heads], [heads], [heads vdim]; memory: -, -, [heads vdim]; gla: -, [heads dim], [vdim] */
 	const float *router, *shared_sg; /* moe: [experts + identity][width]; [width]: the shared expert times sigmoid(shared_sg . x), NULL: times 1 */
 	/* matrices of weight_dtype */
 	const void *w_in;  /* latent: [q_rank (+ kv_rank if own latent)][width] (query down, latent down), with q_rank = 0
-	                      [heads (dim + rot_dim) + kv_rank + rot_dim][width] (queries, latent down, rotated key part);
+	                      [heads (dim + rot_dim) (+ kv_rank + rot_dim if own latent) (+ heads vdim if out_gate)][width]
+	                      (queries, latent down, rotated key part, gate);
 	                      rglru: [2 rec_width][width] (gate branch, recurrent branch);
 	                      delta: [2 kv_heads dim + heads vdim + (gate_rank | heads vdim) + heads + (decay_rank | heads)][width]
 	                      (q, k, v, output gate, beta, decay);
@@ -482,7 +495,7 @@ typedef struct yalm_seq_layer {
 	const float *rel;              /* attn: [rel_rows][heads], see rel_rows */
 	const float *d_skip;           /* ssm: [heads] */
 	const float *join_w, *side_join_w; /* side != NULL: [width] each, or both NULL (see side_join_scale) */
-	const void *w_a2, *w_g2;       /* delta: see decay_rank / gate_rank */
+	const void *w_a2, *w_g2;       /* delta, gla (w_a2): see decay_rank / gate_rank */
 	const struct yalm_seq_layer *side; /* HOST pointer or NULL: a second mixer that reads the same input beside this
 	                                  one (its mixer fields and tensors only; no norms, no feed-forward, no side of its
 	                                  own), with caches and states of its own; the two results are each rms-normed over
@@ -500,18 +513,24 @@ typedef struct yalm_seq_config {
 	int pre_norm;     /* 1: a sublayer reads norm1 / norm2 of the stream; 0: it reads the stream itself (norm1 / norm2 unused) */
 	int pos_embed;    /* 1: the interleaved sin / cos position vector (frequencies 10000^(-2i / width)) is added to the embedding */
 	float logit_scale; /* logits = head . norm(x) * logit_scale */
-	int block_kind;   /* YALM_BLOCK_*; parallel blocks need pre_norm = 1 */
+	int block_kind;   /* YALM_BLOCK_*; parallel blocks need pre_norm = 1, post-norm blocks pre_norm = 0 */
 	float residual_scale; /* every sublayer's result times this as it joins the stream */
 	float logit_softcap;  /* > 0: logits <- logit_softcap tanh(logits / logit_softcap) */
+	float stream_scale;   /* post-norm blocks: the stream times this as a sublayer's result is added to it */
+	int bigram_buckets;   /* > 0: a row of the table `bigram` joins every token's embedding (see there) */
+	long long bigram_mul_prev, bigram_mul_cur;
 } yalm_seq_config;
 
 typedef struct yalm_seq_weights {
 	const void *embed;       /* [vocab][width] */
-	const float *final_norm; /* [width] (YALM_NORM_TANH: [2 width + 1], as every norm) */
+	const float *final_norm; /* [width] (YALM_NORM_LAYER_BIAS: [2 width], YALM_NORM_TANH: [2 width + 1], as every norm) */
 	const void *head;        /* [vocab][width] */
 	const yalm_seq_layer *layers; /* HOST array of n_layers entries, copied by yalm_seq_create */
 	const float *embed_norm;  /* [width] or NULL: the embedding row (scaled, with its position vector) is normed
 	                             with this weight before it becomes the stream */
+	const void *bigram;       /* [bigram_buckets + 1][width] of weight_dtype: row (previous token * bigram_mul_prev + token *
+	                             bigram_mul_cur) mod bigram_buckets is added to the embedding (not scaled), the last row for
+	                             a sequence's first token; the previous token is part of the sequence's state */
 } yalm_seq_weights;
 
 typedef struct yalm_seq_s *yalm_seq;

@@ -1,7 +1,7 @@
 // seq.hip — the layer-list engine of the C ABI (include/yalm_hip.h, "layer-list models"):
 // a decoder whose layers each name their token mixer (latent attention, real-gated linear
 // recurrence, gated delta rule, softmax attention with a window or chunk mask, selective
-// state-space layer, matrix memory with exponential gates, or two of them side by side) and
+// state-space layer, matrix memory with exponential gates, gated linear attention, or two of them side by side) and
 // feed-forward (dense GLU, routed experts, plain), holding one sequence's latent and
 // key / value caches and recurrent / convolution states in HBM. One step function
 // serves whole prompts, portions of prompts and single decoded tokens; the device greedy
@@ -48,6 +48,11 @@ struct yalm_seq_s {
 	float *Y3 = nullptr;         // the result of a layer's second mixer (side) before the two are joined
 	float *Yout = nullptr;       // where the mixer being enqueued leaves its result: Y, or Y3
 	const float *embed_norm = nullptr;
+	// token-pair embedding: the table, the token before the next one (-1: none) as the host knows it and,
+	// during a greedy loop, on the device; q->tok[-1] is the token before the portion's first
+	const void *bigram = nullptr;
+	int host_prev = -1;
+	int *prev = nullptr;
 	std::vector<int> side_of;    // per layer: index in L of its second mixer, or -1 (sides follow the n_layers entries)
 	std::vector<float *> rel_dist; // attn with a distance bias: [rel_far + 1][heads], the bucketed table per distance
 	std::vector<int> rel_far;
@@ -119,7 +124,8 @@ static int in_rows(const yalm_seq_layer &l) {
 	switch (l.mixer) {
 	case YALM_MIX_LATENT:
 		if (l.q_rank == 0)
-			return l.heads * (l.dim + l.rot_dim) + l.kv_rank + l.rot_dim;
+			return l.heads * (l.dim + l.rot_dim) + (l.kv_from < 0 ? l.kv_rank + l.rot_dim : 0) +
+			       (l.out_gate == 2 ? l.heads * l.vdim : 0);
 		return l.q_rank + (l.kv_from < 0 ? l.kv_rank : 0);
 	case YALM_MIX_RGLRU: return 2 * l.rec_width;
 	case YALM_MIX_ATTN:
@@ -127,6 +133,7 @@ static int in_rows(const yalm_seq_layer &l) {
 		       (l.out_gate == 2 ? l.heads * l.vdim : (l.out_gate ? l.heads : 0));
 	case YALM_MIX_SSM: return 2 * l.heads * l.vdim + 2 * l.ssm_groups * l.ssm_state + l.heads;
 	case YALM_MIX_MEMORY: return 2 * l.heads * (l.dim + l.vdim + 1);
+	case YALM_MIX_GLA: return 2 * l.heads * (l.dim + l.vdim) + l.decay_rank;
 	default:
 		return 2 * l.kv_heads * l.dim + l.heads * l.vdim + (l.gate_rank > 0 ? l.gate_rank : l.heads * l.vdim) + l.heads +
 		       (l.decay_rank > 0 ? l.decay_rank : l.heads);
@@ -156,11 +163,16 @@ static size_t memory_state(const yalm_seq_layer &l) {
 static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> &L) {
 	ARGCHK(c.width > 0 && c.vocab > 0 && c.n_layers > 0 && c.max_tokens > 0, "yalm_seq_create: bad model sizes");
 	ARGCHK(c.weight_dtype == YALM_BF16 || c.weight_dtype == YALM_F32, "yalm_seq_create: weight_dtype must be bf16 or f32");
-	ARGCHK(c.norm_kind == YALM_NORM_RMS || c.norm_kind == YALM_NORM_LAYER || c.norm_kind == YALM_NORM_TANH,
+	ARGCHK(c.norm_kind == YALM_NORM_RMS || c.norm_kind == YALM_NORM_LAYER || c.norm_kind == YALM_NORM_TANH ||
+	           c.norm_kind == YALM_NORM_LAYER_BIAS,
 	       "yalm_seq_create: unknown norm kind");
 	ARGCHK(c.logit_softcap >= 0.0f, "yalm_seq_create: bad logit cap");
-	ARGCHK(c.block_kind == YALM_BLOCK_SERIAL || (c.block_kind == YALM_BLOCK_PARALLEL && c.pre_norm),
-	       "yalm_seq_create: blocks are serial, or parallel with pre_norm");
+	ARGCHK(c.block_kind == YALM_BLOCK_SERIAL || (c.block_kind == YALM_BLOCK_PARALLEL && c.pre_norm) ||
+	           (c.block_kind == YALM_BLOCK_POST && !c.pre_norm),
+	       "yalm_seq_create: blocks are serial, parallel with pre_norm, or post-norm without");
+	ARGCHK(c.bigram_buckets >= 0 && c.bigram_mul_prev >= 0 && c.bigram_mul_cur >= 0 &&
+	           (c.bigram_buckets == 0 || (c.bigram_mul_prev <= (1LL << 61) / c.vocab && c.bigram_mul_cur <= (1LL << 61) / c.vocab)),
+	       "yalm_seq_create: bad token-pair table constants");
 	const bool par = c.block_kind == YALM_BLOCK_PARALLEL;
 	std::vector<int> owner; // of each second mixer: the layer it stands beside
 	for (int i = 0; i < c.n_layers; ++i)
@@ -188,13 +200,17 @@ static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> 
 		       at + "unknown feed-forward activation (clamp and silu belong to gated pairs, relu^2 and the exact gelu to ungated ones)");
 		ARGCHK(!l.pre_add || i == 0 || par, at + "a vector added before an entry after the first needs parallel blocks");
 		if (latent_direct(l)) {
-			ARGCHK(l.heads > 0 && l.dim > 0 && l.vdim > 0 && l.kv_rank > 0 && l.rot_dim >= 0 && l.kv_from < 0,
-			       at + "bad latent attention sizes");
+			ARGCHK(l.heads > 0 && l.dim > 0 && l.vdim > 0 && l.kv_rank > 0 && l.rot_dim >= 0, at + "bad latent attention sizes");
+			ARGCHK(l.kv_from < 0 || (!is_side && l.kv_from < i && latent_direct(L[l.kv_from]) && L[l.kv_from].kv_from < 0 &&
+			                         L[l.kv_from].kv_rank == l.kv_rank && L[l.kv_from].rot_dim == l.rot_dim),
+			       at + "kv_from must name an earlier latent attention layer with its own latent of the same rank and rot_dim");
+			ARGCHK((l.rot_pairs == YALM_ROT_INTERLEAVED || l.rot_pairs == YALM_ROT_HALVES) && (l.out_gate == 0 || l.out_gate == 2),
+			       at + "unknown rotary layout or output gate");
 			if ((size_t)l.heads * ((l.kv_rank + 3) / 4) > (size_t)SA_MAX_NA4 * SEQ_THREADS) {
 				set_err(at + "heads x kv_rank above 16384 is not implemented by the attention kernels");
 				return YALM_ERR_UNSUPPORTED;
 			}
-			ARGCHK(l.kv_norm && l.w_ukt && (l.w_uv || l.w_ukv), at + "missing latent attention tensors");
+			ARGCHK((l.kv_norm || l.kv_from >= 0) && l.w_ukt && (l.w_uv || l.w_ukv), at + "missing latent attention tensors");
 			ARGCHK(l.mask_kind == YALM_MASK_CAUSAL || ((l.mask_kind == YALM_MASK_WINDOW || l.mask_kind == YALM_MASK_CHUNK) && l.mask_size > 0),
 			       at + "bad attention mask");
 			ARGCHK(l.rot_dims >= 0 && l.rot_dims <= l.rot_dim && l.rot_dims % 2 == 0 && (l.rot_dims == 0 || l.rot_base > 0.0f),
@@ -251,6 +267,15 @@ static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> 
 				return YALM_ERR_UNSUPPORTED;
 			}
 			ARGCHK(l.out_norm, at + "missing matrix memory tensors");
+		} else if (l.mixer == YALM_MIX_GLA) {
+			ARGCHK(l.heads > 0 && l.dim > 0 && l.vdim > 0 && l.decay_rank > 0 && l.decay_tau > 0.0f &&
+			           (l.gate_act == YALM_GATE_SILU || l.gate_act == YALM_GATE_SIGMOID),
+			       at + "bad gated linear attention sizes");
+			if (l.dim > 256) {
+				set_err(at + "dim above 256 is not implemented by the recurrence kernel");
+				return YALM_ERR_UNSUPPORTED;
+			}
+			ARGCHK(l.w_a2 && l.dt_bias && l.out_norm, at + "missing gated linear attention tensors");
 		} else if (l.mixer == YALM_MIX_ATTN) {
 			ARGCHK(l.heads > 0 && l.kv_heads > 0 && l.heads % l.kv_heads == 0 && l.dim > 0 && l.vdim > 0,
 			       at + "bad attention sizes");
@@ -288,10 +313,13 @@ static int validate(const yalm_seq_config &c, const std::vector<yalm_seq_layer> 
 			           l.groups_keep <= l.groups && l.top <= l.groups_keep * (l.experts / l.groups) + l.identity,
 			       at + "bad router sizes");
 			ARGCHK(l.router_kind == YALM_ROUTER_SOFTMAX_TOP || l.router_kind == YALM_ROUTER_SIGMOID_GROUPS ||
-			           ((l.router_kind == YALM_ROUTER_TOP_SOFTMAX || l.router_kind == YALM_ROUTER_SOFTMAX_NORMED) && l.groups == 1),
+			           ((l.router_kind == YALM_ROUTER_TOP_SOFTMAX || l.router_kind == YALM_ROUTER_SOFTMAX_NORMED ||
+			             l.router_kind == YALM_ROUTER_SIGMOID_TOP) &&
+			            l.groups == 1),
 			       at + "unknown router kind (groups belong to the first and third only)");
 			ARGCHK(l.identity >= 0 && (l.identity == 0 || (l.router_kind == YALM_ROUTER_SOFTMAX_NORMED && c.pre_norm)),
 			       at + "identity outputs belong to the softmax router with renormalised weights, in blocks with opening norms");
+			ARGCHK(!l.expert_in_weighted || l.identity == 0, at + "weights on the experts' inputs leave no place for identity outputs");
 			ARGCHK(l.router && l.w_up && l.w_down && (par || ((l.norm2 || !c.pre_norm) && l.norm2b)), at + "missing expert tensors");
 			if (l.shared_ff > 0)
 				ARGCHK((l.ws_gate || !l.w_gate) && l.ws_up && l.ws_down, at + "missing shared expert tensors");
@@ -407,10 +435,15 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 			q->L.push_back(*q->L[i].side);
 		}
 	q->embed_norm = w->embed_norm;
+	q->bigram = w->bigram;
 	q->embed = w->embed;
 	q->head = w->head;
 	q->final_norm = w->final_norm;
 	int rc = validate(q->c, q->L);
+	if (rc == YALM_OK && q->c.bigram_buckets > 0 && !q->bigram) {
+		set_err("yalm_seq_create: the token-pair table is missing");
+		rc = YALM_ERR_ARG;
+	}
 	if (rc != YALM_OK) {
 		delete q;
 		return rc;
@@ -455,6 +488,9 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 		} else if (l.mixer == YALM_MIX_MEMORY) {
 			bw = std::max(bw, (size_t)l.heads * (l.vdim + 1));
 			arena += memory_state(l);
+		} else if (l.mixer == YALM_MIX_GLA) {
+			bw = std::max({bw, (size_t)l.heads * l.dim, (size_t)l.heads * l.vdim});
+			arena += (size_t)l.heads * l.dim * l.vdim;
 		} else if (l.mixer == YALM_MIX_SSM) {
 			const size_t cc = (size_t)l.heads * l.vdim + 2 * (size_t)l.ssm_groups * l.ssm_state;
 			bw = std::max({bw, cc, (size_t)2 * l.heads});
@@ -499,7 +535,9 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 		STRY(sallocT(q, &q->B[i], cap * bw));
 	if (bf && pf_gemm_bf16)
 		STRY(sallocT(q, &q->a16, cap * bw));
-	STRY(sallocT(q, &q->tok, cap));
+	STRY(sallocT(q, &q->tok, cap + 1));
+	q->tok += 1; // [-1]: the token before the portion's first
+	STRY(sallocT(q, &q->prev, 1));
 	STRY(sallocT(q, &q->want, cap));
 	STRY(sallocT(q, &q->logits, (size_t)LOGIT_ROWS * c.vocab));
 	STRY(sallocT(q, &q->idx, cap * max_top));
@@ -562,7 +600,10 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 	for (int i = 0; i < NL; ++i) {
 		const yalm_seq_layer &l = q->L[i];
 		if (latent_direct(l)) {
-			STRY(salloc(q, &q->cache[i], (size_t)c.max_tokens * (l.kv_rank + l.rot_dim) * (bf ? 2 : 4)));
+			if (l.kv_from < 0)
+				STRY(salloc(q, &q->cache[i], (size_t)c.max_tokens * (l.kv_rank + l.rot_dim) * (bf ? 2 : 4)));
+			else
+				q->cache[i] = q->cache[l.kv_from]; // an earlier entry
 			q->vcache[i] = q->cache[i];
 			STRY(attn_setup(q, i));
 		} else if (l.mixer == YALM_MIX_LATENT) {
@@ -582,6 +623,9 @@ static int create_seq(const yalm_seq_config *config, const yalm_seq_weights *w, 
 		} else if (l.mixer == YALM_MIX_MEMORY) {
 			q->S[i] = q->arena + off;
 			off += memory_state(l);
+		} else if (l.mixer == YALM_MIX_GLA) {
+			q->S[i] = q->arena + off;
+			off += (size_t)l.heads * l.dim * l.vdim;
 		} else if (l.mixer == YALM_MIX_SSM) {
 			const size_t cc = (size_t)l.heads * l.vdim + 2 * (size_t)l.ssm_groups * l.ssm_state;
 			q->S[i] = q->arena + off;
@@ -647,6 +691,7 @@ extern "C" int yalm_seq_reset(yalm_seq q) {
 		HIPCHK(hipGetLastError());
 	}
 	q->host_pos = 0;
+	q->host_prev = -1;
 	return YALM_OK;
 }
 
@@ -692,7 +737,7 @@ static int gemm(Seq *q, const GemmArgs &a, int batches = 1, int max_m = -1, bool
 	const bool pair = a.W2 != nullptr && (a.epi == EPI_GLU_GELU || a.epi == EPI_GLU_CLAMP || a.epi == EPI_GLU_SILU) && !a.bias;
 	const bool single = !a.W2 && (a.epi == EPI_NONE || a.epi == EPI_GELU || a.epi == EPI_RELU2 || a.epi == EPI_GELU_ERF);
 	const int act1 = a.epi == EPI_GELU ? 1 : (a.epi == EPI_RELU2 ? 2 : (a.epi == EPI_GELU_ERF ? 3 : 0)); // the large-tile door's activation
-	if (q->a16 && batches == 1 && max_m >= 2 * GB_BM && !a.rows && !a.w_sel && a.z_split == 0 && a.ldw == a.K &&
+	if (q->a16 && batches == 1 && max_m >= 2 * GB_BM && !a.rows && !a.row_scale && !a.gate && !a.w_sel && a.z_split == 0 && a.ldw == a.K &&
 	    a.K % 64 == 0 && (pair ? a.N % 64 == 0 : (single && a.N >= 128))) {
 		const size_t n8 = (size_t)a.M * (a.K / 8);
 		seq_to_bf16_kernel<<<(unsigned)std::min<size_t>((n8 + SEQ_THREADS - 1) / SEQ_THREADS, 4096), SEQ_THREADS, 0,
@@ -846,9 +891,10 @@ static int mixer_rglru(Seq *q, int li, int n) {
 }
 
 // The recurrence kernel over a portion: the gated delta rule (gv: one decay per head and key
-// channel), the state-space walk, or the matrix memory (mg: its log gates; scale: on the read-outs).
+// channel), the state-space walk, the matrix memory (mg: its log gates; scale: on the read-outs), or
+// gated linear attention (gv: its decays; mg.scale: on the read-outs).
 // K: key / state size, P: value size (the matrix memory's state has one column more).
-enum { WALK_DELTA, WALK_SSM, WALK_MEMORY };
+enum { WALK_DELTA, WALK_SSM, WALK_MEMORY, WALK_GLA };
 struct MemGates {
 	const float *lg; // log gates (or their logits, cap > 0) [t][ld]: input gates, then forget gates
 	int ld;
@@ -865,6 +911,9 @@ static int delta_launch(Seq *q, const float *qkv, int ldq, int qo, int ko, int v
 			seq_delta_kernel<RR, TC, true, false, LPC, true><<<g, SEQ_THREADS, 0, q->stream>>>(                        \
 			    qkv, ldq, qo, ko, vo, KH, K, H, P, nullptr, nullptr, nullptr, state, o, n, mg.lg, mg.ld, mg.cap,       \
 			    mg.scale, mg.running);                                                                                 \
+		else if (walk == WALK_GLA)                                                                                     \
+			seq_delta_kernel<RR, TC, true, true, LPC><<<g, SEQ_THREADS, 0, q->stream>>>(                               \
+			    qkv, ldq, qo, ko, vo, KH, K, H, P, nullptr, gv, nullptr, state, o, n, nullptr, 0, 0.0f, mg.scale);     \
 		else if (walk == WALK_SSM)                                                                                     \
 			seq_delta_kernel<RR, TC, true, false, LPC><<<g, SEQ_THREADS, 0, q->stream>>>(                              \
 			    qkv, ldq, qo, ko, vo, KH, K, H, P, bg, nullptr, dskip, state, o, n);                                   \
@@ -964,11 +1013,35 @@ static int mixer_memory(Seq *q, int li, int n) {
 	return gemm(q, plain(on, HV, l.w_o, HV, q->Yout, c.width, n, c.width, HV));
 }
 
+// Gated linear attention: one input projection (queries, keys, values, output gate, decay rows), the
+// low-rank decays' second factor with the root of the sigmoid as its epilogue, the recurrence kernel on
+// the projection's own rows, the read-outs normed per head and gated, the output projection.
+static int mixer_gla(Seq *q, int li, int n) {
+	const yalm_seq_layer &l = q->L[li];
+	const yalm_seq_config &c = q->c;
+	const int H = l.heads, D = l.dim, V = l.vdim, zin = in_rows(l), HD = H * D, HV = H * V;
+	const int gcol = 2 * HD + HV, acol = gcol + HV;
+	float *gv = q->B[0], *o = q->B[1], *on = q->B[2];
+	TRY(gemm(q, plain(q->In, c.width, l.w_in, c.width, q->Z, zin, n, zin, c.width)));
+	GemmArgs a = plain(q->Z + acol, zin, l.w_a2, l.decay_rank, gv, HD, n, HD, l.decay_rank);
+	a.bias = l.dt_bias;
+	a.epi = EPI_SIG_ROOT;
+	a.limit = l.decay_tau;
+	TRY(gemm(q, a));
+	MemGates mg{};
+	mg.scale = 1.0f / std::sqrt((float)D);
+	TRY(delta_launch(q, q->Z, zin, 0, HD, 2 * HD, H, D, H, V, nullptr, gv, nullptr, q->S[li], o, n, WALK_GLA, mg));
+	seq_delta_out_kernel<<<n, SEQ_THREADS, 0, q->stream>>>(o, H, V, l.out_norm, c.norm_eps, q->Z, zin, gcol, on,
+	                                                       l.gate_act == YALM_GATE_SIGMOID);
+	HIPCHK(hipGetLastError());
+	return gemm(q, plain(on, HV, l.w_o, HV, q->Yout, c.width, n, c.width, HV));
+}
+
 // ---- the closing norm of a single token, owed to the product that reads the stream next
 static int add_norm(Seq *q, const float *wb, const float *w_next, int n, const yalm_seq_layer *moe);
 
 static bool an_foldable(const Seq *q, int n) {
-	return n == 1 && !q->c.pre_norm && q->nk != NK_TANH && !q->dump_on && q->Xalt && q->c.width % 8 == 0 && q->c.width <= 8 * 1024;
+	return n == 1 && !q->c.pre_norm && q->c.block_kind == YALM_BLOCK_SERIAL && q->nk != NK_TANH && !q->dump_on && q->Xalt && q->c.width % 8 == 0 && q->c.width <= 8 * 1024;
 }
 static int flush_norm(Seq *q, int n) {
 	if (!q->pend_wb)
@@ -1206,7 +1279,7 @@ static int mixer_attn(Seq *q, int li, int n) {
 }
 
 // Latent attention with directly projected queries, a rotated key part shared by all heads, a
-// mask and a sink. With k_j = W_uk c_j and v_j = W_uv c_j: q.k_j = (W_uk^T q).c_j and sum_j p_j
+// mask, a sink and an elementwise output gate; kv_from: the cache rows are another layer's. With k_j = W_uk c_j and v_j = W_uv c_j: q.k_j = (W_uk^T q).c_j and sum_j p_j
 // v_j = W_uv sum_j p_j c_j, so head h attends with the query [W_uk[h]^T q_plain | q_rot] over
 // the cache rows [c_j | k_rot_j] themselves and sums their first kv_rank entries: the softmax-
 // attention kernels with one key/value head, key size kv_rank + rot_dim, value size kv_rank,
@@ -1237,15 +1310,17 @@ static int mixer_latent_direct(Seq *q, int li, int n) {
 	const bool expand = l.w_ukv && n > 1 && rows <= q->ex_rows && (n >= 32 || !absorbed_ok);
 	TRY(gemm(q, plain(q->In, c.width, l.w_in, c.width, q->Z, zin, n, zin, c.width)));
 	const size_t rot_lds = (size_t)std::max(l.rot_dims, 2) * sizeof(float);
+	const float *kv_w = l.kv_from < 0 ? l.kv_norm : nullptr; // another layer's cache rows: queries (and gate) only
+	const float *ge = l.out_gate == 2 ? q->Z + (zin - H * V) : nullptr; // elementwise gate logits close the projection
 	const dim3 pg(n, n <= GEMV_MAX_M ? 4 : 1); // a few tokens: each token's work spread over four workgroups
 	if (bf)
 		seq_latent_prep_kernel<uint16_t><<<pg, SEQ_THREADS, rot_lds, q->stream>>>(
-		    q->Z, zin, H, D, R, rk, l.rot_dims, q->rot_freq[li], l.kv_norm, c.norm_eps, l.attn_scale, q->st, qp, qa,
-		    (uint16_t *)q->cache[li], (int)expand);
+		    q->Z, zin, H, D, R, rk, l.rot_dims, q->rot_freq[li], kv_w, c.norm_eps, l.attn_scale, q->st, qp, qa,
+		    (uint16_t *)q->cache[li], (int)expand, l.rot_pairs == YALM_ROT_HALVES);
 	else
 		seq_latent_prep_kernel<float><<<pg, SEQ_THREADS, rot_lds, q->stream>>>(
-		    q->Z, zin, H, D, R, rk, l.rot_dims, q->rot_freq[li], l.kv_norm, c.norm_eps, l.attn_scale, q->st, qp, qa,
-		    (float *)q->cache[li], (int)expand);
+		    q->Z, zin, H, D, R, rk, l.rot_dims, q->rot_freq[li], kv_w, c.norm_eps, l.attn_scale, q->st, qp, qa,
+		    (float *)q->cache[li], (int)expand, l.rot_pairs == YALM_ROT_HALVES);
 	HIPCHK(hipGetLastError());
 	AttnArgs a;
 	a.H = H;
@@ -1293,8 +1368,8 @@ static int mixer_latent_direct(Seq *q, int li, int n) {
 		const size_t eb = bf ? 2 : 4;
 		const void *kc = (const char *)q->ex_k - (size_t)klo * a.KL * eb;
 		const void *vc = (const char *)q->ex_v - (size_t)klo * a.VL * eb;
-		TRY(bf ? attn_core_t<uint16_t>(q, li, n, a, qa, nullptr, oh, kc, vc)
-		       : attn_core_t<float>(q, li, n, a, qa, nullptr, oh, kc, vc));
+		TRY(bf ? attn_core_t<uint16_t>(q, li, n, a, qa, nullptr, oh, kc, vc, ge, zin)
+		       : attn_core_t<float>(q, li, n, a, qa, nullptr, oh, kc, vc, ge, zin));
 	} else {
 		{ // columns [0, kv_rank) of head h's query: W_uk[h]^T q_plain[h], per head [n][dim] x [rank][dim]^T
 			GemmArgs g = plain(qp, H * D, l.w_ukt, D, qa, H * KR, n, rk, D);
@@ -1314,6 +1389,9 @@ static int mixer_latent_direct(Seq *q, int li, int n) {
 			b.a_bs = rk;
 			b.w_bs = (long)V * rk;
 			b.c_bs = V;
+			b.gate = ge;
+			b.ldgate = zin;
+			b.gate_bs = V;
 			TRY(gemm(q, b, H));
 		}
 	}
@@ -1367,9 +1445,10 @@ static int ff_moe(Seq *q, int li, int n) {
 	const yalm_seq_config &c = q->c;
 	const int E = l.experts, ER = E + l.identity, top = l.top, ff = l.ff, slots = n * top;
 	float *hx = q->B[0], *yx = q->B[1], *hs = q->B[2], *ys = q->B[3];
-	// the renormalised softmax router's choice is one wave's work: more waves for its logits
-	auto router = l.router_kind == YALM_ROUTER_SOFTMAX_NORMED ? seq_router_kernel<1024> : seq_router_kernel<SEQ_THREADS>;
-	const int rth = l.router_kind == YALM_ROUTER_SOFTMAX_NORMED ? 1024 : SEQ_THREADS;
+	// a choice that is one wave's work: more waves for the logits
+	const bool one_wave = l.router_kind == YALM_ROUTER_SOFTMAX_NORMED || l.router_kind == YALM_ROUTER_SIGMOID_TOP;
+	auto router = one_wave ? seq_router_kernel<1024> : seq_router_kernel<SEQ_THREADS>;
+	const int rth = one_wave ? 1024 : SEQ_THREADS;
 	router<<<n, rth, (2 * ER + l.groups) * sizeof(float), q->stream>>>(q->In, c.width, l.router, ER, top, l.groups,
 	                                                                    l.groups_keep, l.router_scale,
 	                                                                    l.shared_ff > 0 ? l.shared_sg : nullptr, q->idx,
@@ -1392,6 +1471,10 @@ static int ff_moe(Seq *q, int li, int n) {
 		a.c_bs = ff;
 		a.epi = epi;
 		a.limit = l.limit;
+		if (l.expert_in_weighted) { // batch z is slot z
+			a.row_scale = q->wt;
+			a.row_scale_bs = 1;
+		}
 		GemmArgs b = plain(hx, ff, l.w_down, ff, yx, c.width, 1, c.width, ff);
 		b.a_bs = ff;
 		b.w_sel = q->idx;
@@ -1429,6 +1512,7 @@ static int ff_moe(Seq *q, int li, int n) {
 		a.a_div = top;
 		a.epi = epi;
 		a.limit = l.limit;
+		a.row_scale = l.expert_in_weighted ? q->wt : nullptr; // result rows are slots
 		TRY(gemm(q, a, E, n));
 		GemmArgs b = plain(hx, ff, l.w_down, ff, yx, c.width, n, c.width, ff);
 		b.w_bs = (long)c.width * ff;
@@ -1448,6 +1532,11 @@ static int ff_moe(Seq *q, int li, int n) {
 	return YALM_OK; // the combine of yx (B[1]) and ys (B[3]) happens in the closing norm's launch (add_norm, par_close)
 }
 
+// The weights of the experts' combine; none where they have been applied to the experts' inputs.
+static const float *combine_wt(const Seq *q, const yalm_seq_layer &l) {
+	return l.expert_in_weighted ? nullptr : q->wt;
+}
+
 // The seam after a parallel block: both sublayers' results join the stream (the experts' combine
 // happens here), the next entry's pre_add and opening norm follow in the same launch.
 static int par_close(Seq *q, int li, int n) {
@@ -1459,7 +1548,7 @@ static int par_close(Seq *q, int li, int n) {
 	const bool joined = q->side_of[li] >= 0; // two mixers side by side: their normed results meet in this launch
 	float *dump = q->dump_on && q->dump ? q->dump + (size_t)li * n * c.width : nullptr;
 #define PC_ARGS                                                                                                        \
-	q->X, q->Y, l.ls1, (l.ff_kind != YALM_FF_NONE && !moe) ? q->Y2 : nullptr, l.ls2, moe ? q->B[1] : nullptr, q->wt,    \
+	q->X, q->Y, l.ls1, (l.ff_kind != YALM_FF_NONE && !moe) ? q->Y2 : nullptr, l.ls2, moe ? q->B[1] : nullptr, combine_wt(q, l),    \
 	    moe ? l.top : 0, moe && l.shared_ff > 0 ? q->B[3] : nullptr, gated ? q->sgate : nullptr, dump,                 \
 	    nx ? nx->pre_add : nullptr, c.norm_eps, c.width, nx ? nx->norm1 : nullptr, q->Hn, q->nk, c.residual_scale,                  \
 	    (nx && nx->ff_kind != YALM_FF_NONE) ? nx->norm2 : nullptr, q->Hn2, joined ? q->Y3 : nullptr, l.join_w,        \
@@ -1481,6 +1570,27 @@ static int par_close(Seq *q, int li, int n) {
 	return YALM_OK;
 }
 
+// The seam after a sublayer of a post-norm block; moe as in add_norm.
+static int post_close(Seq *q, const float *wb, int n, const yalm_seq_layer *moe) {
+	const yalm_seq_config &c = q->c;
+	const int w = c.width;
+#define PO_ARGS                                                                                                        \
+	q->X, q->Y, moe ? q->B[1] : nullptr, moe ? combine_wt(q, *moe) : nullptr, moe ? moe->top : 0,                      \
+	    moe && moe->shared_ff > 0 ? q->B[3] : nullptr, moe && moe->shared_ff > 0 && moe->shared_sg ? q->sgate : nullptr, wb, \
+	    c.norm_eps, w, q->nk, c.stream_scale, c.residual_scale
+	if (w <= 4 * SEQ_THREADS)
+		seq_post_close_reg_kernel<4><<<n, SEQ_THREADS, 0, q->stream>>>(PO_ARGS);
+	else if (w <= 8 * SEQ_THREADS)
+		seq_post_close_reg_kernel<8><<<n, SEQ_THREADS, 0, q->stream>>>(PO_ARGS);
+	else if (w <= 16 * SEQ_THREADS)
+		seq_post_close_reg_kernel<16><<<n, SEQ_THREADS, 0, q->stream>>>(PO_ARGS);
+	else
+		seq_post_close_kernel<<<n, SEQ_THREADS, (size_t)w * sizeof(float), q->stream>>>(PO_ARGS);
+#undef PO_ARGS
+	HIPCHK(hipGetLastError());
+	return YALM_OK;
+}
+
 // moe: the layer's routed experts feed the norm (their combine happens inside it) instead of Y
 static int add_norm(Seq *q, const float *wb, const float *w_next, int n, const yalm_seq_layer *moe) {
 	const int w = q->c.width;
@@ -1493,7 +1603,8 @@ static int add_norm(Seq *q, const float *wb, const float *w_next, int n, const y
 #undef AN_LAUNCH
 	} else {
 		seq_add_norm_kernel<<<n, SEQ_THREADS, w * sizeof(float), q->stream>>>(
-		    q->X, q->Y, wb, q->c.norm_eps, w, w_next, q->Hn, moe ? q->B[1] : nullptr, q->wt, moe ? moe->top : 0,
+		    q->X, q->Y, wb, q->c.norm_eps, w, w_next, q->Hn, moe ? q->B[1] : nullptr,
+		    moe ? combine_wt(q, *moe) : nullptr, moe ? moe->top : 0,
 		    moe && moe->shared_ff > 0 ? q->B[3] : nullptr, moe && moe->shared_sg ? q->sgate : nullptr, q->nk,
 		    q->c.residual_scale, q->idx, moe ? moe->experts : 0, moe && moe->identity > 0 ? q->In : nullptr);
 	}
@@ -1519,23 +1630,29 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 	const bool fold = an_foldable(q, n);
 	// the closing norm of a sublayer: applied now, or owed to the product that reads the stream next
 	auto close = [&](const float *wb, const float *w_next, const yalm_seq_layer *moe) {
+		if (c.block_kind == YALM_BLOCK_POST)
+			return post_close(q, wb, n, moe);
 		if (fold && !moe && !w_next) {
 			q->pend_wb = wb;
 			return (int)YALM_OK;
 		}
 		return add_norm(q, wb, w_next, n, moe);
 	};
-	const int eb = q->nk == NK_TANH && !q->embed_norm ? cdiv(c.width, SEQ_THREADS) : 1; // no row statistics: elementwise
+	Bigram bg;
+	if (c.bigram_buckets > 0)
+		bg = Bigram{q->bigram, c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur, q->prev};
+	// no row statistics: elementwise (in the greedy loop the one workgroup that also passes the previous token on)
+	const int eb = q->nk == NK_TANH && !q->embed_norm && (tokens_dev || !bg.table) ? cdiv(c.width, SEQ_THREADS) : 1;
 	if (c.weight_dtype == YALM_F32)
 		seq_embed_kernel<WF32><<<dim3(n, eb), SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
 		                                                         c.vocab, c.embed_scale, q->X, first_norm, c.norm_eps,
 		                                                         q->Hn, q->nk, q->L[0].pre_add, q->embed_norm, first_norm2,
-		                                                         q->Hn2);
+		                                                         q->Hn2, bg);
 	else
 		seq_embed_kernel<WBF16><<<dim3(n, eb), SEQ_THREADS, 0, q->stream>>>(q->st, tokens_dev, q->embed, q->inv_freq, c.width,
 		                                                          c.vocab, c.embed_scale, q->X, first_norm, c.norm_eps,
 		                                                          q->Hn, q->nk, q->L[0].pre_add, q->embed_norm, first_norm2,
-		                                                          q->Hn2);
+		                                                          q->Hn2, bg);
 	HIPCHK(hipGetLastError());
 	auto run_mixer = [&](int mi) {
 		const yalm_seq_layer &m = q->L[mi];
@@ -1551,6 +1668,8 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 			return mixer_ssm(q, mi, n);
 		if (m.mixer == YALM_MIX_MEMORY)
 			return mixer_memory(q, mi, n);
+		if (m.mixer == YALM_MIX_GLA)
+			return mixer_gla(q, mi, n);
 		return mixer_delta(q, mi, n);
 	};
 	for (int li = 0; li < c.n_layers; ++li) {
@@ -1646,6 +1765,8 @@ extern "C" int yalm_seq_step(yalm_seq q, const int *tokens, int n, const int *wa
 		const int m = std::min(q->cap, n - t0);
 		HIPCHK(hipMemcpyAsync(q->tok, tokens + t0, (size_t)m * sizeof(int), hipMemcpyHostToDevice, q->stream));
 		set_step_kernel<<<1, 1, 0, q->stream>>>(q->st, 0, q->host_pos, 0);
+		if (q->bigram)
+			seq_fill_int_kernel<<<1, 1, 0, q->stream>>>(q->tok - 1, 1, q->host_prev);
 		HIPCHK(hipGetLastError());
 		q->cur_pos = q->host_pos;
 		if (q->dump_on) {
@@ -1655,6 +1776,7 @@ extern "C" int yalm_seq_step(yalm_seq q, const int *tokens, int n, const int *wa
 		}
 		TRY(enqueue_portion(q, q->tok, m));
 		q->host_pos += m;
+		q->host_prev = std::max(tokens[t0 + m - 1], 0);
 		int w1 = wi;
 		while (w1 < n_want && want[w1] < t0 + m)
 			++w1;
@@ -1709,6 +1831,8 @@ extern "C" int yalm_seq_generate_greedy(yalm_seq q, int token, int n_steps, int 
 		TRY(ensure_greedy_graph(q));
 	set_step_kernel<<<1, 1, 0, q->stream>>>(q->st, token, q->host_pos, 1);
 	seq_fill_int_kernel<<<1, 1, 0, q->stream>>>(q->want, 1, 0);
+	if (q->bigram)
+		seq_fill_int_kernel<<<1, 1, 0, q->stream>>>(q->prev, 1, q->host_prev);
 	HIPCHK(hipGetLastError());
 	for (int i = 0; i < n_steps; ++i) {
 		if (graph)
@@ -1719,6 +1843,7 @@ extern "C" int yalm_seq_generate_greedy(yalm_seq q, int token, int n_steps, int 
 	HIPCHK(hipMemcpyAsync(out_tokens, q->gen_tokens, (size_t)n_steps * sizeof(int), hipMemcpyDeviceToHost, q->stream));
 	HIPCHK(hipStreamSynchronize(q->stream));
 	q->host_pos += n_steps;
+	q->host_prev = n_steps > 1 ? out_tokens[n_steps - 2] : token; // the last token fed
 	return YALM_OK;
 }
 
@@ -1745,6 +1870,8 @@ extern "C" int yalm_seq_time_step(yalm_seq q, int n, int pos0, int iters, float 
 		tk[i] = (int)(((unsigned)i * 2654435761u) % (unsigned)q->c.vocab);
 	HIPCHK(hipMemcpy(q->tok, tk.data(), (size_t)n * sizeof(int), hipMemcpyHostToDevice));
 	seq_fill_int_kernel<<<1, 1, 0, q->stream>>>(q->want, 1, n - 1);
+	if (q->bigram)
+		seq_fill_int_kernel<<<1, 1, 0, q->stream>>>(q->tok - 1, 1, pos0 > 0 ? 0 : -1);
 	hipEvent_t e0, e1;
 	HIPCHK(hipEventCreate(&e0));
 	HIPCHK(hipEventCreate(&e1));

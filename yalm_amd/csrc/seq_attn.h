@@ -279,8 +279,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_attn_prep_kernel(const float 
 // which fills columns [0, rank) of Qa) and its rotated part, rotated and scaled, in columns
 // [rank, rank + R) of Qa [t][H][rank + R]: the attention kernels then see H independent heads
 // over ONE key/value head whose key row is the cache row and whose value is its first rank
-// entries. Rotation: the first rot_dims <= R entries in interleaved pairs, as in
-// seq_attn_prep_kernel. expanded != 0 (the portion attends over expanded per-head keys and
+// entries. Rotation: the first rot_dims <= R entries in interleaved or (rot_half) half-split pairs, as in
+// seq_attn_prep_kernel. kv_w == nullptr: the token's cache row is another layer's; Z holds the queries only. expanded != 0 (the portion attends over expanded per-head keys and
 // values, seq_latent_expand_kernel): Qp is not written and Qa is [t][H][D + R], head h's
 // scaled plain part followed by its rotated part. The workgroups of a token (gridDim.y) share its
 // outputs (each works the rotation table and the latent's rms out for itself). Dynamic LDS:
@@ -292,7 +292,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_latent_prep_kernel(const floa
                                                                       const float *__restrict__ kv_w, float eps,
                                                                       float scale, const StepState *__restrict__ st,
                                                                       float *__restrict__ Qp, float *__restrict__ Qa,
-                                                                      CT *__restrict__ cache, int expanded) {
+                                                                      CT *__restrict__ cache, int expanded,
+                                                                      int rot_half = 0) {
 	extern __shared__ float rot[];
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x, tid = threadIdx.x;
@@ -309,22 +310,27 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_latent_prep_kernel(const floa
 	const int QH = D + R, QN = H * QH, KR = rank + R;
 	const float *z = Z + (size_t)t * ldz;
 	const float *lat = z + QN;
-	float ss = 0.0f;
-	for (int i = tid; i < rank; i += SEQ_THREADS)
-		ss = fmaf(lat[i], lat[i], ss);
-	const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)rank + eps); // also orders rot[] before its readers
 	CT *crow = cache + (size_t)p * KR;
-	for (int i = i0; i < rank; i += istep)
-		cache_store<CT>(crow + i, lat[i] * r * kv_w[i]);
+	if (kv_w) {
+		float ss = 0.0f;
+		for (int i = tid; i < rank; i += SEQ_THREADS)
+			ss = fmaf(lat[i], lat[i], ss);
+		const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)rank + eps);
+		for (int i = i0; i < rank; i += istep)
+			cache_store<CT>(crow + i, lat[i] * r * kv_w[i]);
+	}
+	__syncthreads(); // rot[] before its readers
 	// the rotated parts: job 0 is the shared key part, job 1 + h head h's query part
-	for (int i = i0; i < (H + 1) * R; i += istep) {
+	for (int i = i0 + (kv_w ? 0 : R); i < (H + 1) * R; i += istep) {
 		const int job = i / R, d = i - job * R;
 		const float *src = job == 0 ? lat + rank : z + (size_t)(job - 1) * QH + D;
 		float v;
 		if (d < rot_dims) {
-			const float u = src[d & ~1], w = src[d | 1];
-			const float c = rot[d >> 1], sn = rot[half + (d >> 1)];
-			v = (d & 1) ? w * c + u * sn : u * c - w * sn;
+			const int pr = rot_half ? (d < half ? d : d - half) : d >> 1; // the pair, its two entries
+			const int d0 = rot_half ? pr : d & ~1, d1 = rot_half ? pr + half : d | 1;
+			const float u = src[d0], w = src[d1];
+			const float c = rot[pr], sn = rot[half + pr];
+			v = d == d1 ? w * c + u * sn : u * c - w * sn;
 		} else {
 			v = src[d];
 		}

@@ -68,11 +68,18 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
 
 // The norm kinds (YALM_NORM_*): an rms norm divides a row by sqrt(mean(x^2) + eps); a layer
 // norm first takes the row's mean off, then divides by sqrt(mean(deviation^2) + eps). Both are
-// followed by a weight and have no bias. Kernels take the kind `nk` and for a layer norm
+// followed by a weight. Kernels take the kind `nk` and for a layer norm
 // subtract the mean from the entries they hold before the sum of squares (two passes over values
-// already in registers or LDS, so the variance is that of the deviations themselves). A tanh norm
-// has no statistics: tanh(alpha x) w + b per entry, its weight vector being [w: n | b: n | alpha].
-enum { NK_RMS = YALM_NORM_RMS, NK_LAYER = YALM_NORM_LAYER, NK_TANH = YALM_NORM_TANH };
+// already in registers or LDS, so the variance is that of the deviations themselves). A layer norm
+// with a bias has the weight vector [w: n | b: n]. A tanh norm has no statistics: tanh(alpha x) w + b
+// per entry, its weight vector being [w: n | b: n | alpha].
+enum { NK_RMS = YALM_NORM_RMS, NK_LAYER = YALM_NORM_LAYER, NK_TANH = YALM_NORM_TANH, NK_LAYER_B = YALM_NORM_LAYER_BIAS };
+__device__ __forceinline__ bool nk_centred(int nk) {
+	return nk == NK_LAYER || nk == NK_LAYER_B;
+}
+__device__ __forceinline__ float norm_bias(int nk, const float *__restrict__ w, int n, int i) {
+	return nk == NK_LAYER_B ? w[n + i] : 0.0f;
+}
 __device__ __forceinline__ float tanh_norm(const float *__restrict__ w, int n, int i, float x) {
 	return fmaf(tanhf(w[2 * n] * x), w[i], w[n + i]);
 }
@@ -82,8 +89,18 @@ __device__ __forceinline__ float tanh_norm(const float *__restrict__ w, int n, i
 // st->pos + t if inv_freq), rms-normed with weight e_norm if e_norm (no mean taken off)
 // (+ pre_add, a vector the first layer adds to the stream before its
 // opening norm); tokens == nullptr: the single device-resident token of the greedy
-// loop. w_next != nullptr: also Hn[t] = norm(X[t]) * w_next, the first layer's opening norm,
+// loop. bg.table != nullptr: the row of a token and the one before it is added (see Bigram).
+// w_next != nullptr: also Hn[t] = norm(X[t]) * w_next, the first layer's opening norm,
 // and with w_next2 Hn2[t] = norm(X[t]) * w_next2 (the norm its feed-forward reads).
+// A table of token pairs: row (prev mul_prev + cur mul_cur) mod buckets, row `buckets` for a sequence's
+// first token. The token before the portion's first one is tokens[-1] (-1: none), or, in the greedy
+// loop, *prev, which the launch then replaces by its own token (one workgroup per token there).
+struct Bigram {
+	const void *table = nullptr;
+	int buckets = 0;
+	long long mul_prev = 0, mul_cur = 0;
+	int *prev = nullptr;
+};
 template <class WT>
 __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState *__restrict__ st,
                                                                 const int *__restrict__ tokens,
@@ -95,11 +112,23 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
                                                                 const float *__restrict__ pre_add = nullptr,
                                                                 const float *__restrict__ e_norm = nullptr,
                                                                 const float *__restrict__ w_next2 = nullptr,
-                                                                float *__restrict__ Hn2 = nullptr) {
+                                                                float *__restrict__ Hn2 = nullptr,
+                                                                Bigram bg = Bigram{}) {
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
 	int tok = tokens ? tokens[t] : st->token;
 	tok = min(max(tok, 0), vocab - 1);
+	size_t pair_row = 0;
+	if (bg.table) {
+		int prev = tokens ? tokens[t - 1] : *bg.prev;
+		prev = min(t > 0 ? max(prev, 0) : prev, vocab - 1);
+		pair_row = prev < 0 ? (size_t)bg.buckets : (size_t)((prev * bg.mul_prev + tok * bg.mul_cur) % bg.buckets);
+		if (!tokens) {
+			__syncthreads(); // every thread has read the previous token
+			if (threadIdx.x == 0)
+				*bg.prev = tok;
+		}
+	}
 	const float p = (float)(st->pos + t);
 	// tanh norms without an embedding norm: the workgroups of a token (gridDim.y) share its entries
 	const int i0 = blockIdx.y * SEQ_THREADS + threadIdx.x, istep = gridDim.y * SEQ_THREADS;
@@ -111,6 +140,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 			pe = (i & 1) ? cosf(ang) : sinf(ang);
 		}
 		float v = wload<WT>(emb, (size_t)tok * width + i) * scale + pe;
+		if (bg.table)
+			v += wload<WT>(bg.table, pair_row * width + i);
 		if (pre_add && !e_norm)
 			v += pre_add[i];
 		X[(size_t)t * width + i] = v;
@@ -148,7 +179,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 		return;
 	}
 	float mu = 0.0f;
-	if (nk == NK_LAYER) {
+	if (nk_centred(nk)) {
 		mu = block_sum(sm, red) / (float)width;
 		ss = 0.0f;
 		for (int i = threadIdx.x; i < width; i += SEQ_THREADS) {
@@ -160,9 +191,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_embed_kernel(const StepState 
 	const float r = 1.0f / sqrtf(ss / (float)width + eps);
 	for (int i = threadIdx.x; i < width; i += SEQ_THREADS) {
 		const float v = (X[(size_t)t * width + i] - mu) * r;
-		Hn[(size_t)t * width + i] = v * w_next[i];
+		Hn[(size_t)t * width + i] = v * w_next[i] + norm_bias(nk, w_next, width, i);
 		if (w_next2)
-			Hn2[(size_t)t * width + i] = v * w_next2[i];
+			Hn2[(size_t)t * width + i] = v * w_next2[i] + norm_bias(nk, w_next2, width, i);
 	}
 }
 
@@ -191,7 +222,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_norm_kernel(const float *__re
 		return;
 	}
 	float mu = 0.0f;
-	if (nk == NK_LAYER) {
+	if (nk_centred(nk)) {
 		float sm = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
 			sm += x[i];
@@ -205,7 +236,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_norm_kernel(const float *__re
 	ss = block_sum(ss, red);
 	const float r = post / sqrtf(ss / (float)n + eps);
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
-		const float v = (x[i] - mu) * r * w[i];
+		const float v = (x[i] - mu) * r * w[i] + norm_bias(nk, w, n, i) * post;
 		if constexpr (sizeof(OT) == 2)
 			o[i] = f2bf(v);
 		else
@@ -259,7 +290,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
                                                                        float *__restrict__ Hn, int nk, float rs) {
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x;
-	float y[E], x[E], b[E], wn[E];
+	float y[E], x[E], b[E], wn[E], bb[E], nb[E]; // bb, nb: the biases of layer norms that have one
 #pragma unroll
 	for (int e = 0; e < E; ++e) {
 		const int i = threadIdx.x + e * SEQ_THREADS;
@@ -268,8 +299,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 		x[e] = in ? X[(size_t)t * n + i] : 0.0f;
 		b[e] = in ? wb[i] : 0.0f;
 		wn[e] = (in && w_next) ? w_next[i] : 0.0f;
+		bb[e] = in ? rs * norm_bias(nk, wb, n, i) : 0.0f;
+		nb[e] = (in && w_next) ? norm_bias(nk, w_next, n, i) : 0.0f;
 	}
-	if (nk == NK_LAYER) { // entries past the row's end stay 0
+	if (nk_centred(nk)) { // entries past the row's end stay 0
 		float sm = 0.0f;
 #pragma unroll
 		for (int e = 0; e < E; ++e)
@@ -300,7 +333,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 #pragma unroll
 	for (int e = 0; e < E; ++e) {
 		const int i = threadIdx.x + e * SEQ_THREADS;
-		x[e] = x[e] + y[e] * r * b[e];
+		x[e] = x[e] + (y[e] * r * b[e] + bb[e]);
 		if (i < n) {
 			X[(size_t)t * n + i] = x[e];
 			s2 = fmaf(x[e], x[e], s2);
@@ -318,7 +351,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 		}
 		return;
 	}
-	if (nk == NK_LAYER) {
+	if (nk_centred(nk)) {
 		const float mu = block_sum(sm2, red) / (float)n;
 		s2 = 0.0f;
 #pragma unroll
@@ -334,7 +367,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_reg_kernel(float *__
 	for (int e = 0; e < E; ++e) {
 		const int i = threadIdx.x + e * SEQ_THREADS;
 		if (i < n)
-			Hn[(size_t)t * n + i] = x[e] * r2 * wn[e];
+			Hn[(size_t)t * n + i] = x[e] * r2 * wn[e] + nb[e];
 	}
 }
 
@@ -344,6 +377,11 @@ __device__ __forceinline__ const float *combine_row(const float *Yx, const int *
                                                     int top, int k, int n) {
 	const size_t slot = (size_t)t * top + k;
 	return (hid && idx[slot] >= n_exp) ? hid + (size_t)t * n : Yx + slot * n;
+}
+
+// The weight of a choice in the combine; wt == nullptr: 1 (the weight has been applied to the expert's input).
+__device__ __forceinline__ float combine_weight(const float *wt, size_t slot) {
+	return wt ? wt[slot] : 1.0f;
 }
 
 // Yx != null: Y is not read; its row is the routed experts' combine sum_k wt[t][k] Yx[t top + k]
@@ -369,7 +407,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		if (Yx) {
 			v = 0.0f;
 			for (int k = 0; k < top; ++k)
-				v = fmaf(wt[(size_t)t * top + k], combine_row(Yx, idx, n_exp, hid, t, top, k, n)[i], v);
+				v = fmaf(combine_weight(wt, (size_t)t * top + k), combine_row(Yx, idx, n_exp, hid, t, top, k, n)[i], v);
 			if (Ys)
 				v = fmaf(sgate ? sgate[t] : 1.0f, Ys[(size_t)t * n + i], v);
 		} else {
@@ -380,7 +418,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		sm += v;
 	}
 	float mu = 0.0f;
-	if (nk == NK_LAYER) { // each thread re-reads the entries it wrote
+	if (nk_centred(nk)) { // each thread re-reads the entries it wrote
 		mu = block_sum(sm, red) / (float)n;
 		ss = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
@@ -393,7 +431,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		r = rs / sqrtf(block_sum(ss, red) / (float)n + eps);
 	float s2 = 0.0f, sm2 = 0.0f;
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
-		const float v = x[i] + (nk == NK_TANH ? tanh_norm(wb, n, i, row[i]) * r : (row[i] - mu) * r * wb[i]);
+		const float v = x[i] + (nk == NK_TANH ? tanh_norm(wb, n, i, row[i]) * r : (row[i] - mu) * r * wb[i] + rs * norm_bias(nk, wb, n, i));
 		x[i] = v;
 		row[i] = v;
 		s2 = fmaf(v, v, s2);
@@ -407,7 +445,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 		return;
 	}
 	float mu2 = 0.0f;
-	if (nk == NK_LAYER) {
+	if (nk_centred(nk)) {
 		mu2 = block_sum(sm2, red) / (float)n;
 		s2 = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
@@ -418,7 +456,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_add_norm_kernel(float *__rest
 	s2 = block_sum(s2, red);
 	const float r2 = 1.0f / sqrtf(s2 / (float)n + eps);
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
-		Hn[(size_t)t * n + i] = (row[i] - mu2) * r2 * w_next[i];
+		Hn[(size_t)t * n + i] = (row[i] - mu2) * r2 * w_next[i] + norm_bias(nk, w_next, n, i);
 }
 
 // The seam after a parallel block, one launch: X[t] += rs (s1 * Y1[t] + s2 * Y2[t]) (rs the model's
@@ -477,7 +515,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
 		if (Yx) {
 			float f = 0.0f;
 			for (int k = 0; k < top; ++k)
-				f = fmaf(wt[(size_t)t * top + k], combine_row(Yx, idx, n_exp, hid, t, top, k, n)[i], f);
+				f = fmaf(combine_weight(wt, (size_t)t * top + k), combine_row(Yx, idx, n_exp, hid, t, top, k, n)[i], f);
 			if (Ys)
 				f = fmaf(sgate ? sgate[t] : 1.0f, Ys[(size_t)t * n + i], f);
 			v = fmaf(rs * (s2 ? s2[i] : 1.0f), f, v);
@@ -504,7 +542,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
 		return;
 	}
 	float mu = 0.0f;
-	if (nk == NK_LAYER) { // each thread re-reads the entries it wrote
+	if (nk_centred(nk)) { // each thread re-reads the entries it wrote
 		mu = block_sum(sm, red) / (float)n;
 		ss = 0.0f;
 		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
@@ -516,9 +554,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_kernel(float *__res
 	const float r = 1.0f / sqrtf(ss / (float)n + eps);
 	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
 		const float v = (row[i] - mu) * r;
-		Hn[(size_t)t * n + i] = v * w_next[i];
+		Hn[(size_t)t * n + i] = v * w_next[i] + norm_bias(nk, w_next, n, i);
 		if (w_next2)
-			Hn2[(size_t)t * n + i] = v * w_next2[i];
+			Hn2[(size_t)t * n + i] = v * w_next2[i] + norm_bias(nk, w_next2, n, i);
 	}
 }
 
@@ -549,7 +587,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	__shared__ float red[SEQ_THREADS / 64];
 	const int t = blockIdx.x, c0 = blockIdx.y * E * SEQ_THREADS + threadIdx.x;
 	float x[E], y1[E], a1[E], f[E], a2[E], ad[E], wn[E];
-	float wn2[E], nb[E] = {}, nb2[E] = {}, al = 0.0f, al2 = 0.0f; // nb, al: biases and alphas of tanh norms
+	float wn2[E], nb[E] = {}, nb2[E] = {}, al = 0.0f, al2 = 0.0f; // nb, al: biases (tanh norms, layer norms that have one) and alphas
 	const bool tn = nk == NK_TANH && w_next;
 	const bool ff = Yx || Y2;
 #pragma unroll
@@ -564,7 +602,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 		wn[e] = (in && w_next) ? w_next[i] : 0.0f;
 		f[e] = (in && Y2 && !Yx) ? Y2[(size_t)t * n + i] : 0.0f;
 		wn2[e] = (in && w_next && w_next2) ? w_next2[i] : 0.0f;
-		if (tn && in) {
+		if ((tn || (nk == NK_LAYER_B && w_next)) && in) {
 			nb[e] = w_next[n + i];
 			nb2[e] = w_next2 ? w_next2[n + i] : 0.0f;
 		}
@@ -604,7 +642,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 #pragma unroll
 			for (int u = 0; u < KB; ++u) {
 				const int k = min(k0 + u, top - 1);
-				w[u] = k0 + u < top ? wt[(size_t)t * top + k] : 0.0f;
+				w[u] = k0 + u < top ? combine_weight(wt, (size_t)t * top + k) : 0.0f;
 				const float *src = combine_row(Yx, idx, n_exp, hid, t, top, k, n);
 #pragma unroll
 				for (int e = 0; e < E; ++e) {
@@ -659,7 +697,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 		}
 		return;
 	}
-	if (nk == NK_LAYER) {
+	if (nk_centred(nk)) {
 		const float mu = block_sum(sm, red) / (float)n;
 		ss = 0.0f;
 #pragma unroll
@@ -675,11 +713,145 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_par_close_reg_kernel(float *_
 	for (int e = 0; e < E; ++e) {
 		const int i = c0 + e * SEQ_THREADS;
 		if (i < n) {
-			Hn[(size_t)t * n + i] = x[e] * r * wn[e];
+			Hn[(size_t)t * n + i] = x[e] * r * wn[e] + nb[e];
 			if (w_next2)
-				Hn2[(size_t)t * n + i] = x[e] * r * wn2[e];
+				Hn2[(size_t)t * n + i] = x[e] * r * wn2[e] + nb2[e];
 		}
 	}
+}
+
+// The seam after a sublayer of a post-norm block, one launch: X[t] <- norm(alpha X[t] + rs y) with y =
+// Y[t], or (Yx != nullptr) the routed experts' combine sum_k wt[t][k] Yx[t top + k] (wt == nullptr: all
+// weights 1) + sgate[t] Ys[t] (sgate == nullptr: + Ys[t]), summed in slot order. Rows of up to
+// E * SEQ_THREADS entries, the row in registers: every operand row and vector is loaded at once.
+template <int E>
+__global__ __launch_bounds__(SEQ_THREADS) void seq_post_close_reg_kernel(float *__restrict__ X, const float *__restrict__ Y,
+                                                                         const float *__restrict__ Yx,
+                                                                         const float *__restrict__ wt, int top,
+                                                                         const float *__restrict__ Ys,
+                                                                         const float *__restrict__ sgate,
+                                                                         const float *__restrict__ wb, float eps, int n,
+                                                                         int nk, float alpha, float rs) {
+	__shared__ float red[SEQ_THREADS / 64];
+	const int t = blockIdx.x;
+	float x[E], f[E], w[E], b[E];
+	const float sg = sgate ? sgate[t] : 1.0f;
+#pragma unroll
+	for (int e = 0; e < E; ++e) {
+		const int i = threadIdx.x + e * SEQ_THREADS;
+		const bool in = i < n;
+		x[e] = in ? X[(size_t)t * n + i] : 0.0f;
+		f[e] = (in && !Yx) ? Y[(size_t)t * n + i] : 0.0f;
+		w[e] = in ? wb[i] : 0.0f;
+		b[e] = (in && (nk == NK_LAYER_B || nk == NK_TANH)) ? wb[n + i] : 0.0f;
+	}
+	if (Yx) {
+		constexpr int KB = 4; // choices whose rows are in flight together
+		for (int k0 = 0; k0 < top; k0 += KB) {
+			float cw[KB], v[KB][E];
+#pragma unroll
+			for (int u = 0; u < KB; ++u) {
+				const size_t slot = (size_t)t * top + min(k0 + u, top - 1);
+				cw[u] = k0 + u < top ? combine_weight(wt, slot) : 0.0f;
+#pragma unroll
+				for (int e = 0; e < E; ++e) {
+					const int i = threadIdx.x + e * SEQ_THREADS;
+					v[u][e] = (i < n && k0 + u < top) ? Yx[slot * n + i] : 0.0f;
+				}
+			}
+#pragma unroll
+			for (int u = 0; u < KB; ++u)
+#pragma unroll
+				for (int e = 0; e < E; ++e)
+					f[e] = fmaf(cw[u], v[u][e], f[e]);
+		}
+		if (Ys)
+#pragma unroll
+			for (int e = 0; e < E; ++e) {
+				const int i = threadIdx.x + e * SEQ_THREADS;
+				f[e] = fmaf(sg, i < n ? Ys[(size_t)t * n + i] : 0.0f, f[e]);
+			}
+	}
+	float sm = 0.0f, ss = 0.0f;
+#pragma unroll
+	for (int e = 0; e < E; ++e) { // entries past the row's end stay 0
+		x[e] = fmaf(alpha, x[e], rs * f[e]);
+		sm += x[e];
+		ss = fmaf(x[e], x[e], ss);
+	}
+	if (nk == NK_TANH) {
+		const float al = wb[2 * n];
+#pragma unroll
+		for (int e = 0; e < E; ++e) {
+			const int i = threadIdx.x + e * SEQ_THREADS;
+			if (i < n)
+				X[(size_t)t * n + i] = fmaf(tanhf(al * x[e]), w[e], b[e]);
+		}
+		return;
+	}
+	if (nk_centred(nk)) {
+		const float mu = block_sum(sm, red) / (float)n;
+		ss = 0.0f;
+#pragma unroll
+		for (int e = 0; e < E; ++e)
+			if (threadIdx.x + e * SEQ_THREADS < n) {
+				x[e] -= mu;
+				ss = fmaf(x[e], x[e], ss);
+			}
+	}
+	const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+#pragma unroll
+	for (int e = 0; e < E; ++e) {
+		const int i = threadIdx.x + e * SEQ_THREADS;
+		if (i < n)
+			X[(size_t)t * n + i] = fmaf(x[e] * r, w[e], b[e]);
+	}
+}
+// The same with the row in LDS (any width). Dynamic LDS: n floats.
+__global__ __launch_bounds__(SEQ_THREADS) void seq_post_close_kernel(float *__restrict__ X, const float *__restrict__ Y,
+                                                                     const float *__restrict__ Yx,
+                                                                     const float *__restrict__ wt, int top,
+                                                                     const float *__restrict__ Ys,
+                                                                     const float *__restrict__ sgate,
+                                                                     const float *__restrict__ wb, float eps, int n, int nk,
+                                                                     float alpha, float rs) {
+	extern __shared__ float row[];
+	__shared__ float red[SEQ_THREADS / 64];
+	const int t = blockIdx.x;
+	float *x = X + (size_t)t * n;
+	float sm = 0.0f, ss = 0.0f;
+	for (int i = threadIdx.x; i < n; i += SEQ_THREADS) { // each thread re-reads the entries it wrote
+		float f = 0.0f;
+		if (Yx) {
+			for (int k = 0; k < top; ++k)
+				f = fmaf(combine_weight(wt, (size_t)t * top + k), Yx[((size_t)t * top + k) * n + i], f);
+			if (Ys)
+				f = fmaf(sgate ? sgate[t] : 1.0f, Ys[(size_t)t * n + i], f);
+		} else {
+			f = Y[(size_t)t * n + i];
+		}
+		const float v = fmaf(alpha, x[i], rs * f);
+		row[i] = v;
+		sm += v;
+		ss = fmaf(v, v, ss);
+	}
+	if (nk == NK_TANH) {
+		for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
+			x[i] = tanh_norm(wb, n, i, row[i]);
+		return;
+	}
+	float mu = 0.0f;
+	if (nk_centred(nk)) {
+		mu = block_sum(sm, red) / (float)n;
+		ss = 0.0f;
+		for (int i = threadIdx.x; i < n; i += SEQ_THREADS) {
+			const float d = row[i] - mu;
+			ss = fmaf(d, d, ss);
+		}
+	}
+	const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)n + eps);
+	for (int i = threadIdx.x; i < n; i += SEQ_THREADS)
+		x[i] = fmaf((row[i] - mu) * r, wb[i], norm_bias(nk, wb, n, i));
 }
 
 // Two mixers side by side: Ya[t] <- scale (rms(Ya[t]) wa + rms(Yb[t]) wb), each row divided by
@@ -722,7 +894,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gate_mul_kernel(float *__rest
 
 // ------------------------------------------------------------------ matrix products
 enum { EPI_NONE = 0, EPI_GLU_GELU = 1, EPI_GLU_CLAMP = 2, EPI_SIGMOID = 3, EPI_GELU = 4, EPI_GLU_SILU = 5, EPI_RELU2 = 6,
-       EPI_GELU_ERF = 7, EPI_SOFT_CAP = 8 /* limit tanh(. / limit) */ };
+       EPI_GELU_ERF = 7, EPI_SOFT_CAP = 8, /* limit tanh(. / limit) */
+       EPI_SIG_ROOT = 9 /* sigmoid(.)^(1 / limit): a recurrence's decays */ };
 
 // C[c_row(m)][n] = epi(sum_k A[a_row(m)][k] W[n][k]) for every batch z = blockIdx.z.
 struct GemmArgs {
@@ -761,6 +934,14 @@ struct GemmArgs {
 	const void *W2_b = nullptr;
 	int M_b = 0, N_b = 0, K_b = 0;
 	float limit_b = 0.0f;
+	// result row r's sums times row_scale[r] before the epilogue (batch z: + z * row_scale_bs; the second product of
+	// z_split: not): W (s a) = s (W a), the weight of a routed expert's input
+	const float *row_scale = nullptr;
+	long row_scale_bs = 0;
+	// entry (r, n) of the result times sigmoid(gate[r * ldgate + n]) (batch z: + z * gate_bs)
+	const float *gate = nullptr;
+	int ldgate = 0;
+	long gate_bs = 0;
 };
 
 __device__ __forceinline__ float epi_apply(const GemmArgs &a, float v, float v2, float b, float limit) {
@@ -780,6 +961,7 @@ __device__ __forceinline__ float epi_apply(const GemmArgs &a, float v, float v2,
 	}
 	case EPI_GELU_ERF: return sq_gelu_erf(v + b);
 	case EPI_SOFT_CAP: return sq_soft_cap(v + b, limit);
+	case EPI_SIG_ROOT: return expf(sq_log_sigmoid(v + b) / limit);
 	default: return v + b;
 	}
 }
@@ -792,6 +974,7 @@ struct GemmBatch {
 	const int *rows;
 	int M, N, K, lda, ldw, ldc;
 	float limit;
+	const float *row_scale, *gate;
 };
 template <class WT>
 __device__ __forceinline__ GemmBatch gemm_batch(const GemmArgs &a, int z) {
@@ -818,7 +1001,21 @@ __device__ __forceinline__ GemmBatch gemm_batch(const GemmArgs &a, int z) {
 	b.bias = bias ? bias + (long)z * a.bias_bs : nullptr;
 	b.rows = a.rows ? a.rows + (long)z * a.rows_bs : nullptr;
 	b.M = none ? 0 : (a.counts ? a.counts[z] : a.M);
+	b.row_scale = a.row_scale && !second ? a.row_scale + (long)z * a.row_scale_bs : nullptr;
+	b.gate = a.gate && !second ? a.gate + (long)z * a.gate_bs : nullptr;
 	return b;
+}
+// Entry (rc, n) of the result from the sums of the one or two matrices.
+__device__ __forceinline__ float epi_out(const GemmArgs &a, const GemmBatch &b, int rc, int n, float v, float v2) {
+	if (b.row_scale) {
+		const float s = b.row_scale[rc];
+		v *= s;
+		v2 *= s;
+	}
+	float y = epi_apply(a, v, v2, b.bias ? b.bias[n] : 0.0f, b.limit);
+	if (b.gate)
+		y *= sq_sigmoid(b.gate[(size_t)rc * a.ldgate + n]);
+	return y;
 }
 
 // ---- single tokens and short portions: one wave per output column streams its weight
@@ -965,7 +1162,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_kernel(GemmArgs a) {
 			const float v = wave_sum(acc[m]);
 			const float v2 = GLU ? wave_sum(acc2[m]) : 0.0f;
 			if (lane == 0)
-				b.C[(size_t)crow[m] * b.ldc + n] = epi_apply(a, v, v2, b.bias ? b.bias[n] : 0.0f, b.limit);
+				b.C[(size_t)crow[m] * b.ldc + n] = epi_out(a, b, crow[m], n, v, v2);
 		}
 	}
 }
@@ -1003,7 +1200,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_an_kernel(const float *_
 		}
 	};
 	fetch(n0);
-	float4_t x[KI], y[KI], b[KI];
+	float4_t x[KI], y[KI], b[KI], bb[KI]; // bb: the bias of a layer norm that has one
 	float sm = 0.0f;
 #pragma unroll
 	for (int i = 0; i < KI; ++i) {
@@ -1012,9 +1209,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_an_kernel(const float *_
 		y[i] = in ? *(const float4_t *)(Y + k) : float4_t{0, 0, 0, 0};
 		x[i] = in ? *(const float4_t *)(X + k) : float4_t{0, 0, 0, 0};
 		b[i] = in ? *(const float4_t *)(wb + k) : float4_t{0, 0, 0, 0};
+		bb[i] = (in && nk == NK_LAYER_B) ? *(const float4_t *)(wb + K + k) * rs : float4_t{0, 0, 0, 0};
 		sm += (y[i][0] + y[i][1]) + (y[i][2] + y[i][3]);
 	}
-	if (nk == NK_LAYER) { // entries past the row's end stay 0
+	if (nk_centred(nk)) { // entries past the row's end stay 0
 		const float mu = block_sum(sm, red) / (float)K;
 #pragma unroll
 		for (int i = 0; i < KI; ++i)
@@ -1037,7 +1235,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemv_an_kernel(const float *_
 			continue;
 #pragma unroll
 		for (int e = 0; e < 4; ++e)
-			x[i][e] = fmaf(y[i][e] * r, b[i][e], x[i][e]);
+			x[i][e] = fmaf(y[i][e] * r, b[i][e], x[i][e] + bb[i][e]);
 		*(float4_t *)(xs + k) = x[i];
 		if (blockIdx.x == 0)
 			*(float4_t *)(Xout + k) = x[i];
@@ -1183,13 +1381,12 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_kernel(GemmArgs a) {
 		}
 		const int n = n0 + wn + (lane & 31);
 		if (n < a.N) {
-			const float bias = b.bias ? b.bias[n] : 0.0f;
 #pragma unroll
 			for (int r = 0; r < 16; ++r) {
 				const int ml = wm + (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
 				const int rc = crow[ml];
 				if (rc >= 0)
-					b.C[(size_t)rc * a.ldc + n] = epi_apply(a, acc[r], GLU ? acc2[r] : 0.0f, bias, b.limit);
+					b.C[(size_t)rc * a.ldc + n] = epi_out(a, b, rc, n, acc[r], GLU ? acc2[r] : 0.0f);
 			}
 		}
 	} else {
@@ -1237,8 +1434,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_kernel(GemmArgs a) {
 			for (int j = 0; j < 4; ++j) {
 				const int n = n0 + tx * 4 + j;
 				if (n < a.N)
-					b.C[(size_t)rc * a.ldc + n] =
-					    epi_apply(a, acc[i][j], GLU ? acc2[i][j] : 0.0f, b.bias ? b.bias[n] : 0.0f, b.limit);
+					b.C[(size_t)rc * a.ldc + n] = epi_out(a, b, rc, n, acc[i][j], GLU ? acc2[i][j] : 0.0f);
 			}
 		}
 	}
@@ -1275,8 +1471,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_bf16_kernel(GemmArgs a) 
 		return;
 	constexpr int LD = GT_BK + 8;
 	__shared__ int arow[GB_BM], crow[GB_BM];
-	__shared__ __attribute__((aligned(16))) uint16_t As[2][GB_BM * LD], Bs[2][GB_BN * LD],
-	    Bs2[GLU ? 2 : 1][GLU ? GB_BN * LD : 8];
+	__shared__ __attribute__((aligned(16))) uint16_t smem[(GLU ? 3 : 2) * 2 * GB_BM * LD];
+	// operand x (0: A, 1: W, 2: W2) of buffer `buf`
+	auto slab = [&](int x, int buf) { return smem + (2 * x + buf) * GB_BM * LD; };
 	const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
 	if (tid < GB_BM) {
 		const int m = m0 + tid;
@@ -1349,10 +1546,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_bf16_kernel(GemmArgs a) 
 	auto stash = [&](int buf) {
 #pragma unroll
 		for (int h = 0; h < 2; ++h) {
-			*(u32x4_t *)(As[buf] + (lr + 64 * h) * LD + lk) = pa[h];
-			*(u32x4_t *)(Bs[buf] + (lr + 64 * h) * LD + lk) = pb[h];
+			*(u32x4_t *)(slab(0, buf) + (lr + 64 * h) * LD + lk) = pa[h];
+			*(u32x4_t *)(slab(1, buf) + (lr + 64 * h) * LD + lk) = pb[h];
 			if constexpr (GLU)
-				*(u32x4_t *)(Bs2[buf] + (lr + 64 * h) * LD + lk) = pb2[h];
+				*(u32x4_t *)(slab(2, buf) + (lr + 64 * h) * LD + lk) = pb2[h];
 		}
 	};
 	float16_t acc[2][2] = {}, acc2[GLU ? 2 : 1][GLU ? 2 : 1] = {};
@@ -1370,11 +1567,11 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_bf16_kernel(GemmArgs a) 
 			bf16x8_t fa[2], fb[2], fb2[2];
 #pragma unroll
 			for (int i = 0; i < 2; ++i) {
-				fa[i] = __builtin_bit_cast(bf16x8_t, *(const u32x4_t *)(As[buf] + (wm + 32 * i + (lane & 31)) * LD + kk));
-				fb[i] = __builtin_bit_cast(bf16x8_t, *(const u32x4_t *)(Bs[buf] + (wn + 32 * i + (lane & 31)) * LD + kk));
+				fa[i] = __builtin_bit_cast(bf16x8_t, *(const u32x4_t *)(slab(0, buf) + (wm + 32 * i + (lane & 31)) * LD + kk));
+				fb[i] = __builtin_bit_cast(bf16x8_t, *(const u32x4_t *)(slab(1, buf) + (wn + 32 * i + (lane & 31)) * LD + kk));
 				if constexpr (GLU)
 					fb2[i] = __builtin_bit_cast(bf16x8_t,
-					                            *(const u32x4_t *)(Bs2[buf] + (wn + 32 * i + (lane & 31)) * LD + kk));
+					                            *(const u32x4_t *)(slab(2, buf) + (wn + 32 * i + (lane & 31)) * LD + kk));
 			}
 #pragma unroll
 			for (int i = 0; i < 2; ++i)
@@ -1390,22 +1587,33 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_bf16_kernel(GemmArgs a) 
 		__syncthreads();
 		buf ^= 1;
 	}
+	// The epilogue's code is emitted once per 32 x 32 tile instead of once per register: a tile's sums pass
+	// through the wave's own part of the (now idle) operand buffers.
+	constexpr int LDE = 33;
+	static_assert(GB_BM == GB_BN && 4 * 32 * LDE * 4 * (GLU ? 2 : 1) <= sizeof(smem), "the sums fit in the operand buffers");
+	float *const E1 = (float *)smem + wave * 32 * LDE * (GLU ? 2 : 1), *const E2 = E1 + (GLU ? 32 * LDE : 0);
 #pragma unroll
-	for (int j = 0; j < 2; ++j) {
-		const int n = n0 + wn + 32 * j + (lane & 31);
-		if (n >= a.N)
-			continue;
-		const float bias = b.bias ? b.bias[n] : 0.0f;
+	for (int j = 0; j < 2; ++j)
 #pragma unroll
-		for (int i = 0; i < 2; ++i)
+		for (int i = 0; i < 2; ++i) {
 #pragma unroll
 			for (int r = 0; r < 16; ++r) {
-				const int ml = wm + 32 * i + (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
-				const int rc = crow[ml];
-				if (rc >= 0)
-					b.C[(size_t)rc * a.ldc + n] = epi_apply(a, acc[i][j][r], GLU ? acc2[i][j][r] : 0.0f, bias, b.limit);
+				const int ml = (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
+				E1[ml * LDE + (lane & 31)] = acc[i][j][r];
+				if constexpr (GLU)
+					E2[ml * LDE + (lane & 31)] = acc2[i][j][r];
 			}
-	}
+			__syncthreads();
+			const int n = n0 + wn + 32 * j + (lane & 31);
+#pragma unroll 1
+			for (int it = 0; it < 16; ++it) {
+				const int ml = 2 * it + (lane >> 5), rc = crow[wm + 32 * i + ml];
+				if (rc >= 0 && n < a.N)
+					b.C[(size_t)rc * a.ldc + n] =
+					    epi_out(a, b, rc, n, E1[ml * LDE + (lane & 31)], GLU ? E2[ml * LDE + (lane & 31)] : 0.0f);
+			}
+			__syncthreads();
+		}
 }
 
 // ------------------------------------------------------------------ short causal convolution
@@ -1656,7 +1864,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_mem_gates_kernel(float *__res
 // read-outs O [t][H][V + 1] are oscale S.q, in the last column max(|oscale S.q|, exp(-m)) + 1e-6, the
 // divisor of the others. mst [H][gridDim.x]: the running maximum, one copy per workgroup of a head
 // (each reads and writes its own).
-// GVEC: g is a vector over the key channels, GV [T][H D], instead of one number per head.
+// GVEC: g is a vector over the key channels, GV [T][H D], instead of one number per head. With SSM: gated
+// linear attention, S <- diag(g) S + k v^T, o = oscale S.q (no per-head factors, BG is not read).
 // QKV [T][ldq]: key/query head kh's q at column qo + kh D, its k at ko + kh D, head h's v at vo + h V.
 template <int R, int TC, bool SSM, bool GVEC, int LPC, bool MEM = false>
 __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__restrict__ QKV, int ldq, int qo_, int ko_,
@@ -1669,6 +1878,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
                                                                 int ldlg = 0, float gcap = 0.0f,
                                                                 float oscale = 1.0f, float *__restrict__ mst = nullptr) {
 	constexpr int DP = LPC * R;                    // padded key dimension
+	constexpr bool GLA = SSM && GVEC;
 	constexpr int NS = GVEC ? 3 : 2;               // staged rows per token: k | q (| g)
 	constexpr int NKQ = TC * NS * DP / SEQ_THREADS; // staged values per thread and chunk
 	constexpr int COLS = SEQ_THREADS / LPC, NV = (TC * COLS + SEQ_THREADS - 1) / SEQ_THREADS;
@@ -1725,7 +1935,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 					rlf = mem_log_gate(rlf, gcap, true);
 				}
 			}
-		} else if (tid < 2 * TC) {
+		} else if (!GLA && tid < 2 * TC) {
 			const int t = t0 + (tid >> 1);
 			rbg = t < T ? BG[(size_t)t * 2 * H + (tid & 1) * H + h] : 0.0f;
 		}
@@ -1765,7 +1975,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 				}
 				mrun = __shfl(m, 15);
 			}
-		} else if (tid < 2 * TC) {
+		} else if (!GLA && tid < 2 * TC) {
 			bgs[buf][tid >> 1][tid & 1] = rbg;
 		}
 	};
@@ -1812,8 +2022,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 				}
 			}
 			x.v = vs[buf][tt][tid / LPC];
-			x.beta = bgs[buf][tt][0];
-			x.g = bgs[buf][tt][1];
+			if constexpr (!GLA) {
+				x.beta = bgs[buf][tt][0];
+				x.g = bgs[buf][tt][1];
+			}
 			if constexpr (MEM)
 				x.em = bgs[buf][tt][2];
 		};
@@ -1833,7 +2045,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 				}
 			}
 			float u;
-			if constexpr (SSM)
+			if constexpr (GLA)
+				u = x.v;
+			else if constexpr (SSM)
 				u = x.beta * x.v;
 			else
 				u = x.beta * (x.v - sum_lanes<LPC>(dd0 + dd1));
@@ -1851,6 +2065,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 				o *= oscale;
 				if (col == V)
 					o = fmaxf(fabsf(o), x.em) + 1e-6f;
+			} else if constexpr (GLA) {
+				o *= oscale;
 			} else if constexpr (SSM) {
 				o = fmaf(dsk, x.v, o);
 			}
@@ -2305,7 +2521,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_latent_attn_mfma_kernel(const
 // bias: a group by the sum of its two largest, the `top` largest within the `keep` best groups
 // win (ties: the lower index); weight = score * rscale, without the bias, not renormalised. kind 3:
 // scores = softmax over all E; the `top` largest score + bias win (ties: the lower index, no groups);
-// weight = score / (sum of the chosen scores + 1e-20) * rscale.
+// weight = score / (sum of the chosen scores + 1e-20) * rscale. kind 4: the `top` largest logits + bias
+// win (ties: the lower index, no groups; the sigmoid is monotone, but rounds to 1 above a logit of
+// about 17); weight = sigmoid(logit) * rscale.
 // NT threads (kind 0: SEQ_THREADS).
 // Also the shared expert's gate sigmoid(w_sg . h). Dynamic LDS: 2 E + G floats.
 #define SEQ_MAX_GROUPS 64
@@ -2373,22 +2591,29 @@ __global__ __launch_bounds__(NT) void seq_router_kernel(const float *__restrict_
 	}
 	float *gsc = sc + E; // [G]
 	__shared__ float red[SEQ_THREADS / 64];
-	if (kind == 3) { // one wave: a lane owns experts lane, lane + 64, ... and only touches their entries
+	if (kind >= 3) { // one wave: a lane owns experts lane, lane + 64, ... and only touches their entries
 		if (wave != 0)
 			return;
 		float *sv = gsc + G; // [E] the scores (the weights); sc becomes the choice scores
-		float mx = -FLT_MAX, sum = 0.0f;
-		for (int e = lane; e < E; e += 64)
-			mx = fmaxf(mx, sc[e]);
-		mx = wave_max(mx);
-		for (int e = lane; e < E; e += 64) {
-			sv[e] = expf(sc[e] - mx);
-			sum += sv[e];
-		}
-		const float inv = 1.0f / wave_sum(sum);
-		for (int e = lane; e < E; e += 64) {
-			sv[e] *= inv;
-			sc[e] = sv[e] + (bias ? bias[e] : 0.0f);
+		if (kind == 4) {
+			for (int e = lane; e < E; e += 64) {
+				sv[e] = sq_sigmoid(sc[e]);
+				sc[e] += bias ? bias[e] : 0.0f;
+			}
+		} else {
+			float mx = -FLT_MAX, sum = 0.0f;
+			for (int e = lane; e < E; e += 64)
+				mx = fmaxf(mx, sc[e]);
+			mx = wave_max(mx);
+			for (int e = lane; e < E; e += 64) {
+				sv[e] = expf(sc[e] - mx);
+				sum += sv[e];
+			}
+			const float inv = 1.0f / wave_sum(sum);
+			for (int e = lane; e < E; e += 64) {
+				sv[e] *= inv;
+				sc[e] = sv[e] + (bias ? bias[e] : 0.0f);
+			}
 		}
 		float chosen = 0.0f; // sum of the chosen scores
 		for (int k = 0; k < top; ++k) {
@@ -2418,7 +2643,7 @@ __global__ __launch_bounds__(NT) void seq_router_kernel(const float *__restrict_
 				wt[(size_t)t * top + k] = score;
 			}
 		}
-		const float f = rscale / (chosen + 1e-20f);
+		const float f = kind == 4 ? rscale : rscale / (chosen + 1e-20f);
 		__threadfence_block(); // the weights written by other lanes of this wave
 		for (int k = lane; k < top; k += 64)
 			wt[(size_t)t * top + k] *= f;

@@ -10,9 +10,11 @@ experts). ``Sinulorn`` (latent attention, recurrences, routed experts), ``Lenuze
 blocks with layer scales, a looped run of layers, gated attention, latent attention with a
 rotated key part, a window and a learned sink), ``Lifenex`` (parallel blocks with a norm
 per sublayer, a selective state-space mixer, attention with a distance bias beside a delta
-rule with per-channel decays, grouped sigmoid routing) and ``Faguzen`` (norms without
+rule with per-channel decays, grouped sigmoid routing), ``Faguzen`` (norms without
 statistics, score-capped attention beside a matrix memory, ungated experts with identity
-outputs, a looped run) are such designs.
+outputs, a looped run) and ``Gugozen`` (post-norm blocks, token-pair embedding, gated linear
+attention, latent attention over shared latents, experts weighted at their input) are such
+designs.
 
 Checkpoints are folders with ``config.json`` and ``model.safetensors`` (bf16
 matrices; read with yalmfile.read_yalm, the same container the .yalm files use).
@@ -28,14 +30,15 @@ import numpy as np
 
 from . import models as M
 
-MIX_LATENT, MIX_RGLRU, MIX_DELTA, MIX_ATTN, MIX_SSM, MIX_MEMORY = 0, 1, 2, 3, 4, 5
+MIX_LATENT, MIX_RGLRU, MIX_DELTA, MIX_ATTN, MIX_SSM, MIX_MEMORY, MIX_GLA = 0, 1, 2, 3, 4, 5, 6
 FF_NONE, FF_DENSE, FF_MOE, FF_PLAIN = 0, 1, 2, 3
-NORM_RMS, NORM_LAYER, NORM_TANH = 0, 1, 2
+NORM_RMS, NORM_LAYER, NORM_TANH, NORM_LAYER_BIAS = 0, 1, 2, 3
 MASK_CAUSAL, MASK_WINDOW, MASK_CHUNK = 0, 1, 2
 QK_NONE, QK_HEAD_UNIT, QK_WHOLE, QK_HEAD_W = 0, 1, 2, 3
-BLOCK_SERIAL, BLOCK_PARALLEL = 0, 1
+BLOCK_SERIAL, BLOCK_PARALLEL, BLOCK_POST = 0, 1, 2
 ACT_DEFAULT, ACT_GELU, ACT_CLAMP, ACT_SILU, ACT_RELU2, ACT_GELU_ERF = 0, 1, 2, 3, 4, 5
 ROUTER_SOFTMAX_TOP, ROUTER_TOP_SOFTMAX, ROUTER_SIGMOID_GROUPS, ROUTER_SOFTMAX_NORMED = 0, 1, 2, 3
+ROUTER_SIGMOID_TOP = 4
 ROT_INTERLEAVED, ROT_HALVES = 0, 1
 RAMP_INDEX, RAMP_TURNS = 0, 1
 DELTA_GATE_SILU, DELTA_GATE_SIGMOID = 0, 1
@@ -114,6 +117,10 @@ class LayerSpec:
     softcap: float = 0.0        # scores s -> softcap tanh(s / softcap)
     # matrix memory: cap of the log gates' logits
     gate_cap: float = 0.0
+    # gated linear attention: the decays' root (decay_rank above is the rank of their projection)
+    decay_tau: float = 1.0
+    # routed experts: a choice's weight multiplies its expert's input
+    expert_in_weighted: bool = False
     # routed experts: identity outputs after the experts; experts without gate matrices (ff_act of one matrix)
     identity: int = 0
     ungated: bool = False
@@ -134,7 +141,8 @@ class LayerSpec:
         """Rows of the concatenated input projection w_in."""
         if self.mixer == MIX_LATENT:
             if self.q_rank == 0:
-                return self.heads * (self.dim + self.rot_dim) + self.kv_rank + self.rot_dim
+                return (self.heads * (self.dim + self.rot_dim) + (self.kv_rank + self.rot_dim if self.kv_from < 0 else 0)
+                        + (self.heads * self.vdim if self.out_gate == GATE_ELEMENT else 0))
             return self.q_rank + (self.kv_rank if self.kv_from < 0 else 0)
         if self.mixer == MIX_RGLRU:
             return 2 * self.rec_width
@@ -145,6 +153,8 @@ class LayerSpec:
             return 2 * self.heads * self.vdim + 2 * self.ssm_groups * self.ssm_state + self.heads
         if self.mixer == MIX_MEMORY:
             return 2 * self.heads * (self.dim + self.vdim + 1)
+        if self.mixer == MIX_GLA:
+            return 2 * self.heads * (self.dim + self.vdim) + self.decay_rank
         return (2 * self.kv_heads * self.dim + self.heads * self.vdim + (self.gate_rank or self.heads * self.vdim)
                 + self.heads + (self.decay_rank or self.heads))
 
@@ -173,14 +183,20 @@ class LayeredConfig:
     embed_normed: bool = False  # the embedding row is rms-normed (weight embed_norm) before it becomes the stream
     residual_scale: float = 1.0  # every sublayer's result times this as it joins the stream
     logit_softcap: float = 0.0   # logits z -> logit_softcap tanh(z / logit_softcap)
+    stream_scale: float = 1.0    # BLOCK_POST: x <- norm(stream_scale x + f(x))
+    # > 0: row (previous token * bigram_mul_prev + token * bigram_mul_cur) mod bigram_buckets of the table
+    # "bigram" joins the embedding (the last row for a sequence's first token)
+    bigram_buckets: int = 0
+    bigram_mul_prev: int = 0
+    bigram_mul_cur: int = 0
 
     def with_(self, **kw) -> "LayeredConfig":
         return dataclasses.replace(self, **kw)
 
 
 def norm_shape(c: LayeredConfig) -> tuple:
-    """Shape of a norm's vector: the weight, or (tanh norms) weight | bias | alpha."""
-    return (2 * c.width + 1,) if c.norm_kind == NORM_TANH else (c.width,)
+    """Shape of a norm's vector: the weight, or weight | bias, or (tanh norms) weight | bias | alpha."""
+    return {NORM_TANH: (2 * c.width + 1,), NORM_LAYER_BIAS: (2 * c.width,)}.get(c.norm_kind, (c.width,))
 
 
 def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False, shared_in: bool = False) -> dict:
@@ -257,6 +273,8 @@ def packed_shapes(c: LayeredConfig, l: LayerSpec, side: bool = False, shared_in:
         if l.in_biased:
             out["in_bias"] = ((in_rows,), "f")
         out["out_norm"] = ((l.heads * l.vdim,), "f")
+    elif l.mixer == MIX_GLA:
+        out.update(w_a2=((l.heads * l.dim, l.decay_rank), "w"), dt_bias=((l.heads * l.dim,), "f"), out_norm=((l.vdim,), "f"))
     elif l.mixer == MIX_SSM:
         inner, cc = l.heads * l.vdim, l.heads * l.vdim + 2 * l.ssm_groups * l.ssm_state
         out.update(conv_w=((cc, l.conv), "f"), conv_b=((cc,), "f"), a_log=((l.heads,), "f"), dt_bias=((l.heads,), "f"),
@@ -1233,6 +1251,193 @@ def faguzen_random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0) -> dict:
     return out
 
 
+# ------------------------------------------------------------------ Gugozen
+# x = E[token] + B[row], row a hash of the previous and the current token. Post-norm blocks: x <- n1(a x +
+# mix(x)), x <- n2(a x + ff(x)), n a layer norm with weight and bias. Three mixers:
+#   "gla":              gated linear attention, one decay sigmoid(W_a2 W_a1 h + b)^(1 / tau) per head and key
+#                       channel, read-outs rms-normed per head, times silu(W_g h);
+#   "latent_attention": queries [dim plain | rot_dim rotated] per head, a cached rms-normed latent and one
+#                       rotated key part shared by all heads, half-split pairs, the heads times
+#                       sigmoid(W_g h); with kv_from the cache rows of that layer are read;
+#   "attention":        grouped key/value heads, whole-projection rms norms of queries and keys, half-split
+#                       rotary pairs, a learned sink in the softmax's denominator.
+# Feed-forward "moe": clamped experts, the top router logits win, weight sigmoid(logit) on the expert's
+# input; plus a shared expert with a clamp of its own. Logits: the embedding table on the final norm.
+GUGOZEN_MIXERS = ("gla", "latent_attention", "attention")
+
+
+def _gugozen_layer(e: dict, decay_rank: int) -> LayerSpec:
+    m = e["mixer"]
+    H = m["heads"]
+    if e["type"] == "gla":
+        s = LayerSpec(MIX_GLA, heads=H, dim=m["dim"], vdim=m["vdim"], decay_rank=decay_rank, decay_tau=float(m["tau"]),
+                      gate_act=DELTA_GATE_SILU)
+    else:
+        rot = m.get("rot") or {"dims": 0, "base": 1.0}
+        common = dict(heads=H, dim=m["dim"], vdim=m["vdim"], attn_scale=float(m["scale"]), mask_kind=MASK_CAUSAL,
+                      rot_dims=int(rot["dims"]), rot_base=float(rot["base"]), rot_pairs=ROT_HALVES)
+        if e["type"] == "latent_attention":
+            src = m.get("kv_from")
+            s = LayerSpec(MIX_LATENT, kv_rank=m["kv_rank"], q_rank=0, rot_dim=int(m["rot_dim"]),
+                          kv_from=-1 if src is None else int(src), out_gate=GATE_ELEMENT, **common)
+        elif e["type"] == "attention":
+            s = LayerSpec(MIX_ATTN, kv_heads=m.get("kv_heads", H), qk_norm=QK_WHOLE, sink=1, sink_learned=True, **common)
+        else:
+            raise ValueError(f"unknown mixer type {e['type']!r}")
+    mlp = e.get("mlp")
+    if mlp:
+        if mlp["kind"] != "moe":
+            raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+        r, x = mlp["router"], mlp["expert"]
+        s.ff_kind, s.ff, s.limit, s.ff_act = FF_MOE, x["ff"], float(x["limit"]), ACT_CLAMP
+        s.experts, s.top, s.router_kind, s.expert_in_weighted = r["experts"], r["top"], ROUTER_SIGMOID_TOP, True
+        s.shared_gated = False
+        if mlp.get("shared"):
+            s.shared_ff, s.shared_limit = mlp["shared"]["ff"], float(mlp["shared"]["limit"])
+    return s
+
+
+def gugozen_config(cfg: dict, max_tokens: int = 4096, weight_dtype: int = M.BF16, shapes: dict = None) -> LayeredConfig:
+    """config.json of a Gugozen checkpoint -> LayeredConfig. Every size and every constant that can
+    differ between models of the design is read from cfg; the rank of a gla layer's decays, which
+    config.json does not name, is its tensor's own: shapes maps tensor names to shapes."""
+    layers = []
+    for i, e in enumerate(cfg["layers"]):
+        if e["type"] == "gla" and shapes is None:
+            raise ValueError("a Gugozen 'gla' layer takes its decay rank from the checkpoint's tensor shapes")
+        layers.append(_gugozen_layer(e, int(shapes[f"l{i}.mix.a1"][0]) if e["type"] == "gla" else 0))
+    bi = (cfg.get("embedding") or {}).get("bigram")
+    return LayeredConfig(
+        arch="Gugozen", width=cfg["width"], vocab=cfg["vocab"], layers=layers, embed_scale=1.0,
+        norm_eps=float(cfg["norm"]["eps"]), max_tokens=max_tokens, weight_dtype=weight_dtype, norm_kind=NORM_LAYER_BIAS,
+        pre_norm=False, pos_embed=False, tied_head=True, block_kind=BLOCK_POST, stream_scale=float(cfg["postln_alpha"]),
+        bigram_buckets=int(bi["buckets"]) if bi else 0, bigram_mul_prev=int(bi["mul_prev"]) if bi else 0,
+        bigram_mul_cur=int(bi["mul_cur"]) if bi else 0,
+    )
+
+
+def gugozen_tensor_shapes(cfg: dict, decay_rank: int = 8) -> dict:
+    """Checkpoint tensor name -> shape for a Gugozen config.json; the decays' rank is an argument."""
+    W = cfg["width"]
+    out = {"embed": (cfg["vocab"], W)}
+    bi = (cfg.get("embedding") or {}).get("bigram")
+    if bi:
+        out["bigram"] = (bi["buckets"] + 1, W)
+
+    def norm(name):
+        out[name] = out[name + ".b"] = (W,)
+
+    norm("final.norm")
+    for i, e in enumerate(cfg["layers"]):
+        p, m = f"l{i}.", e["mixer"]
+        x = p + "mix."
+        norm(p + "norm1")
+        H, D, V = m["heads"], m["dim"], m["vdim"]
+        if e["type"] == "gla":
+            for n, rows in (("q", H * D), ("k", H * D), ("v", H * V), ("g", H * V), ("a1", decay_rank)):
+                out[x + n] = (rows, W)
+            out[x + "a2"], out[x + "a2.b"], out[x + "norm"] = (H * D, decay_rank), (H * D,), (V,)
+        elif e["type"] == "latent_attention":
+            R, rank = m["rot_dim"], m["kv_rank"]
+            out[x + "q"], out[x + "uk"], out[x + "uv"] = (H * (D + R), W), (H * D, rank), (H * V, rank)
+            out[x + "g"] = (H * V, W)
+            if m.get("kv_from") is None:
+                out[x + "dkv"], out[x + "dkv.norm"] = (rank + R, W), (rank,)
+        else:
+            G = m.get("kv_heads", H)
+            out[x + "q"], out[x + "k"], out[x + "v"] = (H * D, W), (G * D, W), (G * V, W)
+            out[x + "q.norm"], out[x + "k.norm"], out[x + "sink"] = (H * D,), (G * D,), (H,)
+        out[x + "o"] = (W, H * V)
+        mlp = e.get("mlp")
+        if not mlp:
+            continue
+        norm(p + "norm2")
+        f, ff, E = p + "mlp.", mlp["expert"]["ff"], mlp["router"]["experts"]
+        for k in range(E):
+            out[f"{f}e{k}.gate"] = out[f"{f}e{k}.up"] = (ff, W)
+            out[f"{f}e{k}.down"] = (W, ff)
+        out[f + "router"] = (E, W)
+        if mlp.get("shared"):
+            sf = mlp["shared"]["ff"]
+            out[f + "shared.gate"] = out[f + "shared.up"] = (sf, W)
+            out[f + "shared.down"] = (W, sf)
+    return out
+
+
+def gugozen_pack(c: LayeredConfig, t: dict) -> dict:
+    """Checkpoint tensors -> the engine's tensors (see sinulorn_pack). w_in holds q | k | v | gate | decay
+    rows (gla), q (| latent | rotated key part) | gate (latent attention), q | k | v (attention); a norm
+    is weight | bias."""
+    dt = c.weight_dtype
+
+    def w(*names):
+        parts = [_as_weight(t[n], dt) for n in names]
+        return parts[0] if len(parts) == 1 else np.ascontiguousarray(np.concatenate(parts, axis=0))
+
+    def f(name):
+        return np.ascontiguousarray(_as_f32(t[name]))
+
+    def norm(name):
+        return np.concatenate([f(name), f(name + ".b")])
+
+    layers = []
+    for i, l in enumerate(c.layers):
+        p, x, m = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
+        d = {"norm1b": norm(p + "norm1"), "w_o": w(x + "o")}
+        if l.mixer == MIX_GLA:
+            d.update(w_in=w(*[x + n for n in ("q", "k", "v", "g", "a1")]), w_a2=w(x + "a2"), dt_bias=f(x + "a2.b"),
+                     out_norm=f(x + "norm"))
+        elif l.mixer == MIX_LATENT:
+            own = l.kv_from < 0
+            d.update(w_in=w(*[x + n for n in (("q", "dkv", "g") if own else ("q", "g"))]), w_ukv=w(x + "uk", x + "uv"))
+            if own:
+                d["kv_norm"] = f(x + "dkv.norm")
+            uk = _as_weight(t[x + "uk"], dt).reshape(l.heads, l.dim, l.kv_rank)
+            d["w_ukt"] = np.ascontiguousarray(uk.transpose(0, 2, 1))
+        else:
+            d.update(w_in=w(x + "q", x + "k", x + "v"), q_norm=f(x + "q.norm"), kv_norm=f(x + "k.norm"), sink_w=f(x + "sink"))
+        if l.ff_kind != FF_NONE:
+            d.update(norm2b=norm(p + "norm2"), router=f(m + "router"))
+            for k in ("gate", "up", "down"):
+                d["w_" + k] = np.ascontiguousarray(
+                    np.stack([_as_weight(t[f"{m}e{e}.{k}"], dt) for e in range(l.experts)]))
+            if l.shared_ff:
+                d.update(ws_gate=w(m + "shared.gate"), ws_up=w(m + "shared.up"), ws_down=w(m + "shared.down"))
+        _check_packed(f"layer {i}", packed_shapes(c, l), d)
+        layers.append(d)
+    emb = w("embed")
+    out = {"embed": emb, "final_norm": norm("final.norm"), "head": emb, "layers": layers}
+    if c.bigram_buckets:
+        out["bigram"] = w("bigram")
+        if out["bigram"].shape != (c.bigram_buckets + 1, c.width):
+            raise ValueError(f"tensor bigram has shape {out['bigram'].shape}, the configuration gives "
+                             f"{(c.bigram_buckets + 1, c.width)}")
+    return out
+
+
+def gugozen_random_tensors(cfg: dict, seed: int = 0, gain: float = 1.0, decay_rank: int = 8) -> dict:
+    """Random checkpoint tensors for a Gugozen config.json, as float32 arrays already rounded to
+    bf16 values (the f32 and bf16 engines and a float64 restatement see the same weights)."""
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in gugozen_tensor_shapes(cfg, decay_rank).items():
+        leaf = name.split(".")[-1]
+        if leaf in ("norm1", "norm2", "norm"):
+            a = 1.0 + 0.2 * rng.standard_normal(shape)
+        elif name.endswith(".a2.b"):  # decays between fast and nearly none
+            a = rng.uniform(-2.0, 4.0, shape)
+        elif leaf == "b":
+            a = 0.3 * rng.standard_normal(shape)
+        elif leaf == "sink":
+            a = rng.uniform(-1.0, 2.0, shape)
+        elif leaf in ("embed", "bigram"):
+            a = 0.7 * rng.standard_normal(shape)
+        else:
+            a = gain * rng.standard_normal(shape) / np.sqrt(shape[-1])
+        out[name] = bf16_to_f32(f32_to_bf16(np.asarray(a, np.float32))).reshape(shape)
+    return out
+
+
 # ------------------------------------------------------------------ registry
 # design name (config.json "architecture") -> (config reader, weight packer). A reader takes (cfg,
 # max_tokens, weight_dtype, shapes of the checkpoint's tensors), a packer (LayeredConfig, tensors, cfg).
@@ -1242,6 +1447,7 @@ DESIGNS = {
     "Mirorax": (lambda cfg, n, dt, shapes: mirorax_config(cfg, n, dt), mirorax_pack),
     "Lifenex": (lifenex_config, lambda c, t, cfg: lifenex_pack(c, t)),
     "Faguzen": (lambda cfg, n, dt, shapes: faguzen_config(cfg, n, dt), faguzen_pack),
+    "Gugozen": (gugozen_config, lambda c, t, cfg: gugozen_pack(c, t)),
 }
 
 

@@ -159,7 +159,8 @@ class SeqLayer(ctypes.Structure):
         + [(n, c_int) for n in ("ssm_state", "ssm_groups", "norm_groups", "decay_rank", "gate_rank", "gate_act")]
         + [("q_temp_coef", c_float), ("q_temp_every", c_int), ("rel_rows", c_int), ("rel_max", c_float),
            ("join_scale", c_float), ("side_join_scale", c_float), ("rot_pairs", c_int), ("rot_ramp", c_int),
-           ("softcap", c_float), ("gate_cap", c_float), ("identity", c_int)]
+           ("softcap", c_float), ("gate_cap", c_float), ("identity", c_int), ("decay_tau", c_float),
+           ("expert_in_weighted", c_int)]
         + [(n, c_void_p) for n in PTRS]
     )
 
@@ -168,12 +169,13 @@ class SeqConfig(ctypes.Structure):
     _fields_ = [("width", c_int), ("vocab", c_int), ("n_layers", c_int), ("max_tokens", c_int),
                 ("embed_scale", c_float), ("norm_eps", c_float), ("weight_dtype", c_int), ("norm_kind", c_int),
                 ("pre_norm", c_int), ("pos_embed", c_int), ("logit_scale", c_float), ("block_kind", c_int),
-                ("residual_scale", c_float), ("logit_softcap", c_float)]
+                ("residual_scale", c_float), ("logit_softcap", c_float), ("stream_scale", c_float),
+                ("bigram_buckets", c_int), ("bigram_mul_prev", ctypes.c_longlong), ("bigram_mul_cur", ctypes.c_longlong)]
 
 
 class SeqWeights(ctypes.Structure):
     _fields_ = [("embed", c_void_p), ("final_norm", c_void_p), ("head", c_void_p), ("layers", ctypes.POINTER(SeqLayer)),
-                ("embed_norm", c_void_p)]
+                ("embed_norm", c_void_p), ("bigram", c_void_p)]
 
 
 _sig("yalm_seq_create", c_int, [ctypes.POINTER(SeqConfig), ctypes.POINTER(SeqWeights), c_void_p,
@@ -668,8 +670,9 @@ class SeqModel:
         for k in ("embed", "final_norm", "head"):
             # a tied head aliases the embedding table instead of a second upload
             self.ptrs[k] = self.ptrs["embed"] if k == "head" and packed[k] is packed["embed"] else self._up(packed[k])
-        if packed.get("embed_norm") is not None:
-            self.ptrs["embed_norm"] = self._up(packed["embed_norm"])
+        for k in ("embed_norm", "bigram"):
+            if packed.get(k) is not None:
+                self.ptrs[k] = self._up(packed[k])
         seen = {}  # layer runs that share tensors hold the same arrays: one upload each
 
         def up(d):
@@ -733,6 +736,8 @@ class SeqModel:
         self.ptrs["head"] = self.ptrs["embed"] if cfg.tied_head else make("head", (cfg.vocab, cfg.width), "w")
         if cfg.embed_normed:
             self.ptrs["embed_norm"] = make("embed_norm", (cfg.width,), "f")
+        if cfg.bigram_buckets:
+            self.ptrs["bigram"] = make("bigram", (cfg.bigram_buckets + 1, cfg.width), "w", fan_in=100.0)
         for i, l in enumerate(cfg.layers):
             ptrs = {k: make(f"l{i}.{k}", shape, kind) for k, (shape, kind) in layered.packed_shapes(cfg, l).items()}
             if l.side is not None and l.shares < 0:
@@ -770,8 +775,10 @@ class SeqModel:
         arr._sides = sides  # kept alive with the layer array
         sc = SeqConfig(cfg.width, cfg.vocab, len(cfg.layers), cfg.max_tokens, cfg.embed_scale, cfg.norm_eps,
                        cfg.weight_dtype, cfg.norm_kind, int(cfg.pre_norm), int(cfg.pos_embed), cfg.logit_scale,
-                       cfg.block_kind, cfg.residual_scale, cfg.logit_softcap)
-        sw = SeqWeights(self.ptrs["embed"], self.ptrs["final_norm"], self.ptrs["head"], arr, self.ptrs.get("embed_norm"))
+                       cfg.block_kind, cfg.residual_scale, cfg.logit_softcap, cfg.stream_scale, cfg.bigram_buckets,
+                       cfg.bigram_mul_prev, cfg.bigram_mul_cur)
+        sw = SeqWeights(self.ptrs["embed"], self.ptrs["final_norm"], self.ptrs["head"], arr, self.ptrs.get("embed_norm"),
+                        self.ptrs.get("bigram"))
         return sc, sw, arr
 
     def close(self):
