@@ -79,7 +79,7 @@ def parse():
                          "(Sinulorn-shaped stacks, random bf16 weights) at a few real layer sizes, each beside a "
                          "Llama-shaped decoder of equal width, depth and feed-forward size; one JSON line")
     ap.add_argument("--layered-sizes", default="1024,2048,4096", help="model widths of the --layered legs")
-    ap.add_argument("--layered-design", default="sinulorn", choices=["sinulorn", "lenuzen", "mirorax", "lifenex", "faguzen"],
+    ap.add_argument("--layered-design", default="sinulorn", choices=["sinulorn", "lenuzen", "mirorax", "lifenex", "faguzen", "gugozen"],
                     help="which layer-list design the --layered stack is shaped like")
     return ap.parse_args()
 
@@ -636,6 +636,32 @@ def faguzen_stack(Ly, M, width, max_tokens):
                             block_kind=Ly.BLOCK_PARALLEL, residual_scale=0.5, logit_softcap=30.0)
 
 
+def gugozen_stack(Ly, M, width, max_tokens):
+    """A Gugozen-shaped stack at a real layer size, six post-norm layers with routed experts: latent
+    attention, gated linear attention, attention, latent attention over the first layer's rows, gated
+    linear attention, attention. Attention heads of 128 with four query heads per key/value head, half
+    of a head rotated, whole-projection norms and a sink; latent attention with 64 rotated entries and
+    rank 512; linear-attention heads of 128 x 128, half as many as attention heads, rank-16 decays; the
+    clamped experts and shared expert of the Lifenex-shaped stack's hidden sizes, top 4 of 16."""
+    heads = width // 128
+    ff = width * 7 // 2
+    moe = dict(ff_kind=Ly.FF_MOE, ff=ff // 8, experts=16, top=4, limit=7.0, shared_ff=ff // 2, shared_limit=7.0,
+               shared_gated=False, ff_act=Ly.ACT_CLAMP, router_kind=Ly.ROUTER_SIGMOID_TOP, expert_in_weighted=True)
+    lat = dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=0, attn_scale=192 ** -0.5,
+               mask_kind=Ly.MASK_CAUSAL, rot_dims=64, rot_base=10000.0, rot_pairs=Ly.ROT_HALVES, out_gate=Ly.GATE_ELEMENT)
+    att = dict(heads=heads, kv_heads=max(heads // 4, 1), dim=128, vdim=128, attn_scale=128 ** -0.5,
+               mask_kind=Ly.MASK_CAUSAL, qk_norm=Ly.QK_WHOLE, sink=1, sink_learned=True, rot_dims=64, rot_base=500000.0,
+               rot_pairs=Ly.ROT_HALVES)
+    gla = dict(heads=max(heads // 2, 1), dim=128, vdim=128, decay_rank=16, decay_tau=16.0)
+    L = Ly.LayerSpec
+    layers = [L(Ly.MIX_LATENT, **lat, **moe), L(Ly.MIX_GLA, **gla, **moe), L(Ly.MIX_ATTN, **att, **moe),
+              L(Ly.MIX_LATENT, kv_from=0, **lat, **moe), L(Ly.MIX_GLA, **gla, **moe), L(Ly.MIX_ATTN, **att, **moe)]
+    return Ly.LayeredConfig("Gugozen", width, 32000, layers, embed_scale=1.0, norm_eps=1e-5, max_tokens=max_tokens,
+                            weight_dtype=M.BF16, norm_kind=Ly.NORM_LAYER_BIAS, pre_norm=False, pos_embed=False,
+                            tied_head=True, block_kind=Ly.BLOCK_POST, stream_scale=2.0, bigram_buckets=65521,
+                            bigram_mul_prev=31, bigram_mul_cur=17)
+
+
 def layered_bench(args, out_file):
     """--layered: tokens/s of a prompt portion (n = 2048 at position 0) and of single-token
     decoding (the device greedy loop at context ~1024) for the layer-list engine, and for a
@@ -650,7 +676,7 @@ def layered_bench(args, out_file):
     legs = []
     for width in [int(x) for x in args.layered_sizes.split(",")]:
         make = {"lenuzen": lenuzen_stack, "mirorax": mirorax_stack, "lifenex": lifenex_stack,
-                "faguzen": faguzen_stack}.get(args.layered_design, layered_stack)
+                "faguzen": faguzen_stack, "gugozen": gugozen_stack}.get(args.layered_design, layered_stack)
 
         def timed(cfg):
             model = runtime.SeqModel.synthetic(cfg, seed=3)
@@ -673,8 +699,10 @@ def layered_bench(args, out_file):
                "decode_ms_per_token": round(dt / steps * 1e3, 4), "decode_tok_s": round(steps / dt, 2)}
         # the closest layer-list design at the same width, depth and feed-forward size: Sinulorn for Lifenex
         # (delta rule, a linear recurrence, grouped routed experts with a gated shared expert, attention),
-        # Lifenex for Faguzen (attention and a recurrence side by side, routed experts)
-        near = {"lifenex": ("Sinulorn", layered_stack), "faguzen": ("Lifenex", lifenex_stack)}.get(args.layered_design)
+        # Lifenex for Faguzen (attention and a recurrence side by side, routed experts), Mirorax for Gugozen
+        # (latent attention with a rotated key part, attention, clamped feed-forwards, routed experts)
+        near = {"lifenex": ("Sinulorn", layered_stack), "faguzen": ("Lifenex", lifenex_stack),
+                "gugozen": ("Mirorax", mirorax_stack)}.get(args.layered_design)
         if near:
             npf, ndt = timed(near[1](Ly, M, width, n_pf + 64))
             leg.update(near_design=near[0], near_prefill_ms=round(npf, 3), near_prefill_tok_s=round(n_pf / npf * 1e3, 1),

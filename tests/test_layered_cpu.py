@@ -297,7 +297,7 @@ def test_bench_stacks_are_valid_layer_list_configurations():
 
     for width in (1024, 2048, 4096):
         for make in (bench.layered_stack, bench.lenuzen_stack, bench.mirorax_stack, bench.lifenex_stack,
-                     bench.faguzen_stack):
+                     bench.faguzen_stack, bench.gugozen_stack):
             c = make(Ly, M, width, 2112)
             assert c.width == width and len(c.layers) == 6
             for l in c.layers:
@@ -582,3 +582,139 @@ def test_faguzen_restatement_mechanisms():
            "r.e0.down": np.ones((2, 1))}
     h = np.array([[1.0, -4.0]])  # the identity output wins: the input itself
     assert np.allclose(FR.feed_forward(one, "r.", h, {"router": {"experts": 1, "identity": 1, "top": 1}}), h)
+
+
+# ------------------------------------------------------------------ Gugozen
+def _gugozen(cfg, wdt=M.F32, seed=3, **kw):
+    t = Ly.gugozen_random_tensors(cfg, seed=seed, **kw)
+    return Ly.gugozen_config(cfg, max_tokens=77, weight_dtype=wdt, shapes={k: v.shape for k, v in t.items()}), t
+
+
+def test_gugozen_config_reads_every_size_and_constant():
+    import gugozen_cases as GC
+
+    cfg = GC.MIXED
+    c, _ = _gugozen(cfg, decay_rank=5)
+    assert (c.arch, c.width, c.vocab, c.max_tokens, c.weight_dtype) == ("Gugozen", 96, 211, 77, M.F32)
+    assert (c.norm_kind, c.block_kind, c.pre_norm, c.stream_scale, c.norm_eps) == (Ly.NORM_LAYER_BIAS, Ly.BLOCK_POST, False, 1.7, 1e-5)
+    assert (c.bigram_buckets, c.bigram_mul_prev, c.bigram_mul_cur, c.tied_head, c.pos_embed) == (73, 29, 11, True, False)
+    assert [l.mixer for l in c.layers] == [Ly.MIX_LATENT, Ly.MIX_GLA, Ly.MIX_ATTN, Ly.MIX_LATENT, Ly.MIX_GLA, Ly.MIX_LATENT,
+                                           Ly.MIX_ATTN, Ly.MIX_LATENT]
+    assert [l.kv_from for l in c.layers] == [-1, -1, -1, 0, -1, -1, -1, 5]
+    a = c.layers[0]
+    assert (a.heads, a.dim, a.rot_dim, a.vdim, a.kv_rank, a.q_rank, a.attn_scale) == (3, 24, 8, 20, 36, 0, 0.19)
+    assert (a.rot_dims, a.rot_base, a.rot_pairs, a.out_gate, a.sink, a.mask_kind) == (8, 300.0, Ly.ROT_HALVES, Ly.GATE_ELEMENT, 0, Ly.MASK_CAUSAL)
+    assert (a.ff, a.limit, a.shared_ff, a.shared_limit, a.experts, a.top) == (40, 1.5, 24, 0.8, 6, 2)
+    assert (a.router_kind, a.expert_in_weighted, a.shared_gated, a.ff_act) == (Ly.ROUTER_SIGMOID_TOP, True, False, Ly.ACT_CLAMP)
+    assert a.in_rows == 3 * 32 + 36 + 8 + 60 and c.layers[3].in_rows == 5 * 24 + 60
+    g = c.layers[1]
+    assert (g.heads, g.dim, g.vdim, g.decay_rank, g.decay_tau, g.gate_act, g.shared_ff) == (3, 20, 28, 5, 6.0, Ly.DELTA_GATE_SILU, 0)
+    assert g.in_rows == 2 * 60 + 2 * 84 + 5 and c.layers[4].decay_tau == 0.5
+    m = c.layers[6]
+    assert (m.heads, m.kv_heads, m.dim, m.vdim, m.attn_scale, m.qk_norm, m.sink, m.sink_learned) == (3, 1, 32, 24, 0.17, Ly.QK_WHOLE, 1, True)
+    assert c.layers[2].rot_base == 40.0 and c.layers[2].rot_dims == 16 and c.layers[2].ff_kind == Ly.FF_NONE
+    one = {**cfg, "layers": [{**cfg["layers"][0], "mixer": {**cfg["layers"][0]["mixer"], "kv_from": None}}]}
+    del one["embedding"]
+    assert Ly.gugozen_config(one).bigram_buckets == 0 and Ly.gugozen_config(one).layers[0].kv_from == -1
+
+
+def test_gugozen_unknown_names_are_refused():
+    import gugozen_cases as GC
+
+    for bad in ({"type": "parallel", "mixer": GC.attn()[1], "mlp": None},
+                {"type": "attention", "mixer": GC.attn()[1], "mlp": {"kind": "dense", "ff": 8}},
+                {"type": "gla", "mixer": GC.gla()[1], "mlp": None}):  # a gla layer's rank comes from its tensor
+        with pytest.raises(ValueError):
+            Ly.gugozen_config({**GC.ONLY_ATTN, "layers": [bad]})
+
+
+@pytest.mark.parametrize("wdt", [M.F32, M.BF16])
+def test_gugozen_pack_joins_projections_and_norms(wdt):
+    import gugozen_cases as GC
+
+    cfg = GC.MIXED
+    c, t = _gugozen(cfg, wdt)
+    assert set(t) == set(Ly.gugozen_tensor_shapes(cfg))
+    assert "l3.mix.dkv" not in t and "l0.mix.dkv" in t
+    p = Ly.gugozen_pack(c, t)
+    f = (lambda a: a) if wdt == M.F32 else Ly.bf16_to_f32
+    W = cfg["width"]
+    for packed, name in ((p["final_norm"], "final.norm"), (p["layers"][0]["norm1b"], "l0.norm1"),
+                         (p["layers"][0]["norm2b"], "l0.norm2")):
+        assert packed.dtype == np.float32 and packed.shape == (2 * W,)
+        assert np.array_equal(packed[:W], t[name]) and np.array_equal(packed[W:], t[name + ".b"])
+    assert p["head"] is p["embed"] and np.array_equal(f(p["bigram"]), t["bigram"])
+    for i, names in ((0, ("q", "dkv", "g")), (3, ("q", "g")), (1, ("q", "k", "v", "g", "a1")), (2, ("q", "k", "v"))):
+        assert np.array_equal(f(p["layers"][i]["w_in"]), np.concatenate([t[f"l{i}.mix.{n}"] for n in names]))
+    d = p["layers"][3]
+    assert np.array_equal(f(d["w_ukt"][2]), t["l3.mix.uk"][32:48].T) and "kv_norm" not in d
+    assert np.array_equal(f(d["w_ukv"]), np.concatenate([t["l3.mix.uk"], t["l3.mix.uv"]]))
+    assert np.array_equal(p["layers"][1]["dt_bias"], t["l1.mix.a2.b"]) and "ws_up" not in p["layers"][1]
+    assert np.array_equal(p["layers"][2]["sink_w"], t["l2.mix.sink"])
+    assert np.array_equal(f(p["layers"][0]["w_gate"][5]), t["l0.mlp.e5.gate"])
+    for l, d in zip(c.layers, p["layers"]):
+        assert set(Ly.packed_shapes(c, l)) == set(d)
+    with pytest.raises(ValueError):
+        Ly.gugozen_pack(c, {**t, "bigram": t["bigram"][:-1]})
+
+
+def test_gugozen_checkpoint_folder_is_read(tmp_path):
+    """The registry picks the design by config.json's name; the decays' rank is the tensor's."""
+    import json
+
+    import gugozen_cases as GC
+    from yalm_amd.yalmfile import write_yalm
+
+    cfg = GC.ODD
+    t = Ly.gugozen_random_tensors(cfg, seed=4, decay_rank=3)
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    write_yalm(str(tmp_path / "model.safetensors"), {k: Ly.f32_to_bf16(v).reshape(v.shape) for k, v in t.items()}, {},
+               {k: "BF16" for k in t})
+    c, p = Ly.read_checkpoint(str(tmp_path), 50, M.F32)
+    q = Ly.gugozen_pack(c, t)
+    assert c.arch == "Gugozen" and c.max_tokens == 50 and c.layers[2].decay_rank == 3
+    assert np.array_equal(p["bigram"], q["bigram"])
+    for a, b in zip(p["layers"], q["layers"]):
+        assert set(a) == set(b) and all(np.array_equal(a[k], b[k]) for k in b)
+
+
+def test_gugozen_restatement_mechanisms():
+    """The restatement itself: causality; the pair rows; the norm; the rotation's pairing; the linear
+    attention against the sum it stands for; the sink; the router and the side of an expert its weight
+    sits on; shared rows."""
+    import gugozen_cases as GC
+    import gugozen_ref as GR
+
+    cfg = GC.MIXED
+    w = {k: v.astype(np.float64) for k, v in Ly.gugozen_random_tensors(cfg, seed=4).items()}
+    a = GC.tokens(cfg, 40, 1)
+    b = list(a)
+    b[30] = (b[30] + 1) % cfg["vocab"]
+    ra, rb = GR.forward(cfg, w, a), GR.forward(cfg, w, b)
+    assert np.array_equal(ra[:30], rb[:30]) and not np.allclose(ra[30], rb[30]) and not np.allclose(ra[39], rb[39])
+    assert GR.bigram_rows([4, 9, 2], {"buckets": 10, "mul_prev": 3, "mul_cur": 7}) == [10, (12 + 63) % 10, (27 + 14) % 10]
+    n = GR.layer_norm(np.array([[1.0, 3.0]]), {"n": np.array([2.0, 3.0]), "n.b": np.array([0.5, -1.0])}, "n", 0.0)
+    assert np.allclose(n, [[-1.5, 2.0]])
+    x = np.zeros((2, 1, 5))
+    x[1, 0] = [1.0, 0.0, 0.0, 2.0, 7.0]
+    r = GR.rotate_halves(x, {"dims": 4, "base": 16.0})  # angles 1 and 1/4 at position 1
+    assert np.allclose(r[1, 0], [np.cos(1.0), -2 * np.sin(0.25), np.sin(1.0), 2 * np.cos(0.25), 7.0])
+    rng = np.random.default_rng(2)
+    q, k, v = rng.standard_normal((12, 1, 3)), rng.standard_normal((12, 1, 3)), rng.standard_normal((12, 1, 2))
+    g = rng.uniform(0.3, 1.0, (12, 1, 3))
+    o = GR.gla_scan(q, k, v, g)
+    for t in range(12):
+        want = sum((q[t, 0] * g[s_ + 1:t + 1, 0].prod(axis=0) * k[s_, 0]).sum() * v[s_, 0] for s_ in range(t + 1))
+        assert np.allclose(o[t, 0], want)
+    p = GR.causal_softmax(np.log(np.array([[1.0, 9.0], [1.0, 2.0]])), np.log(3.0))
+    assert np.allclose(p, [[0.25, 0.0], [1 / 6, 2 / 6]])
+    idx, wt = GR.route(np.array([0.0, 3.0, -1.0, 40.0, 39.0]), 3)
+    assert idx.tolist() == [3, 4, 1] and np.allclose(wt, [1.0, 1.0, 1 / (1 + np.exp(-3.0))])
+    one = {"r.router": np.array([[0.0, 0.0]]), "r.e0.gate": np.array([[4.0, 0.0]]), "r.e0.up": np.array([[0.0, -6.0]]),
+           "r.e0.down": np.array([[1.0], [2.0]])}
+    h = np.array([[1.0, 1.0]])  # weight 1/2: gate 2 -> 1.5 (limit), up -3 -> -1.5
+    e = 1.5 / (1 + np.exp(-1.702 * 1.5)) * -0.5
+    assert np.allclose(GR.feed_forward(one, "r.", h, {"router": {"experts": 1, "top": 1}, "expert": {"limit": 1.5}}), [[e, 2 * e]])
+    rows = {}
+    GR.layer(cfg, w, 0, GR.embedding(cfg, w, a), rows)
+    assert rows[0][0].shape == (40, 36) and rows[0][1].shape == (40, 8)
