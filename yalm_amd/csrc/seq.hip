@@ -1123,6 +1123,7 @@ static int attn_core_t(Seq *q, int li, int n, const AttnArgs &a, const float *Q,
 		if (ks <= 1) TRY(attn_mfma_launch<1>(q, kc, vc, n, a, Q, gate, ctx));
 		else if (ks <= 2) TRY(attn_mfma_launch<2>(q, kc, vc, n, a, Q, gate, ctx));
 		else if (ks <= 4) TRY(attn_mfma_launch<4>(q, kc, vc, n, a, Q, gate, ctx));
+		else if (ks <= 6) TRY(attn_mfma_launch<6>(q, kc, vc, n, a, Q, gate, ctx));
 		else if (ks <= 8) TRY(attn_mfma_launch<8>(q, kc, vc, n, a, Q, gate, ctx));
 		else TRY(attn_mfma_launch<16>(q, kc, vc, n, a, Q, gate, ctx));
 		return gate_after();
@@ -1440,7 +1441,12 @@ static int ff_dense(Seq *q, int li, int n, float *out) {
 	return gemm(q, plain(q->B[0], l.ff, l.w_down, l.ff, out, c.width, n, c.width, l.ff));
 }
 
-static int ff_moe(Seq *q, int li, int n) {
+// pn: the seam that makes this feed-forward's input, not yet applied (post_routes)
+static bool post_routes(const Seq *q, const yalm_seq_layer &l) {
+	return q->c.block_kind == YALM_BLOCK_POST && l.ff_kind == YALM_FF_MOE && l.router_kind >= YALM_ROUTER_SOFTMAX_NORMED &&
+	       (size_t)q->c.width + 2 * (l.experts + l.identity) <= 12 * 1024;
+}
+static int ff_moe(Seq *q, int li, int n, const PostNorm *pn = nullptr) {
 	const yalm_seq_layer &l = q->L[li];
 	const yalm_seq_config &c = q->c;
 	const int E = l.experts, ER = E + l.identity, top = l.top, ff = l.ff, slots = n * top;
@@ -1449,10 +1455,14 @@ static int ff_moe(Seq *q, int li, int n) {
 	const bool one_wave = l.router_kind == YALM_ROUTER_SOFTMAX_NORMED || l.router_kind == YALM_ROUTER_SIGMOID_TOP;
 	auto router = one_wave ? seq_router_kernel<1024> : seq_router_kernel<SEQ_THREADS>;
 	const int rth = one_wave ? 1024 : SEQ_THREADS;
-	router<<<n, rth, (2 * ER + l.groups) * sizeof(float), q->stream>>>(q->In, c.width, l.router, ER, top, l.groups,
-	                                                                    l.groups_keep, l.router_scale,
-	                                                                    l.shared_ff > 0 ? l.shared_sg : nullptr, q->idx,
-	                                                                    q->wt, q->sgate, l.router_kind, l.router_bias);
+	size_t lds = (2 * ER + l.groups) * sizeof(float);
+	if (pn) { // the post-norm seam before this feed-forward, in the router's launch
+		router = seq_router_kernel<1024, true>;
+		lds += ((c.width + 3) & ~3) * sizeof(float);
+	}
+	router<<<n, rth, lds, q->stream>>>(q->In, c.width, l.router, ER, top, l.groups, l.groups_keep, l.router_scale,
+	                                   l.shared_ff > 0 ? l.shared_sg : nullptr, q->idx, q->wt, q->sgate, l.router_kind,
+	                                   l.router_bias, pn ? *pn : PostNorm{});
 	HIPCHK(hipGetLastError());
 	// experts without gate matrices are plain: one matrix, its activation, the second matrix
 	const bool glu = l.w_gate != nullptr;
@@ -1500,7 +1510,7 @@ static int ff_moe(Seq *q, int li, int n) {
 		return gemm(q, b, slots + (shared ? 1 : 0));
 	} else { // tokens grouped by expert: one batch per expert over its row list
 		seq_fill_int_kernel<<<cdiv(E, 256), 256, 0, q->stream>>>(q->counts, E, 0);
-		seq_moe_lists_kernel<<<cdiv(slots, SEQ_THREADS), SEQ_THREADS, 0, q->stream>>>(q->idx, slots, q->counts, q->lists,
+		seq_moe_lists_kernel<<<cdiv(slots, SEQ_THREADS), SEQ_THREADS, 2 * E * sizeof(int), q->stream>>>(q->idx, slots, q->counts, q->lists,
 		                                                                              q->cap, E);
 		HIPCHK(hipGetLastError());
 		GemmArgs a = plain(q->In, c.width, glu ? l.w_gate : l.w_up, c.width, hx, ff, n, ff, c.width);
@@ -1722,11 +1732,15 @@ static int enqueue_portion(Seq *q, const int *tokens_dev, int n) {
 		if (l.ff_kind == YALM_FF_NONE) {
 			TRY(close(l.norm1b, next, nullptr));
 		} else {
-			TRY(close(l.norm1b, pre ? l.norm2 : nullptr, nullptr));
+			const bool routed = post_routes(q, l); // the seam runs in the router's launch
+			const PostNorm pn{q->X, q->Y, l.norm1b, c.norm_eps, c.stream_scale, c.residual_scale, q->nk};
+			if (!routed)
+				TRY(close(l.norm1b, pre ? l.norm2 : nullptr, nullptr));
 			if (l.ff_kind != YALM_FF_PLAIN)
 				TRY(flush_norm(q, n));
 			TRY(l.ff_kind == YALM_FF_DENSE ? ff_dense(q, li, n, q->Y)
-			                               : (l.ff_kind == YALM_FF_PLAIN ? ff_plain(q, li, n, q->Y) : ff_moe(q, li, n)));
+			                               : (l.ff_kind == YALM_FF_PLAIN ? ff_plain(q, li, n, q->Y)
+			                                                             : ff_moe(q, li, n, routed ? &pn : nullptr)));
 			TRY(close(l.norm2b, next, l.ff_kind == YALM_FF_MOE ? &l : nullptr));
 		}
 		if (q->dump_on && q->dump)

@@ -918,7 +918,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_attn_mfma_kernel(const float 
 	const int TB = 4 / HW, tb = wave / HW, hl = blockIdx.z * HW + wave % HW;
 	const bool active = hl < rep;
 	const int h = g * rep + min(hl, rep - 1);
-	const int t0 = blockIdx.x * 16 * TB, tw0 = t0 + 16 * tb;
+	// the last tokens see the most keys: their workgroups start first
+	const int t0 = (gridDim.x - 1 - blockIdx.x) * 16 * TB, tw0 = t0 + 16 * tb;
 	const int pos0 = st->pos;
 	const int t_last = min(t0 + 16 * TB, n_tok) - 1;
 	const int klo = attn_first_key(a.mask_kind, a.mask_size, pos0 + t0), khi = pos0 + t_last;

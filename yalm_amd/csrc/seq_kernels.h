@@ -1846,8 +1846,9 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_mem_gates_kernel(float *__res
 }
 
 // The recurrence itself. The columns of a head's [dim][vdim] state never mix, so one group
-// of LPC (8 or 16) lanes owns one column (each lane a contiguous slice of R dim entries, in
-// registers; LPC R >= dim) and walks the portion's tokens in order:
+// of LPC (8 or 16) lanes owns one column (each lane R dim entries, in registers, as groups of 4 that
+// alternate with the other lanes': the column's lanes then read a staged row as contiguous 16-byte
+// pieces, on all LDS banks; LPC R >= dim) and walks the portion's tokens in order:
 //   S *= g;  u = beta (v - S.k);  S += k u;  o = S.q
 // (the read-out after the write). The workgroup's 256 / LPC columns share the head's k and q:
 // chunks of TC tokens are staged through two LDS buffers, the next chunk's global loads in
@@ -1891,12 +1892,13 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 	const int c0 = blockIdx.x * COLS, col = c0 + tid / LPC, sub = tid % LPC;
 	const int VS = MEM ? V + 1 : V; // columns of the state
 	const bool live = col < VS;
-	const int d0 = sub * R; // this lane's slice of the key dimension: d0 .. d0 + R - 1
+	static_assert(R % 4 == 0, "a lane holds groups of four entries of the key dimension");
+	auto dim_of = [&](int i) { return (i >> 2) * 4 * LPC + 4 * sub + (i & 3); }; // this lane's i-th entry
 	float S[R];
 	float *sp = state + (size_t)h * D * VS;
 #pragma unroll
 	for (int i = 0; i < R; ++i)
-		S[i] = (live && d0 + i < D) ? sp[(size_t)(d0 + i) * VS + col] : 0.0f;
+		S[i] = (live && dim_of(i) < D) ? sp[(size_t)dim_of(i) * VS + col] : 0.0f;
 	const int qo = qo_ + kh * D, ko = ko_ + kh * D, vo = vo_ + h * V;
 	const float dsk = (SSM && dskip) ? dskip[h] : 0.0f;
 	// a chunk of TC tokens: global -> registers (in flight while the previous chunk is applied) -> LDS
@@ -1995,30 +1997,21 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 			float v, beta, g, em;
 		};
 		auto load = [&](int tt, Tok &x) {
-			if constexpr (R % 4 == 0) {
 #pragma unroll
-				for (int i = 0; i < R / 4; ++i) {
-					const float4_t k4 = *(const float4_t *)&kq[buf][tt][d0 + 4 * i];
-					const float4_t q4 = *(const float4_t *)&kq[buf][tt][DP + d0 + 4 * i];
+			for (int i = 0; i < R / 4; ++i) {
+				const int d = dim_of(4 * i);
+				const float4_t k4 = *(const float4_t *)&kq[buf][tt][d];
+				const float4_t q4 = *(const float4_t *)&kq[buf][tt][DP + d];
 #pragma unroll
-					for (int e = 0; e < 4; ++e) {
-						x.k[4 * i + e] = k4[e];
-						x.q[4 * i + e] = q4[e];
-					}
-					if constexpr (GVEC) {
-						const float4_t g4 = *(const float4_t *)&kq[buf][tt][2 * DP + d0 + 4 * i];
-#pragma unroll
-						for (int e = 0; e < 4; ++e)
-							x.gv[4 * i + e] = g4[e];
-					}
+				for (int e = 0; e < 4; ++e) {
+					x.k[4 * i + e] = k4[e];
+					x.q[4 * i + e] = q4[e];
 				}
-			} else {
+				if constexpr (GVEC) {
+					const float4_t g4 = *(const float4_t *)&kq[buf][tt][2 * DP + d];
 #pragma unroll
-				for (int i = 0; i < R; ++i) {
-					x.k[i] = kq[buf][tt][d0 + i];
-					x.q[i] = kq[buf][tt][DP + d0 + i];
-					if constexpr (GVEC)
-						x.gv[i] = kq[buf][tt][2 * DP + d0 + i];
+					for (int e = 0; e < 4; ++e)
+						x.gv[4 * i + e] = g4[e];
 				}
 			}
 			x.v = vs[buf][tt][tid / LPC];
@@ -2093,8 +2086,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 	if (live) {
 #pragma unroll
 		for (int i = 0; i < R; ++i)
-			if (d0 + i < D)
-				sp[(size_t)(d0 + i) * VS + col] = S[i];
+			if (dim_of(i) < D)
+				sp[(size_t)dim_of(i) * VS + col] = S[i];
 	}
 	if (MEM && tid == 0)
 		mst[(size_t)h * gridDim.x + blockIdx.x] = mrun;
@@ -2526,18 +2519,74 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_latent_attn_mfma_kernel(const
 // about 17); weight = sigmoid(logit) * rscale.
 // NT threads (kind 0: SEQ_THREADS).
 // Also the shared expert's gate sigmoid(w_sg . h). Dynamic LDS: 2 E + G floats.
+// POST: the row it routes is the post-norm seam's result, made here: h = norm(alpha X[t] + rs Y[t]) (see
+// seq_post_close_reg_kernel), kept in LDS for the logits and written to X[t]; Hn is not read. Dynamic
+// LDS: width (rounded up to 4) floats more, at its start.
 #define SEQ_MAX_GROUPS 64
+struct PostNorm {
+	float *X = nullptr;
+	const float *Y = nullptr, *wb = nullptr;
+	float eps = 0.0f, alpha = 1.0f, rs = 1.0f;
+	int nk = NK_RMS;
+};
 template <int NT>
+__device__ __forceinline__ float block_sum_of(float v, float *red) { // block_sum over NT threads
+	v = wave_sum(v);
+	__syncthreads();
+	if ((threadIdx.x & 63) == 0)
+		red[threadIdx.x >> 6] = v;
+	__syncthreads();
+	float t = 0.0f;
+#pragma unroll
+	for (int i = 0; i < NT / 64; ++i)
+		t += red[i];
+	return t;
+}
+template <int NT, bool POST = false>
 __global__ __launch_bounds__(NT) void seq_router_kernel(const float *__restrict__ Hn, int width,
                                                                  const float *__restrict__ Wr, int E, int top, int G,
                                                                  int keep, float rscale,
                                                                  const float *__restrict__ w_sg, int *__restrict__ idx,
                                                                  float *__restrict__ wt, float *__restrict__ sgate,
-                                                                 int kind = 0, const float *__restrict__ bias = nullptr) {
-	extern __shared__ float sc[];
+                                                                 int kind = 0, const float *__restrict__ bias = nullptr,
+                                                                 PostNorm pn = PostNorm{}) {
+	extern __shared__ __attribute__((aligned(16))) float router_lds[];
+	float *sc = router_lds + (POST ? (width + 3) & ~3 : 0);
 	const int t = blockIdx.x;
 	const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
 	const float *h = Hn + (size_t)t * width;
+	if constexpr (POST) {
+		__shared__ float pred[NT / 64];
+		float *row = router_lds, *x = pn.X + (size_t)t * width;
+		const float *y = pn.Y + (size_t)t * width;
+		const int n = width;
+		float sm = 0.0f, ss = 0.0f;
+		for (int i = threadIdx.x; i < n; i += NT) { // each thread re-reads the entries it wrote
+			const float v = fmaf(pn.alpha, x[i], pn.rs * y[i]);
+			row[i] = v;
+			sm += v;
+			ss = fmaf(v, v, ss);
+		}
+		float mu = 0.0f, r = 1.0f;
+		if (nk_centred(pn.nk)) {
+			mu = block_sum_of<NT>(sm, pred) / (float)n;
+			ss = 0.0f;
+			for (int i = threadIdx.x; i < n; i += NT) {
+				const float d = row[i] - mu;
+				ss = fmaf(d, d, ss);
+			}
+		}
+		if (pn.nk != NK_TANH)
+			r = 1.0f / sqrtf(block_sum_of<NT>(ss, pred) / (float)n + pn.eps);
+		for (int i = threadIdx.x; i < n; i += NT) {
+			const float v = pn.nk == NK_TANH ? tanh_norm(pn.wb, n, i, row[i])
+			                                 : fmaf((row[i] - mu) * r, pn.wb[i], norm_bias(pn.nk, pn.wb, n, i));
+			row[i] = v;
+			x[i] = v;
+		}
+		__syncthreads();
+		h = row;
+	}
 	for (int e = wave; e < E + (w_sg ? 1 : 0); e += NT / 64) {
 		const float *w = e < E ? Wr + (size_t)e * width : w_sg;
 		float a = 0.0f;
@@ -2751,18 +2800,25 @@ __global__ __launch_bounds__(NT) void seq_router_kernel(const float *__restrict_
 
 // Slot s = t * top + k goes onto its expert's list (any order: every slot's rows are
 // computed independently of their neighbours in the list); choices past the n_exp experts
-// (identity outputs) go nowhere.
+// (identity outputs) go nowhere. A workgroup counts its slots per expert in LDS and takes one range
+// of every list it adds to. Dynamic LDS: 2 n_exp ints.
 __global__ __launch_bounds__(SEQ_THREADS) void seq_moe_lists_kernel(const int *__restrict__ idx, int n_slots,
                                                                     int *__restrict__ counts, int *__restrict__ lists,
                                                                     int cap, int n_exp) {
+	extern __shared__ int lds_counts[];
+	int *mine = lds_counts, *base = lds_counts + n_exp;
+	for (int e = threadIdx.x; e < n_exp; e += SEQ_THREADS)
+		mine[e] = 0;
+	__syncthreads();
 	const int s = blockIdx.x * SEQ_THREADS + threadIdx.x;
-	if (s >= n_slots)
-		return;
-	const int e = idx[s];
-	if (e >= n_exp)
-		return;
-	const int p = atomicAdd(&counts[e], 1);
-	lists[(size_t)e * cap + p] = s;
+	const int e = s < n_slots ? idx[s] : n_exp;
+	const int at = e < n_exp ? atomicAdd(&mine[e], 1) : 0;
+	__syncthreads();
+	for (int x = threadIdx.x; x < n_exp; x += SEQ_THREADS)
+		base[x] = mine[x] > 0 ? atomicAdd(&counts[x], mine[x]) : 0;
+	__syncthreads();
+	if (e < n_exp)
+		lists[(size_t)e * cap + base[e] + at] = s;
 }
 __global__ void seq_fill_int_kernel(int *p, int n, int v) {
 	const int i = blockIdx.x * blockDim.x + threadIdx.x;
