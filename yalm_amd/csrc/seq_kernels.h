@@ -1881,9 +1881,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 	constexpr int DP = LPC * R;                    // padded key dimension
 	constexpr bool GLA = SSM && GVEC;
 	constexpr int NS = GVEC ? 3 : 2;               // staged rows per token: k | q (| g)
-	constexpr int NKQ = TC * NS * DP / SEQ_THREADS; // staged values per thread and chunk
+	constexpr int PD = DP / 4;                     // pieces of 4 entries per staged row
+	constexpr int NP = (TC * PD + SEQ_THREADS - 1) / SEQ_THREADS; // pieces per thread, staged part and chunk
 	constexpr int COLS = SEQ_THREADS / LPC, NV = (TC * COLS + SEQ_THREADS - 1) / SEQ_THREADS;
-	static_assert((LPC == 8 || LPC == 16) && (TC * NS * DP) % SEQ_THREADS == 0, "staging assumes whole passes of the workgroup");
+	static_assert((LPC == 8 || LPC == 16) && SEQ_THREADS % PD == 0, "a thread stages the same entries of every token");
 	__shared__ __attribute__((aligned(16))) float kq[2][TC][NS * DP];
 	static_assert(!MEM || (SSM && !GVEC && TC <= 16), "the matrix memory walks as the state-space form, at most 16 tokens a chunk");
 	__shared__ float vs[2][TC][COLS], bgs[2][TC][MEM ? 3 : 2];
@@ -1892,7 +1893,7 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 	const int c0 = blockIdx.x * COLS, col = c0 + tid / LPC, sub = tid % LPC;
 	const int VS = MEM ? V + 1 : V; // columns of the state
 	const bool live = col < VS;
-	static_assert(R % 4 == 0, "a lane holds groups of four entries of the key dimension");
+	static_assert(R % 4 == 0 && TC % 2 == 0, "a lane holds groups of four entries of the key dimension");
 	auto dim_of = [&](int i) { return (i >> 2) * 4 * LPC + 4 * sub + (i & 3); }; // this lane's i-th entry
 	float S[R];
 	float *sp = state + (size_t)h * D * VS;
@@ -1902,30 +1903,39 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 	const int qo = qo_ + kh * D, ko = ko_ + kh * D, vo = vo_ + h * V;
 	const float dsk = (SSM && dskip) ? dskip[h] : 0.0f;
 	// a chunk of TC tokens: global -> registers (in flight while the previous chunk is applied) -> LDS
-	float rkq[NKQ], rv[NV], rbg = 0.0f, rlf = 0.0f;
+	float4_t rkq[NS][NP];
+	float rv[NV], rbg = 0.0f, rlf = 0.0f;
 	float mrun = MEM ? mst[(size_t)h * gridDim.x + blockIdx.x] : 0.0f; // kept by the first wave
+	// this thread's entries sd .. sd + 3 of k, q (and g) of tokens st0, st0 + SEQ_THREADS / PD, ...
+	const int st0 = tid / PD, sd = 4 * (tid % PD);
+	const int sdc = sd < D ? sd : 0;
+	const float *src[3] = {QKV + ko + sdc, QKV + qo + sdc, GVEC ? GV + (size_t)h * D + sdc : nullptr};
+	const size_t sld[3] = {(size_t)ldq, (size_t)ldq, (size_t)H * D};
+	const bool vec = D % 4 == 0 && ldq % 4 == 0 && ko % 4 == 0 && qo % 4 == 0 && ((size_t)QKV | (size_t)(GVEC ? GV : QKV)) % 16 == 0;
+	const bool in_row = sd < D;
+	// Tokens past the portion's end repeat its last one (never applied); entries past D become zeros only
+	// as they are stored to LDS, so that every load of a chunk is in flight at once.
 	auto fetch = [&](int t0) {
+		if (vec) {
 #pragma unroll
-		for (int i = 0; i < NKQ; ++i) {
-			const int idx = tid + i * SEQ_THREADS;
-			const int tt = idx / (NS * DP), e = idx % (NS * DP), d = e % DP, part = e / DP;
-			const int t = t0 + tt;
-			float x = 0.0f;
-			if (t < T && d < D) {
-				if (GVEC && part == 2)
-					x = GV[((size_t)t * H + h) * D + d];
-				else
-					x = QKV[(size_t)t * ldq + (part == 0 ? ko : qo) + d];
-			}
-			rkq[i] = x;
+			for (int p = 0; p < NS; ++p)
+#pragma unroll
+				for (int i = 0; i < NP; ++i)
+					rkq[p][i] = *(const float4_t *)(src[p] + min(t0 + st0 + i * (SEQ_THREADS / PD), T - 1) * sld[p]);
+		} else {
+#pragma unroll
+			for (int p = 0; p < NS; ++p)
+#pragma unroll
+				for (int i = 0; i < NP; ++i)
+#pragma unroll
+					for (int e = 0; e < 4; ++e)
+						rkq[p][i][e] = sd + e < D ? src[p][min(t0 + st0 + i * (SEQ_THREADS / PD), T - 1) * sld[p] + e] : 0.0f;
 		}
 #pragma unroll
 		for (int i = 0; i < NV; ++i) {
 			const int idx = tid + i * SEQ_THREADS;
 			const int tt = idx / COLS, cc = idx % COLS, t = t0 + tt;
-			rv[i] = (tt < TC && t < T && c0 + cc < V) ? QKV[(size_t)t * ldq + vo + c0 + cc] : 0.0f;
-			if (MEM && c0 + cc == V)
-				rv[i] = 1.0f;
+			rv[i] = QKV[(size_t)min(tt < TC ? t : 0, T - 1) * ldq + vo + min(c0 + cc, V - 1)];
 		}
 		if constexpr (MEM) {
 			if (tid < TC) { // identities of the scan past the portion's end
@@ -1944,15 +1954,17 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 	};
 	auto stash = [&](int buf) {
 #pragma unroll
-		for (int i = 0; i < NKQ; ++i) {
-			const int idx = tid + i * SEQ_THREADS;
-			kq[buf][idx / (NS * DP)][idx % (NS * DP)] = rkq[i];
-		}
+		for (int p = 0; p < NS; ++p)
+#pragma unroll
+			for (int i = 0; i < NP; ++i)
+				if (TC * PD >= SEQ_THREADS || st0 < TC)
+					*(float4_t *)&kq[buf][st0 + i * (SEQ_THREADS / PD)][p * DP + sd] =
+					    in_row ? rkq[p][i] : float4_t{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
 		for (int i = 0; i < NV; ++i) {
 			const int idx = tid + i * SEQ_THREADS;
-			if (idx < TC * COLS)
-				vs[buf][idx / COLS][idx % COLS] = rv[i];
+			if (idx < TC * COLS) // columns past V are never read (the normaliser's v is 1)
+				vs[buf][idx / COLS][idx % COLS] = (MEM && c0 + idx % COLS == V) ? 1.0f : rv[i];
 		}
 		if constexpr (MEM) {
 			if (tid < 64) {
@@ -1990,6 +2002,8 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 		if (more)
 			fetch(t0 + TC);
 		const int nt = min(TC, T - t0);
+		constexpr int NK = (TC + LPC - 1) / LPC;
+		float keep[NK] = {};
 		// One token's operands out of LDS, one token ahead of the arithmetic (two register sets in
 		// turn), so that the LDS round trip runs under the previous token's dependent chain.
 		struct Tok {
@@ -2063,20 +2077,37 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_delta_kernel(const float *__r
 			} else if constexpr (SSM) {
 				o = fmaf(dsk, x.v, o);
 			}
-			if (sub == 0 && live)
-				O[(size_t)(t0 + tt) * H * VS + h * VS + col] = o;
+#pragma unroll
+			for (int x2 = 0; x2 < NK; ++x2) // lane `sub` keeps the read-outs of tokens sub, sub + LPC, ...
+				keep[x2] = sub + x2 * LPC == tt ? o : keep[x2];
 		};
 		Tok xa, xb;
 		load(0, xa);
-		for (int tt = 0; tt < nt; tt += 2) {
-			if (tt + 1 < nt)
+		if (nt == TC) { // whole chunks without branches: the waits then cover one token's reads, not all in flight
+#pragma unroll
+			for (int tt = 0; tt < TC; tt += 2) {
 				load(tt + 1, xb);
-			apply(tt, xa);
-			if (tt + 1 < nt) {
-				if (tt + 2 < nt)
+				apply(tt, xa);
+				if (tt + 2 < TC)
 					load(tt + 2, xa);
 				apply(tt + 1, xb);
 			}
+		} else
+			for (int tt = 0; tt < nt; tt += 2) {
+				if (tt + 1 < nt)
+					load(tt + 1, xb);
+				apply(tt, xa);
+				if (tt + 1 < nt) {
+					if (tt + 2 < nt)
+						load(tt + 2, xa);
+					apply(tt + 1, xb);
+				}
+			}
+#pragma unroll
+		for (int x = 0; x < NK; ++x) { // every lane of a column holds its sums: one store per chunk
+			const int tt = sub + x * LPC;
+			if (live && tt < nt)
+				O[((size_t)(t0 + tt) * H + h) * VS + col] = keep[x];
 		}
 		if (more)
 			stash(buf ^ 1); // last read while the chunk before this one was applied
