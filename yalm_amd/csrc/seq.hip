@@ -711,7 +711,7 @@ static int gemm_t(Seq *q, const GemmArgs &a, int batches, int max_m) {
 			seq_gemv_kernel<WT, true><<<g, SEQ_THREADS, 0, q->stream>>>(a);
 		else
 			seq_gemv_kernel<WT, false><<<g, SEQ_THREADS, 0, q->stream>>>(a);
-	} else if (WT::BYTES == 2 && max_m > GT_BM) {
+	} else if (WT::BYTES == 2 && max_m > GT_BM && (batches > 1 || a.K > GT_BN)) { // (short sums: the epilogue's work, over more workgroups)
 		const dim3 g(cdiv(a.N, GB_BN), cdiv(max_m, GB_BM), batches);
 		if (glu)
 			seq_gemm_bf16_kernel<true><<<g, SEQ_THREADS, 0, q->stream>>>(a);

@@ -1309,7 +1309,10 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_kernel(GemmArgs a) {
 
 	if constexpr (WT::BYTES == 2) {
 		constexpr int LD = GT_BK + 8; // bf16 elements per LDS row: 80 bytes, 16-byte aligned pieces
-		__shared__ __attribute__((aligned(16))) uint16_t As[GT_BM * LD], Bs[GT_BN * LD], Bs2[GLU ? GT_BN * LD : 8];
+		constexpr int LDE = 33, OPS = (GLU ? 3 : 2) * GT_BM * LD, SUMS = 4 * 32 * LDE * (GLU ? 2 : 1) * 2;
+		static_assert(GT_BM == GT_BN, "square tiles");
+		__shared__ __attribute__((aligned(16))) uint16_t smem[OPS > SUMS ? OPS : SUMS]; // operand slabs, then the sums
+		uint16_t *As = smem, *Bs = smem + GT_BM * LD, *Bs2 = smem + (GLU ? 2 : 0) * GT_BM * LD;
 		const int wave = tid >> 6, lane = tid & 63;
 		const int wm = (wave & 1) * 32, wn = (wave >> 1) * 32;
 		float16_t acc = {}, acc2 = {};
@@ -1379,15 +1382,25 @@ __global__ __launch_bounds__(SEQ_THREADS) void seq_gemm_kernel(GemmArgs a) {
 				}
 			}
 		}
-		const int n = n0 + wn + (lane & 31);
-		if (n < a.N) {
+		// the epilogue's code once, over sums passed through LDS, instead of once per accumulator register
+		// (its instructions would otherwise be fetched sixteen times over by a workgroup of short sums)
+		__syncthreads();
+		float *const E1 = (float *)smem + wave * 32 * LDE * (GLU ? 2 : 1), *const E2 = E1 + (GLU ? 32 * LDE : 0);
 #pragma unroll
-			for (int r = 0; r < 16; ++r) {
-				const int ml = wm + (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
-				const int rc = crow[ml];
-				if (rc >= 0)
-					b.C[(size_t)rc * a.ldc + n] = epi_out(a, b, rc, n, acc[r], GLU ? acc2[r] : 0.0f);
-			}
+		for (int r = 0; r < 16; ++r) {
+			const int ml = (r & 3) + 8 * (r >> 2) + 4 * (lane >> 5);
+			E1[ml * LDE + (lane & 31)] = acc[r];
+			if constexpr (GLU)
+				E2[ml * LDE + (lane & 31)] = acc2[r];
+		}
+		__syncthreads();
+		const int n = n0 + wn + (lane & 31);
+#pragma unroll 1
+		for (int it = 0; it < 16; ++it) {
+			const int ml = 2 * it + (lane >> 5), rc = crow[wm + ml];
+			if (rc >= 0 && n < a.N)
+				b.C[(size_t)rc * a.ldc + n] =
+				    epi_out(a, b, rc, n, E1[ml * LDE + (lane & 31)], GLU ? E2[ml * LDE + (lane & 31)] : 0.0f);
 		}
 	} else {
 		constexpr int LDF = GT_BM + 4;
